@@ -286,12 +286,12 @@ pf1)        # round 6: the tolerance prompt pass as ONE chunk on one stream (no 
         python /root/repo/tools/probes/prefill_profile.py 8192 2 48 8192 1
     ;;
 ringp)      # round 6: the stand-alone probe of the ring GEMM (dense problem): bit comparison, timing of both forms, stamps
-    hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off -fno-fast-math -Wno-unused-function -o /tmp/grp tools/probes/gemm_ring_probe.hip 2>&1 | grep -E "error" -A3
+    hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off -fno-fast-math -Xclang -target-feature -Xclang -packed-fp32-ops -Wno-unused-function -o /tmp/grp tools/probes/gemm_ring_probe.hip 2>&1 | grep -E "error" -A3
     /tmp/grp 4096 2048 12288 | grep -v "^  mismatch"; /tmp/grp 8192 2048 4096 | grep -v "^  mismatch"; /tmp/grp 2752 2048 12288 | grep -v "^  mismatch"
     ;;
 ringabl)    # round 6: ablations of the ring GEMM's loop (results wrong by construction): what bounds a unit
     for abl in 0 1 2 4 8 3 7 15; do
-        hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off -fno-fast-math -Wno-unused-function -DPFR_ABL=$abl -o /tmp/grp$abl tools/probes/gemm_ring_probe.hip 2>&1 | grep -E "error" -A3
+        hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off -fno-fast-math -Xclang -target-feature -Xclang -packed-fp32-ops -Wno-unused-function -DPFR_ABL=$abl -o /tmp/grp$abl tools/probes/gemm_ring_probe.hip 2>&1 | grep -E "error" -A3
         echo "== PFR_ABL=$abl (1 no de-quantization, 2 no requests in the loop, 4 no fragment reads in the loop, 8 no barriers in the loop)"
         /tmp/grp$abl 4096 2048 12288 | grep "ring   rep [23]\|ring stamps"
     done
