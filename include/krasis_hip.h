@@ -409,17 +409,19 @@ typedef struct {
     float scale;
     int window;                        /* position i sees j with 0 <= i - j < window; 0 = all earlier positions */
     int has_sink;                      /* KR_SERVE_SINK_*: softmax denominator + exp(sink[head]), or + 1 */
-    int kv_from;                       /* -1, or the earlier layer whose cached keys / values this layer attends to (no k / v projections of its own) */
+    int kv_from;                       /* -1, or the earlier layer whose cached keys / values (latents) this layer attends to (no k / v projections of its own) */
     int mlp_kind;
     int ff, dense_act;                 /* dense: down(act(gate h, up h)) */
     int experts, top, groups, keep, renorm;   /* router: scores over all experts; best `keep` of `groups` groups; `top` experts; weights = scores (renorm: / (their sum + 1e-20)) */
     int expert_ff, expert_act; float expert_limit, expert_alpha;
     int shared_ff; float shared_limit;        /* 0 = no shared expert */
     /* ---- mechanisms a design may switch on beside the ones above (all zero = off) */
-    int mixer_kind;                    /* KR_SERVE_MIX_ATTENTION | KR_SERVE_MIX_LATENT */
-    /* latent mixer: queries c_q = rms(W_dq h) * w -> q = W_uq c_q, per head [dim plain | rot_dims rotated]; W_dkv h = [kv_rank | rot_dims]: the first part,
-     * rms-normed with a weight, is the latent c, the second, rotated, one key part shared by all heads; per head k = [W_uk c | shared part], v = W_uv c.
-     * The cache holds c and the shared part only: a step folds W_uk into the queries and applies W_uv to the weighted sum of latents.  kv_heads is 1. */
+    int mixer_kind;                    /* KR_SERVE_MIX_* */
+    /* latent mixer: queries c_q = rms(W_dq h) * w -> q = W_uq c_q, or q = W_q h when q_rank is 0, per head [dim plain | rot_dims rotated];
+     * W_dkv h = [kv_rank | rot_dims]: the first part, rms-normed with a weight, is the latent c, the second, rotated, one key part shared by all heads; per
+     * head k = [W_uk c | shared part], v = W_uv c.  The cache holds c and the shared part only: a step folds W_uk into the queries and applies W_uv to the
+     * weighted sum of latents.  kv_heads is 1.  With kv_from the layer has no W_dkv and reads the other layer's rows (same kv_rank, rot_dims and rotation;
+     * heads, dim and vdim may differ); out_gate ELEM_SIGMOID gates the values W_uv forms. */
     int q_rank, kv_rank;
     int rot_scaling;                   /* KR_SERVE_ROT_LINEAR (f / rot_factor) | KR_SERVE_ROT_BY_PARTS: pair i keeps f_i, is divided by rot_factor, or a blend: */
     double rot_original, rot_fast, rot_slow;   /* pair(t) = rot_dims ln(rot_original / (2 pi t)) / (2 ln base); ramp from floor(pair(fast)) to ceil(pair(slow)); cos, sin * (0.1 ln factor + 1) */
@@ -459,6 +461,12 @@ typedef struct {
     int side_mixer;
     int ssd_heads, ssd_vdim, ssd_state, ssd_groups, ssd_conv, ssd_norm_groups;
     float mix_scale, side_scale;
+    /* ---- router, further */
+    int expert_in_weight;              /* 1: an expert's weight multiplies its INPUT: ff = sum_e expert_e(w_e h), added as they are */
+    /* ---- KR_SERVE_MIX_RGLRU: two branches of rg_width channels, y = gelu_tanh(W_y h + b_y) and u = conv(W_x h + b_x) + conv_b (rg_conv taps, the last column is
+     * the current token's); in each of rg_blocks equal parts of u: r = sigmoid(A u + a), i = sigmoid(B u + b); log d = -rg_rate r softplus(lam),
+     * S_t = d S_(t-1) + sqrt(1 - d^2) i u, per channel, f32; mixer output W_o (S * y).  S and the last rg_conv - 1 rows W_x h + b_x are a request's state. */
+    int rg_width, rg_blocks, rg_conv; float rg_rate;
 } kr_serve_layer;
 #define KR_SERVE_BLOCK_PARALLEL 0
 #define KR_SERVE_BLOCK_SEQUENTIAL 1
@@ -467,6 +475,7 @@ typedef struct {
 #define KR_SERVE_MIX_RETENTION 2       /* S_t = decay_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; k scaled by dim^(-1/2) after the rotation; o / rms(o) per head, times silu(W_g h) */
 #define KR_SERVE_MIX_GLA 4             /* a decay per key channel, formed from the input through a low-rank projection (fields decay_*) */
 #define KR_SERVE_MIX_SSD 5             /* selective state space with one decay per head and token (fields ssd_*) */
+#define KR_SERVE_MIX_RGLRU 6           /* real-gated linear recurrence over channels between a convolution and a gated branch (fields rg_*) */
 #define KR_SERVE_MIX_MLSTM 3           /* exponential input gate and sigmoid forget gate in log space with a running maximum m (m_0 = 0), normaliser state n;
                                         * q scaled by dim^(-1/2); o = S^T q / (max(|n.q|, exp(-m)) + 1e-6); o / rms(o) per head, times a weight, times sigmoid(W_g h) */
 #define KR_SERVE_QKNORM_NONE 0
@@ -509,9 +518,11 @@ enum { KR_SV_EMBED = 0, KR_SV_FINAL_NORM_W, KR_SV_FINAL_NORM_B, KR_SV_HEAD, KR_S
        KR_SV_EMBED_NORM, KR_SV_BIGRAM /* layer = -1 */, KR_SV_PRE_ADD, KR_SV_V_BIAS, KR_SV_Q_CONV, KR_SV_K_CONV, KR_SV_V_CONV,
        KR_SV_DECAY_A1, KR_SV_DECAY_A2, KR_SV_DECAY_A2_B,
        KR_SV_SSD_IN, KR_SV_SSD_CONV, KR_SV_SSD_CONV_B, KR_SV_SSD_DT_BIAS, KR_SV_SSD_A_LOG, KR_SV_SSD_D, KR_SV_SSD_NORM, KR_SV_SSD_O,
+       KR_SV_RG_Y, KR_SV_RG_Y_B, KR_SV_RG_X, KR_SV_RG_X_B, KR_SV_RG_CONV, KR_SV_RG_CONV_B,
+       KR_SV_RG_RA /* [rg_blocks * size, size] */, KR_SV_RG_RA_B /* [rg_blocks, size] */, KR_SV_RG_RI, KR_SV_RG_RI_B, KR_SV_RG_LAM,
        KR_SV_N_ROLES };
 /* layout version of kr_serve_config / kr_serve_layer: a caller built against another one must not use the library */
-#define KR_SERVE_ABI 4
+#define KR_SERVE_ABI 5
 int kr_serve_abi(void);
 int kr_serve_create(int device_ordinal, const kr_serve_config* cfg, const kr_serve_layer* layers, kr_serve** out);
 void kr_serve_destroy(kr_serve* s);

@@ -66,10 +66,11 @@ class ServeLayerC(C.Structure):
                 ("router_score", C.c_int), ("group_score", C.c_int),
                 ("weights_of", C.c_int), ("pre_add", C.c_int), ("proj_conv", C.c_int), ("decay_rank", C.c_int), ("decay_tau", C.c_float), ("side_mixer", C.c_int),
                 ("ssd_heads", C.c_int), ("ssd_vdim", C.c_int), ("ssd_state", C.c_int), ("ssd_groups", C.c_int), ("ssd_conv", C.c_int), ("ssd_norm_groups", C.c_int),
-                ("mix_scale", C.c_float), ("side_scale", C.c_float)]
+                ("mix_scale", C.c_float), ("side_scale", C.c_float),
+                ("expert_in_weight", C.c_int), ("rg_width", C.c_int), ("rg_blocks", C.c_int), ("rg_conv", C.c_int), ("rg_rate", C.c_float)]
 
 
-SERVE_ABI = 4      # layout version of the two structures above (KR_SERVE_ABI in include/krasis_hip.h)
+SERVE_ABI = 5      # layout version of the two structures above (KR_SERVE_ABI in include/krasis_hip.h)
 
 
 _lib = None

@@ -21,7 +21,7 @@ struct SvLayer {
     kr_serve_layer d{};
     // hw: every matrix that multiplies the normed input, row blocks [q | k | v | router | gate | up] (router: E rows, or hi + lo = 2E rows in a bf16
     // store; gate | up: the dense feed-forward's or the shared expert's) -- one GEMM per layer produces them all
-    // A latent mixer's first row blocks are [dq | dkv] instead of [q | k | v]; its up-projections are matrices of their own: uq, and per head ukT
+    // A latent mixer's first row blocks are [dq | dkv] (or [q | dkv]; a borrowed cache leaves dkv out) instead of [q | k | v]; its up-projections are matrices of their own: uq, and per head ukT
     // [kv_rank, dim] (W_uk of the head transposed: it multiplies the QUERY) and uv [vdim, kv_rank].
     DevBuf norm_w, norm_b, norm2_w, norm2_b, post1_w, post1_b, post2_w, post2_b, hw, o, sink, down, egu, edown, sdown, kpool, vpool;
     DevBuf q_norm, k_norm, vmix, router_b, slopes, dq_norm, dkv_norm, uq, ukT, uv;
@@ -35,23 +35,30 @@ struct SvLayer {
     // state-space mixer: convolution taps and bias, dt bias, log rates, skip weights, norm weight; per slot the convolution's ring and S [heads][vdim][state]
     DevBuf sconv_w, sconv_b, dt_bias, a_log, ssd_d, ssd_norm, sconv_state, ssd_state;
     size_t ssd_state_stride = 0;
+    // real-gated linear recurrence: branch biases, convolution taps and bias, both gates' block matrices and biases, -rate softplus(lam); per slot S and the convolution's ring
+    DevBuf rg_yb, rg_xb, rg_conv, rg_convb, rg_w, rg_b, rg_rate, rg_state, rg_ring;
     int wsrc = 0;                // the layer whose tensors this one uses (itself, or d.weights_of - 1); cache pools and state are always the layer's own
-    // row blocks of hw: mixer [q | k | v | out gate | i | f | state-space in-projection] (n_qkv rows in all), then [router | gate | up | residual gate of the feed-forward]
+    // row blocks of hw: mixer [q | k | v | out gate | i | f | state-space in-projection], or the recurrence's branches [y | x] (n_qkv rows in all), then [router | gate | up | residual gate of the feed-forward]
     int rope_id = 0, n_qkv = 0, off_ogate = 0, off_if = 0, off_ssd = 0, off_router = 0, n_router = 0, off_gu = 0, n_gu = 0, off_rg2 = 0, n_h = 0;
     bool latent() const { return d.mixer_kind == KR_SERVE_MIX_LATENT; }
     bool gla() const { return d.mixer_kind == KR_SERVE_MIX_GLA; }
     bool recurrent() const { return d.mixer_kind == KR_SERVE_MIX_RETENTION || d.mixer_kind == KR_SERVE_MIX_MLSTM || gla(); }
     bool chunkable() const { return d.mixer_kind == KR_SERVE_MIX_RETENTION || d.mixer_kind == KR_SERVE_MIX_MLSTM; }      // the block form of the recurrence
     bool ssd_alone() const { return d.mixer_kind == KR_SERVE_MIX_SSD; }
+    bool rglru() const { return d.mixer_kind == KR_SERVE_MIX_RGLRU; }
+    bool no_heads() const { return ssd_alone() || rglru(); }       // neither attention nor a matrix state per head
+    bool lat_direct() const { return latent() && d.q_rank == 0; }
+    int lat_q_rows() const { return d.q_rank ? d.q_rank : d.heads * (d.dim + d.rot_dims); }      // first row block of a latent mixer
+    int lat_kv_rows() const { return d.kv_from < 0 ? d.kv_rank + d.rot_dims : 0; }
     bool has_ssd() const { return ssd_alone() || d.side_mixer == KR_SERVE_MIX_SSD; }
     int ssd_inner() const { return d.ssd_heads * d.ssd_vdim; }
     int ssd_conv_c() const { return ssd_inner() + 2 * d.ssd_groups * d.ssd_state; }
     int ssd_in_rows() const { return 2 * ssd_inner() + 2 * d.ssd_groups * d.ssd_state + d.ssd_heads; }
-    int att_out_cols() const { return ssd_alone() ? 0 : d.heads * d.vdim; }                   // the output projection reads [first mixer | state-space mixer]
+    int att_out_cols() const { return ssd_alone() ? 0 : rglru() ? d.rg_width : d.heads * d.vdim; }                   // the output projection reads [first mixer | state-space mixer]
     int o_cols() const { return att_out_cols() + (has_ssd() ? ssd_inner() : 0); }
     int pconv_c() const { return d.heads * d.dim + d.kv_heads * (d.dim + d.vdim); }
     bool ungated_ff() const { return d.dense_act == KR_SERVE_ACT_RELU2; }
-    bool has_cache() const { return !recurrent() && !ssd_alone() && d.kv_from < 0; }
+    bool has_cache() const { return !recurrent() && !no_heads() && d.kv_from < 0; }
     int att_heads_kv() const { return latent() ? 1 : d.kv_heads; }
     int att_dim() const { return latent() ? d.kv_rank + d.rot_dims : d.dim; }       // key row of the attention kernels
     int att_vdim() const { return latent() ? d.kv_rank : d.vdim; }
@@ -85,6 +92,7 @@ struct kr_serve {
     // per-token gate terms, state / normaliser at every block's start, per-block gate terms
     DevBuf h32, hc, rg, qk_rms, lin_o, lin_tok, lin_sbuf, lin_nbuf, lin_cm;
     DevBuf ssd_z;                                         // the state-space mixer's rows in the block recurrence's layout [q | k | v] per head (prompt portions)
+    DevBuf rg_ab, rg_agg, rg_start;                       // real-gated linear recurrence, portions: per token and per chunk of 64
     DevBuf qkv2, sconv, ga1, gz;                          // convolved q | k | v; convolved x | B | C; the gla decay's low-rank input (storage type) and logits
     DevBuf v_first;                                      // [T, kv_heads * vdim] f32: the values of the first value-mixing layer
     DevBuf lq_c, lq_2, lq_n, lq_e, att2, head_i;         // latent mixer: query latent, W_uq output, plain query parts, folded queries, per-head values, head row tables
@@ -187,10 +195,15 @@ int check_layer(const kr_serve_config& c, const kr_serve_layer* all, int i) {
     if (d.pre_add && (!c.pre_norm || c.canon_taps > 1)) return kr_fail(KR_ERR_VALUE, "layer %d: a vector before the layer needs pre-normed blocks without an input convolution", i);
     if (d.dense_act < 0 || d.dense_act > KR_SERVE_ACT_RELU2 || d.expert_act == KR_SERVE_ACT_RELU2) return kr_fail(KR_ERR_VALUE, "layer %d: activation %d / %d", i, d.dense_act, d.expert_act);
     if (d.dense_act == KR_SERVE_ACT_RELU2 && c.res_gate) return kr_fail(KR_ERR_VALUE, "layer %d: the un-gated feed-forward has no gated residual", i);
-    if (ssd1) {
+    if (d.expert_in_weight && (d.mlp_kind != KR_SERVE_MLP_MOE || d.expert_act == KR_SERVE_ACT_RELU2)) return kr_fail(KR_ERR_VALUE, "layer %d: weights on the experts' inputs need experts", i);
+    const bool rg = d.mixer_kind == KR_SERVE_MIX_RGLRU;
+    if (rg && (!kr_sv_rglru_fits(d.rg_width, d.rg_blocks, d.rg_conv) || !(d.rg_rate > 0.0f)))
+        return kr_fail(KR_ERR_VALUE, "layer %d: recurrence sizes (width %d, blocks %d, taps %d, rate %g)", i, d.rg_width, d.rg_blocks, d.rg_conv, (double)d.rg_rate);
+    if (!rg && (d.rg_width || d.rg_blocks || d.rg_conv || d.rg_rate != 0.0f)) return kr_fail(KR_ERR_VALUE, "layer %d: rg_* fields belong to the gated linear recurrence", i);
+    if (ssd1 || rg) {
         if (d.kv_from >= 0 || d.v_mix || d.qk_unit_norm || d.window || d.chunk || d.has_sink || d.dist_bias || d.proj_bias || d.v_from_k || d.out_gate || d.softcap != 0.0f || d.rot_dims ||
             d.proj_conv || d.gate_cap != 0.0f || d.lin_norm_weight)
-            return kr_fail(KR_ERR_VALUE, "layer %d: an attention-only mechanism is switched on for a state-space mixer", i);
+            return kr_fail(KR_ERR_VALUE, "layer %d: an attention-only mechanism is switched on for a mixer without heads", i);
     } else {
     if (d.heads < 1 || d.kv_heads < 1 || d.heads % d.kv_heads) return kr_fail(KR_ERR_VALUE, "layer %d: heads %d / kv_heads %d", i, d.heads, d.kv_heads);
     if (d.dim < 1 || d.vdim < 1 || d.vdim > 512 || d.dim > 512) return kr_fail(KR_ERR_VALUE, "layer %d: head sizes %d / %d (at most 512)", i, d.dim, d.vdim);
@@ -209,7 +222,8 @@ int check_layer(const kr_serve_config& c, const kr_serve_layer* all, int i) {
         if (d.rot_dims && (d.rot_interleaved || d.mixer_kind != KR_SERVE_MIX_RETENTION)) return kr_fail(KR_ERR_VALUE, "layer %d: recurrent mixers rotate half-split pairs, retention only", i);
     } else if (d.gate_cap != 0.0f || d.lin_norm_weight) return kr_fail(KR_ERR_VALUE, "layer %d: gate_cap / lin_norm_weight belong to recurrent mixers", i);
     if (d.v_from_k && (lat || d.vdim != d.dim || d.v_mix || d.kv_from >= 0)) return kr_fail(KR_ERR_VALUE, "layer %d: values that are the keys need vdim == dim, a cache of their own and no value mixing", i);
-    if ((d.proj_bias || d.out_gate) && lat) return kr_fail(KR_ERR_VALUE, "layer %d: a latent mixer has no projection biases / output gate", i);
+    if ((d.proj_bias || d.softcap != 0.0f || (d.out_gate && d.out_gate != KR_SERVE_OGATE_ELEM_SIGMOID)) && lat)
+        return kr_fail(KR_ERR_VALUE, "layer %d: a latent mixer has no projection biases, no capped scores and no gate per head", i);
     if (d.out_gate < 0 || d.out_gate > KR_SERVE_OGATE_ELEM_SIGMOID || d.softcap < 0.0f || d.router_bias < 0 || d.router_bias > KR_SERVE_RBIAS_CHOICE || d.router_score < 0 ||
         d.router_score > KR_SERVE_RSCORE_SIGMOID || d.group_score < 0 || d.group_score > KR_SERVE_GSCORE_TOP2)
         return kr_fail(KR_ERR_VALUE, "layer %d: output gate %d / softcap %g / router bias %d / score %d / group score %d", i, d.out_gate, (double)d.softcap, d.router_bias, d.router_score, d.group_score);
@@ -224,8 +238,9 @@ int check_layer(const kr_serve_config& c, const kr_serve_layer* all, int i) {
     if (d.qk_unit_norm < 0 || d.qk_unit_norm > KR_SERVE_QKNORM_WHOLE || d.has_sink < 0 || d.has_sink > KR_SERVE_SINK_ZERO || d.v_mix < 0 || d.v_mix > KR_SERVE_VMIX_BLEND)
         return kr_fail(KR_ERR_VALUE, "layer %d: qk norm %d / sink %d / value mixing %d", i, d.qk_unit_norm, d.has_sink, d.v_mix);
     if (lat) {
-        if (d.q_rank < 1 || d.kv_rank < 1 || d.kv_rank > 512 || d.kv_rank + d.rot_dims > 1024) return kr_fail(KR_ERR_VALUE, "layer %d: latent sizes %d / %d", i, d.q_rank, d.kv_rank);
-        if (d.kv_from >= 0 || d.v_mix || d.qk_unit_norm || d.kv_heads != 1) return kr_fail(KR_ERR_VALUE, "layer %d: a latent mixer has one latent per token, no borrowed cache, no value mixing, no q / k norm", i);
+        if (d.q_rank < 0 || d.kv_rank < 1 || d.kv_rank > 512 || d.kv_rank + d.rot_dims > 1024) return kr_fail(KR_ERR_VALUE, "layer %d: latent sizes %d / %d", i, d.q_rank, d.kv_rank);
+        if (d.v_mix || d.qk_unit_norm || d.kv_heads != 1 || (d.kv_from >= 0 && d.q_rank > 0))
+            return kr_fail(KR_ERR_VALUE, "layer %d: a latent mixer has one latent per token, no value mixing, no q / k norm, a cache of its own when its queries pass a latent", i);
     }
     if (d.v_mix == KR_SERVE_VMIX_BLEND) {
         int src = -1;
@@ -238,7 +253,11 @@ int check_layer(const kr_serve_config& c, const kr_serve_layer* all, int i) {
         if (d.kv_from >= i) return kr_fail(KR_ERR_VALUE, "layer %d: kv_from %d is not an earlier layer", i, d.kv_from);
         const kr_serve_layer& o = all[d.kv_from];
         if (o.kv_from >= 0) return kr_fail(KR_ERR_VALUE, "layer %d: kv_from %d has no cache of its own", i, d.kv_from);
-        if (o.mixer_kind != d.mixer_kind || o.kv_heads != d.kv_heads || o.dim != d.dim || o.vdim != d.vdim)
+        if (lat && o.mixer_kind == d.mixer_kind) {      // the cached rows must fit; the layer's own heads expand them as they like
+            if (o.kv_rank != d.kv_rank || o.rot_dims != d.rot_dims || (d.rot_dims && (o.rot_interleaved != d.rot_interleaved || o.rot_base != d.rot_base || o.rot_factor != d.rot_factor ||
+                o.rot_scaling != d.rot_scaling || o.rot_original != d.rot_original || o.rot_fast != d.rot_fast || o.rot_slow != d.rot_slow)))
+                return kr_fail(KR_ERR_VALUE, "layer %d: latent or rotated part differs from layer %d", i, d.kv_from);
+        } else if (o.mixer_kind != d.mixer_kind || o.kv_heads != d.kv_heads || o.dim != d.dim || o.vdim != d.vdim)
             return kr_fail(KR_ERR_VALUE, "layer %d: key / value heads differ from layer %d", i, d.kv_from);
     }
     }      // !ssd1
@@ -298,7 +317,7 @@ int kr_serve_create(int device_ordinal, const kr_serve_config* cfg, const kr_ser
         const kr_serve_layer& d = l.d;
         l.have.assign(KR_SV_N_ROLES, 0);
         l.wsrc = d.weights_of ? d.weights_of - 1 : i;
-        l.n_qkv = l.ssd_alone() ? 0 : l.latent() ? d.q_rank + d.kv_rank + d.rot_dims : d.heads * d.dim + (d.kv_from < 0 ? d.kv_heads * (d.dim + (d.v_from_k ? 0 : d.vdim)) : 0);
+        l.n_qkv = l.ssd_alone() ? 0 : l.rglru() ? 2 * d.rg_width : l.latent() ? l.lat_q_rows() + l.lat_kv_rows() : d.heads * d.dim + (d.kv_from < 0 ? d.kv_heads * (d.dim + (d.v_from_k ? 0 : d.vdim)) : 0);
         l.off_ogate = l.n_qkv;
         if (l.recurrent()) l.n_qkv += d.heads * d.vdim; else if (d.out_gate == KR_SERVE_OGATE_HEAD_SIGMOID) l.n_qkv += d.heads; else if (d.out_gate) l.n_qkv += d.heads * d.vdim;
         l.off_if = l.n_qkv;
@@ -383,6 +402,12 @@ int kr_serve_create(int device_ordinal, const kr_serve_config* cfg, const kr_ser
                 kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "recurrent state of %zu bytes", sb + nb);
             }
         }
+        if (l.rglru()) {
+            const size_t sb = (size_t)cfg->max_slots * d.rg_width * 4, cb = sb * d.rg_conv;
+            if (l.rg_state.ensure(sb) || l.rg_ring.ensure(cb) || hipMemset(l.rg_state.p, 0, sb) != hipSuccess || hipMemset(l.rg_ring.p, 0, cb) != hipSuccess) {
+                kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "recurrence state of %zu bytes", sb + cb);
+            }
+        }
         if (l.has_cache()) {
             const size_t rows = (size_t)s->n_pages * cfg->page_tokens;
             const size_t kb = rows * l.att_heads_kv() * l.att_dim() * s->esz, vb = l.latent() ? 0 : rows * d.kv_heads * d.vdim * s->esz;     // a latent's values are its key rows
@@ -432,7 +457,7 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     if (role < 0 || role >= KR_SV_N_ROLES) return kr_fail(KR_ERR_VALUE, "role %d", role);
     const bool moe = d.mlp_kind == KR_SERVE_MLP_MOE;
     const bool lat = l.latent();
-    if (lat && (role == KR_SV_Q || role == KR_SV_K || role == KR_SV_V)) return kr_fail(KR_ERR_VALUE, "layer %d has a latent mixer", layer);
+    if (lat && ((role == KR_SV_Q && d.q_rank) || role == KR_SV_K || role == KR_SV_V)) return kr_fail(KR_ERR_VALUE, "layer %d has a latent mixer", layer);
     if (!lat && role >= KR_SV_DQ && role <= KR_SV_UV) return kr_fail(KR_ERR_VALUE, "layer %d has no latent mixer", layer);
     const bool rec = l.recurrent();
     int rc = KR_OK;
@@ -440,6 +465,11 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     const int inner = l.ssd_inner(), sgn = d.ssd_groups * d.ssd_state;
     if (role >= KR_SV_SSD_IN && role <= KR_SV_SSD_O && !l.has_ssd()) return kr_fail(KR_ERR_VALUE, "layer %d has no state-space mixer", layer);
     if (role >= KR_SV_DECAY_A1 && role <= KR_SV_DECAY_A2_B && !l.gla()) return kr_fail(KR_ERR_VALUE, "layer %d has no gla mixer", layer);
+    if (lat && !d.q_rank && (role == KR_SV_DQ || role == KR_SV_DQ_NORM || role == KR_SV_UQ)) return kr_fail(KR_ERR_VALUE, "layer %d projects its queries without a latent", layer);
+    if (lat && d.kv_from >= 0 && (role == KR_SV_DKV || role == KR_SV_DKV_NORM)) return kr_fail(KR_ERR_VALUE, "layer %d borrows its latents", layer);
+    if ((role >= KR_SV_RG_Y && role <= KR_SV_RG_LAM) != l.rglru() && ((role >= KR_SV_RG_Y && role <= KR_SV_RG_LAM) || role == KR_SV_Q || role == KR_SV_K || role == KR_SV_V))
+        return kr_fail(KR_ERR_VALUE, "layer %d: role %d does not fit its mixer", layer, role);
+    const int rgs = l.rglru() ? d.rg_width / d.rg_blocks : 0;
     if (l.ssd_alone() && (role == KR_SV_Q || role == KR_SV_K || role == KR_SV_V || role == KR_SV_O)) return kr_fail(KR_ERR_VALUE, "layer %d has a state-space mixer only", layer);
     switch (role) {
     case KR_SV_PRE_ADD:
@@ -466,6 +496,27 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     case KR_SV_SSD_D: SHAPE(1, d.ssd_heads); rc = upload(s, l.ssd_d, n, 0, host, src_dtype, n, true); break;
     case KR_SV_SSD_NORM: SHAPE(1, inner); rc = upload(s, l.ssd_norm, n, 0, host, src_dtype, n, true); break;
     case KR_SV_SSD_O: SHAPE(W, inner); rc = upload_cols(s, l.o, W, l.o_cols(), l.att_out_cols(), host, src_dtype, inner); break;
+    case KR_SV_RG_Y: case KR_SV_RG_X: SHAPE(d.rg_width, W); rc = upload(s, l.hw, (size_t)l.n_h * W, role == KR_SV_RG_X ? (size_t)d.rg_width * W : 0, host, src_dtype, n, false); break;
+    case KR_SV_RG_Y_B: SHAPE(1, d.rg_width); rc = upload(s, l.rg_yb, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_RG_X_B: SHAPE(1, d.rg_width); rc = upload(s, l.rg_xb, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_RG_CONV: SHAPE(d.rg_width, d.rg_conv); rc = upload(s, l.rg_conv, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_RG_CONV_B: SHAPE(1, d.rg_width); rc = upload(s, l.rg_convb, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_RG_RA: case KR_SV_RG_RI: {      // [blocks][2][size][size]: both gates of a block stand together
+        SHAPE(d.rg_width, rgs);
+        const size_t bb = (size_t)rgs * rgs, hb = bb * (src_dtype == KR_SERVE_F32 ? 4 : 2);
+        for (int b = 0; b < d.rg_blocks && !rc; b++) rc = upload(s, l.rg_w, 2 * n, (2 * (size_t)b + (role == KR_SV_RG_RI)) * bb, (const char*)host + b * hb, src_dtype, bb, false);
+        break;
+    }
+    case KR_SV_RG_RA_B: case KR_SV_RG_RI_B: SHAPE(d.rg_blocks, rgs); rc = upload(s, l.rg_b, 2 * n, role == KR_SV_RG_RI_B ? n : 0, host, src_dtype, n, true); break;
+    case KR_SV_RG_LAM: {                       // kept as -rate * softplus(lam)
+        SHAPE(1, d.rg_width);
+        std::vector<float> r(n);
+        for (size_t k = 0; k < n; k++) {
+            const double z = src_dtype == KR_SERVE_F32 ? ((const float*)host)[k] : bf16_to_f32_host(((const uint16_t*)host)[k]);
+            r[k] = (float)(-(double)d.rg_rate * (std::max(z, 0.0) + std::log1p(std::exp(-std::fabs(z)))));
+        }
+        rc = upload(s, l.rg_rate, n, 0, r.data(), KR_SERVE_F32, n, true); break;
+    }
     case KR_SV_Q_BIAS: case KR_SV_K_BIAS: case KR_SV_O_BIAS:
         if (!d.proj_bias) return kr_fail(KR_ERR_VALUE, "layer %d has no projection biases", layer);
         SHAPE(1, role == KR_SV_Q_BIAS ? nq : role == KR_SV_K_BIAS ? nk : W);
@@ -513,7 +564,7 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     case KR_SV_ROUTER_BIAS: if (!moe || !d.router_bias) return kr_fail(KR_ERR_VALUE, "layer %d has no router bias", layer);
         SHAPE(1, d.experts); rc = upload(s, l.router_b, n, 0, host, src_dtype, n, true); break;
     case KR_SV_DQ: SHAPE(d.q_rank, W); rc = upload(s, l.hw, (size_t)l.n_h * W, 0, host, src_dtype, n, false); break;
-    case KR_SV_DKV: SHAPE(d.kv_rank + d.rot_dims, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)d.q_rank * W, host, src_dtype, n, false); break;
+    case KR_SV_DKV: SHAPE(d.kv_rank + d.rot_dims, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)l.lat_q_rows() * W, host, src_dtype, n, false); break;
     case KR_SV_DQ_NORM: SHAPE(1, d.q_rank); rc = upload(s, l.dq_norm, n, 0, host, src_dtype, n, true); break;
     case KR_SV_DKV_NORM: SHAPE(1, d.kv_rank); rc = upload(s, l.dkv_norm, n, 0, host, src_dtype, n, true); break;
     case KR_SV_UQ: SHAPE(d.heads * (d.dim + d.rot_dims), d.q_rank); rc = upload(s, l.uq, n, 0, host, src_dtype, n, false); break;
@@ -531,13 +582,13 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     }
     case KR_SV_NORM_W: SHAPE(1, W); rc = upload_norm_w(s, l.norm_w, host, src_dtype, n); break;
     case KR_SV_NORM_B: SHAPE(1, W); rc = upload(s, l.norm_b, n, 0, host, src_dtype, n, true); break;
-    case KR_SV_Q: SHAPE(nq, W); rc = upload(s, l.hw, (size_t)l.n_h * W, 0, host, src_dtype, n, false); break;
+    case KR_SV_Q: SHAPE(lat ? l.lat_q_rows() : nq, W); rc = upload(s, l.hw, (size_t)l.n_h * W, 0, host, src_dtype, n, false); break;
     case KR_SV_K: if (d.kv_from >= 0) return kr_fail(KR_ERR_VALUE, "layer %d borrows its keys", layer);
         SHAPE(nk, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)nq * W, host, src_dtype, n, false); break;
     case KR_SV_V: if (d.kv_from >= 0 || d.v_from_k) return kr_fail(KR_ERR_VALUE, "layer %d has no value projection", layer);
         SHAPE(nv, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)(nq + nk) * W, host, src_dtype, n, false); break;
-    case KR_SV_O: SHAPE(W, d.heads * d.vdim);
-        if (l.has_ssd()) rc = upload_cols(s, l.o, W, l.o_cols(), 0, host, src_dtype, d.heads * d.vdim);
+    case KR_SV_O: SHAPE(W, l.att_out_cols());
+        if (l.has_ssd()) rc = upload_cols(s, l.o, W, l.o_cols(), 0, host, src_dtype, l.att_out_cols());
         else rc = upload(s, l.o, n, 0, host, src_dtype, n, false);
         break;
     case KR_SV_SINK: if (d.has_sink != KR_SERVE_SINK_TENSOR) return kr_fail(KR_ERR_VALUE, "layer %d has no sink tensor", layer);
@@ -659,8 +710,14 @@ int kr_serve_fill_synthetic(kr_serve* s, uint64_t seed, float amp) {
         }
         if (d.v_mix == KR_SERVE_VMIX_BLEND) { bad |= vec(l.vmix, 1, true); const float half = 0.5f; bad |= hipMemcpy(l.vmix.p, &half, 4, hipMemcpyHostToDevice) != hipSuccess; }
         if (l.latent()) {
-            bad |= vec(l.dq_norm, d.q_rank, true) | vec(l.dkv_norm, d.kv_rank, true) | mat(l.uq, (size_t)d.heads * (d.dim + d.rot_dims) * d.q_rank, d.q_rank) |
-                   mat(l.ukT, (size_t)d.heads * d.kv_rank * d.dim, d.kv_rank) | mat(l.uv, (size_t)d.heads * d.vdim * d.kv_rank, d.kv_rank);
+            if (d.q_rank) bad |= vec(l.dq_norm, d.q_rank, true) | mat(l.uq, (size_t)d.heads * (d.dim + d.rot_dims) * d.q_rank, d.q_rank);
+            if (d.kv_from < 0) bad |= vec(l.dkv_norm, d.kv_rank, true);
+            bad |= mat(l.ukT, (size_t)d.heads * d.kv_rank * d.dim, d.kv_rank) | mat(l.uv, (size_t)d.heads * d.vdim * d.kv_rank, d.kv_rank);
+        }
+        if (l.rglru()) {             // decays between 0.7 and one, as trained recurrences have them
+            const size_t D = d.rg_width;
+            bad |= vec(l.rg_yb, D, false) | vec(l.rg_xb, D, false) | vecu(l.rg_conv, D * d.rg_conv, 1.0f / (float)d.rg_conv, 0.5f / (float)d.rg_conv) | vec(l.rg_convb, D, false) |
+                   mat(l.rg_w, 2 * D * (D / d.rg_blocks), (int)(D / d.rg_blocks)) | vec(l.rg_b, 2 * D, false) | vecu(l.rg_rate, D, -0.35f, 0.34f);
         }
         if (d.mlp_kind == KR_SERVE_MLP_DENSE) bad |= mat(l.down, (size_t)W * d.ff, d.ff);
         if (d.mlp_kind == KR_SERVE_MLP_MOE) {
@@ -695,8 +752,12 @@ int kr_serve_finalize(kr_serve* s) {
         if (s->c.pre_norm && seq && has_ff) { need.push_back(KR_SV_NORM2_W); if (nb) need.push_back(KR_SV_NORM2_B); }
         if (s->c.post_norm) { need.push_back(KR_SV_POST1_W); if (nb) need.push_back(KR_SV_POST1_B); }
         if (s->c.post_norm && has_ff) { need.push_back(KR_SV_POST2_W); if (nb) need.push_back(KR_SV_POST2_B); }
-        if (l.latent()) for (int r : {KR_SV_DQ, KR_SV_DQ_NORM, KR_SV_UQ, KR_SV_DKV, KR_SV_DKV_NORM, KR_SV_UK, KR_SV_UV}) need.push_back(r);
-        else if (!l.ssd_alone()) {
+        if (l.rglru()) for (int r = KR_SV_RG_Y; r <= KR_SV_RG_LAM; r++) need.push_back(r);
+        if (l.latent()) {
+            if (d.q_rank) for (int r : {KR_SV_DQ, KR_SV_DQ_NORM, KR_SV_UQ}) need.push_back(r); else need.push_back(KR_SV_Q);
+            if (d.kv_from < 0) for (int r : {KR_SV_DKV, KR_SV_DKV_NORM}) need.push_back(r);
+            for (int r : {KR_SV_UK, KR_SV_UV}) need.push_back(r);
+        } else if (!l.no_heads()) {
             need.push_back(KR_SV_Q);
             if (d.kv_from < 0) { need.push_back(KR_SV_K); if (!d.v_from_k) need.push_back(KR_SV_V); }
         }
@@ -835,6 +896,9 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     size_t max_pconv = 0, max_sconv = 0, max_ga1 = 0, max_gz = 0, max_ssdz = 0;
     // prompt portions take the chunked form of the recurrent mixers (blocks of 64 tokens on the matrix instruction), decode-sized steps the token-by-token form
     const bool lin_chunked = max_count >= 32;
+    // the gated linear recurrence: one launch when every entry brings one token, else chunks of 64 tokens
+    const bool rg_step = max_count == 1;
+    size_t max_rg = 0;
     for (const SvLayer& l : s->L) {
         const kr_serve_layer& d = l.d;
         if (d.proj_conv) max_pconv = std::max(max_pconv, (size_t)l.pconv_c());
@@ -852,6 +916,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
                 lin_tok = std::max(lin_tok, (size_t)d.heads); lin_sb = std::max(lin_sb, (size_t)d.heads * d.dim * d.vdim); lin_nb = std::max(lin_nb, (size_t)d.heads * d.dim);
             }
         }
+        if (l.rglru() && !rg_step) max_rg = std::max(max_rg, (size_t)d.rg_width);
         if (d.qk_unit_norm == KR_SERVE_QKNORM_WHOLE) whole_norm = true;
         max_qkv = std::max(max_qkv, (size_t)l.n_h); max_att = std::max(max_att, std::max((size_t)d.heads * l.att_vdim(), (size_t)l.o_cols()));
         if (d.v_mix) max_vf = std::max(max_vf, (size_t)d.kv_heads * d.vdim);
@@ -869,7 +934,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     const size_t Ts = (size_t)T;
     if (s->x.ensure(Ts * W * 4) || s->h.ensure(Ts * W * s->esz) || s->qkv.ensure(Ts * max_qkv * 4) || s->att.ensure(Ts * max_att * s->esz) || s->mix.ensure(Ts * W * 4) ||
         s->gu.ensure(Ts * max_gu * 4 + 16) || s->y.ensure(Ts * max_y * s->esz + 16) || s->rows.ensure(Ts * max_rows * 4 + 16) || s->ffout.ensure(Ts * W * 4) ||
-        s->ids.ensure(Ts * max_pairs * 4 + 16) || s->rz.ensure(Ts * (size_t)max_E * 8 + 16) || s->wts.ensure(Ts * max_pairs * 4 + 16) || s->moe_i.ensure((Ts * max_pairs * 3 + 3 * (size_t)max_E + 8) * 4) ||
+        s->ids.ensure(Ts * max_pairs * 4 + 16) || s->rz.ensure(Ts * (size_t)max_E * 8 + 16) || s->wts.ensure(Ts * max_pairs * 4 + 16) || s->moe_i.ensure((Ts * max_pairs * 4 + 3 * (size_t)max_E + 8) * 4) ||
         s->hw.ensure((size_t)std::max(n_want, 1) * W * s->esz) || s->logits.ensure((size_t)std::max(n_want, 1) * c.vocab * 4) || s->amax.ensure((size_t)std::max(n_want, 1) * 4))
         return kr_fail(KR_ERR_HIP, "step scratch for %d tokens", T);
     if ((max_vf && s->v_first.ensure(Ts * max_vf * 4)) ||
@@ -882,13 +947,15 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         return kr_fail(KR_ERR_HIP, "block scratch for %d tokens", T);
     if ((max_pconv && s->qkv2.ensure(Ts * max_pconv * 4)) || (max_sconv && s->sconv.ensure(Ts * max_sconv * 4)) || (max_ga1 && (s->ga1.ensure(Ts * max_ga1 * s->esz) || s->gz.ensure(Ts * max_gz * 4))))
         return kr_fail(KR_ERR_HIP, "convolution / decay scratch for %d tokens", T);
+    if (max_rg && (s->rg_ab.ensure(Ts * max_rg * 8) || s->rg_agg.ensure((size_t)n_chunks * max_rg * 8) || s->rg_start.ensure((size_t)n_chunks * max_rg * 4)))
+        return kr_fail(KR_ERR_HIP, "recurrence scratch for %d tokens", T);
     if (max_ssdz && s->ssd_z.ensure(Ts * max_ssdz * 4)) return kr_fail(KR_ERR_HIP, "state-space block scratch for %d tokens", T);
     for (SvRope& r : s->ropes) if (r.cs.ensure(Ts * (r.dims / 2) * 8)) return kr_fail(KR_ERR_HIP, "rope table");
     if (s->capture) { if (s->cap.ensure((size_t)c.n_layers * Ts * W * 4)) return kr_fail(KR_ERR_HIP, "capture buffer"); s->cap_T = T; }
     std::vector<int> nsplit(c.n_layers, 1);
     for (int li = 0; li < c.n_layers; li++) {
         const SvLayer& l = s->L[li]; const kr_serve_layer& d = l.d;
-        if (l.recurrent() || l.ssd_alone()) continue;
+        if (l.recurrent() || l.no_heads()) continue;
         const int visible = d.window > 0 ? std::min(max_pos + 1, d.window) : (d.chunk > 0 ? std::min(max_pos + 1, d.chunk) : max_pos + 1);
         const int ldk = l.latent() ? l.att_dim() : d.kv_heads * d.dim, ldv = l.latent() ? l.att_dim() : d.kv_heads * d.vdim;
         nsplit[li] = kr_sv_attention_splits(T, d.heads, l.att_heads_kv(), l.att_dim(), l.att_vdim(), ldk, ldv, s->f32, visible);
@@ -911,9 +978,9 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     }
     int* mi = (int*)s->moe_i.p;
     // down projection of a gated feed-forward: decode-sized problems form the activation inside the projection's launch, larger ones write it once
-    auto down_proj = [&](KrSvGemm g, const float* gu, int ld, int rows_m, int F, int kind, float limit, float alpha) {
-        if (kr_sv_gemm_small(g)) { g.act_gu = gu; g.act_ld = ld; g.act_kind = kind; g.act_limit = limit; g.act_alpha = alpha; g.A = nullptr; Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); return; }
-        { Timer tm(s, 5); kr_sv_act(gu, ld, s->y.p, s->f32, rows_m, F, kind, limit, alpha, st); }
+    auto down_proj = [&](KrSvGemm g, const float* gu, int ld, int rows_m, int F, int kind, float limit, float alpha, const float* row_w = nullptr) {
+        if (kr_sv_gemm_small(g)) { g.act_row_w = row_w; g.act_gu = gu; g.act_ld = ld; g.act_kind = kind; g.act_limit = limit; g.act_alpha = alpha; g.A = nullptr; Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); return; }
+        { Timer tm(s, 5); kr_sv_act(gu, ld, s->y.p, s->f32, rows_m, F, kind, limit, alpha, row_w, st); }
         g.A = s->y.p; g.lda = F;
         { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
     };
@@ -938,7 +1005,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             } else if (res_gate_kind == 2 && c.res_gate) { r.gate = (const float*)s->qkv.p + rl.off_rg2; r.ld_gate = rl.n_h; r.gate_b = (const float*)rl.rg2_b.p; }
         }
         if (canon && hand_on && res_to_mixer) r.h32_out = (float*)s->h32.p;
-        r.x = x; r.mix = mixp; r.dense = dense; r.shared = shared; r.rows = rows; r.pair_pos = pair_pos; r.wts = (const float*)s->wts.p; r.top = top;
+        r.x = x; r.mix = mixp; r.dense = dense; r.shared = shared; r.rows = rows; r.pair_pos = pair_pos; r.wts = (res_layer && res_layer->d.expert_in_weight) ? nullptr : (const float*)s->wts.p; r.top = top;
         r.post_w = post_w ? (const float*)post_w->p : nullptr; r.post_b = (post_w && c.norm_bias && post_b) ? (const float*)post_b->p : nullptr; r.mult = c.residual_mult;
         r.norm_w = (hand_on && next_w) ? (const float*)next_w->p : nullptr; r.norm_b = (hand_on && next_w && c.norm_bias && next_b) ? (const float*)next_b->p : nullptr;
         r.h_out = hand_on ? s->h.p : nullptr; r.T = T; r.width = W; r.kind = c.norm_kind; r.eps = c.norm_eps;
@@ -1013,6 +1080,15 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
                 else kr_sv_lin_scan(q, st);
             }
             { Timer tm(s, 2); kr_sv_lin_out(q, s->f32, st); }
+        } else if (l.rglru()) {
+            KrSvRglru q{};
+            q.y = hz; q.x = hz + d.rg_width; q.ld = l.n_h; q.y_b = (const float*)l.rg_yb.p; q.x_b = (const float*)l.rg_xb.p; q.conv = (const float*)l.rg_conv.p;
+            q.conv_b = (const float*)l.rg_convb.p; q.taps = d.rg_conv; q.gw = l.rg_w.p; q.gb = (const float*)l.rg_b.p; q.rate = (const float*)l.rg_rate.p; q.width = d.rg_width; q.blocks = d.rg_blocks;
+            q.state = (float*)run.rg_state.p; q.ring = (float*)run.rg_ring.p; q.ent_off = d_eoff; q.ent_slot = d_eslot; q.n_entries = n_entries; q.ent_chunk0 = d_echunk; q.n_chunks = n_chunks;
+            q.pos = d_pos; q.T = T; q.out = s->att.p; q.out_ld = l.o_cols();
+            q.ab = (float2*)s->rg_ab.p; q.agg = (float2*)s->rg_agg.p; q.start = (float*)s->rg_start.p;
+            Timer tm(s, 3);
+            if (rg_step) kr_sv_rglru_step(q, s->f32, st); else kr_sv_rglru_portions(q, s->f32, st);
         } else if (l.ssd_alone()) {
             // no first mixer: the state-space mixer below is the layer's only one
         } else if (!l.latent()) {
@@ -1038,30 +1114,35 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             { Timer tm(s, 2); kr_sv_qk_prep(a, s->f32, st); }
             { Timer tm(s, 3); kr_sv_attention(a, s->f32, st); }
         } else {
-            // queries: norm the latent, W_uq, turn the rotated part, fold W_uk of every head into the plain part; keys / values: the normed latent and the
+            // queries: norm the latent, W_uq (or as projected), turn the rotated part, fold W_uk of every head into the plain part; keys / values: the normed latent and the
             // turned shared part are the cache row, read by the attention kernels as ONE key / value head whose values are the leading kv_rank of the key row
             const int H = d.heads, R = d.kv_rank, De = l.att_dim();
             KrSvLatent q{};
             q.dz = hz; q.ld = l.n_h; q.q_rank = d.q_rank; q.kv_rank = R; q.rot = d.rot_dims; q.heads = H; q.dim = d.dim;
+            q.rot_interleaved = d.rot_interleaved; q.own_kv = d.kv_from < 0;
             q.dq_norm_w = (const float*)l.dq_norm.p; q.dkv_norm_w = (const float*)l.dkv_norm.p; q.eps = c.norm_eps;
             q.cs = d.rot_dims ? (const float2*)s->ropes[l.rope_id].cs.p : nullptr; q.cq = s->lq_c.p;
-            q.pool = l.kpool.p; q.page_table = d_tab; q.table_ld = s->n_pages; q.slot = d_slot; q.pos = d_pos; q.page_tokens = PT; q.T = T;
+            q.pool = kvl.kpool.p; q.page_table = d_tab; q.table_ld = s->n_pages; q.slot = d_slot; q.pos = d_pos; q.page_tokens = PT; q.T = T;
             int* hseg = (int*)s->head_i.p; int* hrows = hseg + H + 1; int* hgroup = hrows + (size_t)T * H;
             {
                 Timer tm(s, 2);
-                kr_sv_latent_prep(q, s->f32, st);
+                if (l.lat_direct()) kr_sv_latent_direct(q, s->lq_n.p, (float*)s->lq_e.p, s->f32, st);
+                else kr_sv_latent_prep(q, s->f32, st);
                 if (head_rows_for != H) { kr_sv_head_rows(T, H, hseg, hrows, hgroup, st); head_rows_for = H; }
             }
-            g = KrSvGemm{}; g.A = s->lq_c.p; g.lda = d.q_rank; g.W = l.uq.p; g.C = (float*)s->lq_2.p; g.ldc = H * (d.dim + d.rot_dims); g.M = T; g.N = g.ldc; g.K = d.q_rank;
-            { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
-            { Timer tm(s, 2); kr_sv_latent_q(q, (const float*)s->lq_2.p, s->lq_n.p, (float*)s->lq_e.p, s->f32, st); }
+            if (!l.lat_direct()) {
+                g = KrSvGemm{}; g.A = s->lq_c.p; g.lda = d.q_rank; g.W = l.uq.p; g.C = (float*)s->lq_2.p; g.ldc = H * (d.dim + d.rot_dims); g.M = T; g.N = g.ldc; g.K = d.q_rank;
+                { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
+                { Timer tm(s, 2); kr_sv_latent_q(q, (const float*)s->lq_2.p, s->lq_n.p, (float*)s->lq_e.p, s->f32, st); }
+            }
             g = KrSvGemm{}; g.A = s->lq_n.p; g.lda = d.dim; g.a_rows = hrows; g.W = l.ukT.p; g.w_stride = (size_t)R * d.dim; g.C = (float*)s->lq_e.p; g.ldc = De; g.c_rows = hrows;
             g.M = T * H; g.N = R; g.K = d.dim; g.seg = hseg; g.row_group = hgroup; g.n_groups = H; g.rowwise_upto = 16 * H;
             { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
-            a.qkv = (float*)s->lq_e.p; a.ldq = H * De; a.vpool = l.kpool.p; a.ldk = De; a.ldv = De;
+            a.qkv = (float*)s->lq_e.p; a.ldq = H * De; a.vpool = kvl.kpool.p; a.ldk = De; a.ldv = De;
             { Timer tm(s, 3); kr_sv_attention(a, s->f32, st); }
             g = KrSvGemm{}; g.A = s->att.p; g.lda = R; g.a_rows = hrows; g.W = l.uv.p; g.w_stride = (size_t)d.vdim * R; g.C = (float*)s->att2.p; g.ldc = d.vdim; g.c_rows = hrows; g.c_storage = 1;
             g.M = T * H; g.N = d.vdim; g.K = R; g.seg = hseg; g.row_group = hgroup; g.n_groups = H; g.rowwise_upto = 16 * H;
+            if (d.out_gate) { g.o_gate = hz + l.off_ogate; g.o_gate_ld = l.n_h; g.o_gate_div = H; }
             { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
             o_in = s->att2.p;
         }
@@ -1124,18 +1205,19 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         } else if (d.mlp_kind == KR_SERVE_MLP_MOE) {
             const int E = d.experts, top = d.top, F = d.expert_ff, P = T * top;
             int* counts_d = mi; int* seg = mi + E; int* cursor = seg + E + 1; int* src_row = cursor + E; int* row_group = src_row + P; int* pp = row_group + P;
+            float* row_w = d.expert_in_weight ? (float*)(pp + P) : nullptr;
             {
                 Timer tm(s, 4);
                 kr_sv_router_select(hz + l.off_router, l.n_h, s->f32 ? 1 : 2, d.router_bias ? (const float*)l.router_b.p : nullptr, d.router_bias, d.router_score, d.group_score, T, E, top,
                                     d.groups, d.keep, d.renorm, (int*)s->ids.p, (float*)s->wts.p, st);
-                kr_sv_moe_sort((const int*)s->ids.p, T, top, E, counts_d, seg, cursor, src_row, row_group, pp, st);
+                kr_sv_moe_sort((const int*)s->ids.p, T, top, E, counts_d, seg, cursor, src_row, row_group, pp, (const float*)s->wts.p, row_w, st);
             }
             g = KrSvGemm{}; g.A = s->h.p; g.lda = W; g.W = l.egu.p; g.w_stride = (size_t)2 * F * W; g.C = (float*)s->gu.p; g.ldc = 2 * F; g.M = P; g.N = 2 * F; g.K = W;
             g.a_rows = src_row; g.seg = seg; g.row_group = row_group; g.n_groups = E;
             { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
             g = KrSvGemm{}; g.W = l.edown.p; g.w_stride = (size_t)W * F; g.C = (float*)s->rows.p; g.ldc = W; g.M = P; g.N = W; g.K = F;
             g.seg = seg; g.row_group = row_group; g.n_groups = E;
-            down_proj(g, (const float*)s->gu.p, 2 * F, P, F, d.expert_act, d.expert_limit, d.expert_alpha);
+            down_proj(g, (const float*)s->gu.p, 2 * F, P, F, d.expert_act, d.expert_limit, d.expert_alpha, row_w);
             rows = (const float*)s->rows.p; pair_pos = pp;
             if (d.shared_ff > 0) {
                 const int SF = d.shared_ff;
@@ -1170,7 +1252,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         mixin((uint64_t)T); mixin((uint64_t)n_want); mixin(want_amax);
         for (int v : nsplit) mixin((uint64_t)v);
         for (const DevBuf* b : {&s->meta, &s->x, &s->h, &s->qkv, &s->att, &s->mix, &s->gu, &s->y, &s->rows, &s->ffout, &s->ids, &s->wts, &s->rz, &s->moe_i, &s->hw, &s->logits,
-                                &s->amax, &s->part_ml, &s->part_acc, &s->v_first, &s->lq_c, &s->lq_2, &s->lq_n, &s->lq_e, &s->att2, &s->head_i, &s->h32, &s->hc, &s->rg, &s->qk_rms, &s->lin_o, &s->qkv2, &s->sconv, &s->ga1, &s->gz}) mixin((uint64_t)(uintptr_t)b->p);
+                                &s->amax, &s->part_ml, &s->part_acc, &s->v_first, &s->lq_c, &s->lq_2, &s->lq_n, &s->lq_e, &s->att2, &s->head_i, &s->h32, &s->hc, &s->rg, &s->qk_rms, &s->lin_o, &s->qkv2, &s->sconv, &s->ga1, &s->gz, &s->rg_ab, &s->rg_agg, &s->rg_start}) mixin((uint64_t)(uintptr_t)b->p);
         for (const SvRope& r : s->ropes) mixin((uint64_t)(uintptr_t)r.cs.p);
         hipGraphExec_t exec = nullptr;
         for (auto& g : s->graphs) if (g.key == key) exec = g.exec;

@@ -22,7 +22,9 @@ __device__ __forceinline__ float gm_ld(const uint16_t* p) { return kr_bf16_to_f3
 // one element of C: f32, or the storage type when the output feeds another GEMM as it is (BF = a bf16 store)
 template <bool BF>
 __device__ __forceinline__ void gm_store(const KrSvGemm& g, int m, int n, float v) {
-    const size_t i = (size_t)(g.c_rows ? g.c_rows[m] : m) * g.ldc + n;
+    const int row = g.c_rows ? g.c_rows[m] : m;
+    const size_t i = (size_t)row * g.ldc + n;
+    if (g.o_gate) v *= 1.0f / (1.0f + expf(-g.o_gate[(size_t)(row / g.o_gate_div) * g.o_gate_ld + (size_t)(row % g.o_gate_div) * g.N + n]));
     if (BF && g.c_storage) ((uint16_t*)g.C)[i] = kr_f32_to_bf16(v);
     else g.C[i] = v;
 }
@@ -63,13 +65,14 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
     const T* wr[CN];
 #pragma unroll
     for (int c = 0; c < CN; c++) wr[c] = W + (size_t)min(n0 + c, g.N - 1) * g.K;       // columns past N repeat the last one and are not stored
-    const T* ar[MB]; const float* gr[MB];
+    const T* ar[MB]; const float* gr[MB]; float gw[MB];
 #pragma unroll
     for (int m = 0; m < MB; m++) {
         const int r = min(m0 + m, g.M - 1);
         const int src = g.a_rows ? g.a_rows[r] : r;
         ar[m] = ACT ? nullptr : (const T*)g.A + (size_t)src * g.lda;
         gr[m] = ACT ? g.act_gu + (size_t)src * g.act_ld : nullptr;
+        gw[m] = ACT && g.act_row_w ? g.act_row_w[r] : 1.0f;
     }
     const int uoff = g.act_kind == KR_SV_ACT_RELU2 ? 0 : g.K;     // an un-gated activation has no up columns: the second read repeats the first
     float acc[MB][CN];
@@ -92,8 +95,8 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
 #pragma unroll
                         for (int q = 0; q < VEC / 4; q++) {
                             const float4 gg = *reinterpret_cast<const float4*>(gr[m] + k + 4 * q), uu = *reinterpret_cast<const float4*>(gr[m] + uoff + k + 4 * q);
-                            af[4 * q] = gm_round<T>(gm_act(gg.x, uu.x, g.act_kind, g.act_limit, g.act_alpha)); af[4 * q + 1] = gm_round<T>(gm_act(gg.y, uu.y, g.act_kind, g.act_limit, g.act_alpha));
-                            af[4 * q + 2] = gm_round<T>(gm_act(gg.z, uu.z, g.act_kind, g.act_limit, g.act_alpha)); af[4 * q + 3] = gm_round<T>(gm_act(gg.w, uu.w, g.act_kind, g.act_limit, g.act_alpha));
+                            af[4 * q] = gm_round<T>(gm_act(gg.x * gw[m], uu.x * gw[m], g.act_kind, g.act_limit, g.act_alpha)); af[4 * q + 1] = gm_round<T>(gm_act(gg.y * gw[m], uu.y * gw[m], g.act_kind, g.act_limit, g.act_alpha));
+                            af[4 * q + 2] = gm_round<T>(gm_act(gg.z * gw[m], uu.z * gw[m], g.act_kind, g.act_limit, g.act_alpha)); af[4 * q + 3] = gm_round<T>(gm_act(gg.w * gw[m], uu.w * gw[m], g.act_kind, g.act_limit, g.act_alpha));
                         }
                     } else {
                         const gu4 av = *reinterpret_cast<const gu4*>(ar[m] + k);
@@ -130,7 +133,7 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
             for (int m = 0; m < MB; m++) {
                 if (m < mcnt) {
                     float av;
-                    if constexpr (ACT) av = gm_round<T>(gm_act(gr[m][k], gr[m][uoff + k], g.act_kind, g.act_limit, g.act_alpha));
+                    if constexpr (ACT) av = gm_round<T>(gm_act(gr[m][k] * gw[m], gr[m][uoff + k] * gw[m], g.act_kind, g.act_limit, g.act_alpha));
                     else av = gm_ld(ar[m] + k);
 #pragma unroll
                     for (int c = 0; c < CN; c++) acc[m][c] = __builtin_fmaf(av, w[c], acc[m][c]);

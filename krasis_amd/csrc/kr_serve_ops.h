@@ -24,6 +24,9 @@ struct KrSvGemm {
     const int* c_rows;               // optional: problem row r writes C row c_rows[r] (a grouped problem whose rows return to their own order)
     int c_storage;                   // != 0: C holds the storage type (bf16 in a bf16 store) instead of f32 -- the output feeds another GEMM as it is
     int rowwise_upto;                // grouped problems: the wave-per-column form up to this many rows (0 = the default of 64)
+    const float* act_row_w;          // with act_gu: [M] or null, multiplies the gate and up columns of problem row r before the activation (a weight on the expert's input)
+    // [*, o_gate_ld] f32 or null: an element of C is multiplied by sigmoid(o_gate[row / o_gate_div][(row % o_gate_div) * N + n]) before it is stored, row = its row in C
+    const float* o_gate; int o_gate_ld, o_gate_div;
 };
 void kr_sv_gemm(const KrSvGemm& g, bool f32, hipStream_t st);
 bool kr_sv_gemm_small(const KrSvGemm& g);      // true: kr_sv_gemm takes the wave-per-column form for this problem (and honours act_gu)
@@ -123,11 +126,13 @@ void kr_sv_attention(const KrSvAttn& a, bool f32, hipStream_t st);   // windowed
 // 1: the sum of its two largest.  Experts outside the kept groups cannot be chosen, whatever their score.  renorm: weights / (their sum + 1e-20).
 void kr_sv_router_select(const float* z, int ld, int parts, const float* bias, int bias_mode, int score_kind, int group_kind, int T, int E, int top, int groups, int keep,
                          int renorm, int* ids, float* wts, hipStream_t st);
-// rows of every expert: seg[E + 1], src_row[T * top] (token of sorted row), row_group[T * top], pair_pos[T * top] (sorted row of (token, slot))
-void kr_sv_moe_sort(const int* ids, int T, int top, int E, int* counts, int* seg, int* cursor, int* src_row, int* row_group, int* pair_pos, hipStream_t st);
-// gu rows `ld` floats apart (gate at [0, F), up at [F, 2F)) -> y [M, F] storage type
-void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, hipStream_t st);
-// y[t] = mix[t] + (dense[t] + shared[t] + sum_s wts[t][s] * rows[pair_pos[t][s]]) (null terms are skipped); with post_w, y <- norm(y) * post_w (+ post_b);
+// rows of every expert: seg[E + 1], src_row[T * top] (token of sorted row), row_group[T * top], pair_pos[T * top] (sorted row of (token, slot)); with row_w also
+// the weight of every sorted row (wts [T * top])
+void kr_sv_moe_sort(const int* ids, int T, int top, int E, int* counts, int* seg, int* cursor, int* src_row, int* row_group, int* pair_pos, const float* wts, float* row_w,
+                    hipStream_t st);
+// gu rows `ld` floats apart (gate at [0, F), up at [F, 2F)) -> y [M, F] storage type; row_w [M] or null: multiplies a row's gate and up columns first
+void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, const float* row_w, hipStream_t st);
+// y[t] = mix[t] + (dense[t] + shared[t] + sum_s wts[t][s] * rows[pair_pos[t][s]]) (null terms are skipped, null wts are ones); with post_w, y <- norm(y) * post_w (+ post_b);
 // x[t] += mult * y[t].  With h_out the NEW row goes there in the storage type by the same launch: normed with norm_w (+ norm_b) -- the next sublayer's
 // input -- or, without norm_w, as it is.
 struct KrSvResidual {
@@ -144,20 +149,24 @@ struct KrSvResidual {
 };
 void kr_sv_residual_norm(const KrSvResidual& r, bool out_f32, hipStream_t st);
 
-// ---- latent mixer (queries and keys / values through low-rank latents; the cache row is [latent | rotated shared key part])
+// ---- latent mixer (keys / values, and with q_rank > 0 the queries, through low-rank latents; the cache row is [latent | rotated shared key part])
 struct KrSvLatent {
-    const float* dz; int ld;         // [T, ld] f32: W_dq h [q_rank] | W_dkv h [kv_rank + rot]
+    const float* dz; int ld;         // [T, ld] f32: W_dq h [q_rank] or, with q_rank 0, the heads' queries [heads * (dim + rot)] | (own_kv) W_dkv h [kv_rank + rot]
     int q_rank, kv_rank, rot, heads, dim;
+    int rot_interleaved;             // pairs (2i, 2i + 1), else (i, i + rot / 2)
+    int own_kv;                      // 0: the layer reads another layer's cache rows and writes none
     const float* dq_norm_w; const float* dkv_norm_w; float eps;
     const float2* cs;                // rotation table of the step [T, rot / 2]
     void* cq;                        // out [T, q_rank] storage type: rms(W_dq h) * w
     void* pool; const int* page_table; int table_ld; const int* slot; const int* pos; int page_tokens, T;    // cache rows [kv_rank + rot] storage type
 };
-// normed query latent -> cq; normed key / value latent and the rotated shared key part -> the cache row of (slot, position)
+// normed query latent -> cq (q_rank > 0); normed key / value latent and the rotated shared key part -> the cache row of (slot, position)
 void kr_sv_latent_prep(const KrSvLatent& a, bool f32, hipStream_t st);
 // q2 [T, heads, dim + rot] f32 (W_uq c_q): the plain part -> qn [T, heads, dim] storage type (to be folded into the latent space by a GEMM), the rotated
 // part, turned, -> qe [T, heads, kv_rank + rot] f32 at column kv_rank
 void kr_sv_latent_q(const KrSvLatent& a, const float* q2, void* qn, float* qe, bool f32, hipStream_t st);
+// q_rank 0: both of the above in one launch, the queries read from dz
+void kr_sv_latent_direct(const KrSvLatent& a, void* qn, float* qe, bool f32, hipStream_t st);
 // rows of a problem grouped by head over [T, heads, *] arrays: seg[h] = h * T, rows[h * T + t] = t * heads + h, group[h * T + t] = h
 void kr_sv_head_rows(int T, int heads, int* seg, int* rows, int* group, hipStream_t st);
 
@@ -226,6 +235,32 @@ struct KrSvSsdOut {
     void* out; int out_ld; int T;
 };
 void kr_sv_ssd_out(const KrSvSsdOut& a, bool f32, hipStream_t st);
+// ---- real-gated linear recurrence (kr_serve_rglru.hip).  Per channel c of block b (size = width / blocks):
+//   u_t = conv_b + sum_j conv[c][j] (x + x_b)(position(t) - taps + 1 + j),   r_t, i_t = sigmoid(G_r u_t + g_r), sigmoid(G_i u_t + g_i) over the block's u,
+//   log d = rate[c] r_t,   S_t = d S_(t-1) + sqrt(1 - d^2) i_t u_t,   out_t = S_t * gelu_tanh(y_t + y_b).
+// Everything is f32 but the stored gate matrices (and `out`): in a bf16 store u meets them as three bf16 terms that add up to it exactly.
+// State of a request slot: S [width] and the ring of the last rows x + x_b, [taps][width], position p at p % taps.
+struct KrSvRglru {
+    const float* y; const float* x; int ld;          // [T, ld] f32 each
+    const float* y_b; const float* x_b;              // [width]
+    const float* conv; const float* conv_b; int taps;   // [width, taps], [width]
+    const void* gw;                  // [blocks][2][size][size] storage type: G_r, then G_i of every block
+    const float* gb;                 // [2][width]
+    const float* rate;               // [width]
+    int width, blocks;
+    float* state; float* ring;       // [slots][width], [slots][taps][width]
+    const int* ent_off; const int* ent_slot; int n_entries;   // rows [ent_off[e], ent_off[e + 1]) belong to slot ent_slot[e]
+    const int* ent_chunk0; int n_chunks;                      // entry e owns the 64-token chunks [ent_chunk0[e], ent_chunk0[e + 1])
+    const int* pos; int T;
+    void* out; int out_ld;           // [T, out_ld] storage type
+    // portions: per token the product of the decays and the state since its chunk's start (from zero), the same of whole chunks, the state at a chunk's start
+    float2* ab; float2* agg; float* start;           // [T, width], [n_chunks, width], [n_chunks, width]
+};
+bool kr_sv_rglru_fits(int width, int blocks, int taps);
+// every entry brings one token: one launch
+void kr_sv_rglru_step(const KrSvRglru& a, bool f32, hipStream_t st);
+// portions of any length: chunk-local recurrences in parallel, a serial launch over the chunks, the outputs in parallel
+void kr_sv_rglru_portions(const KrSvRglru& a, bool f32, hipStream_t st);
 void kr_sv_argmax(const float* logits, int R, int vocab, int* out, hipStream_t st);
 // uniform values in [-amp, amp) from a counter hash of (seed, element); amp = 0 writes zeros
 void kr_sv_fill_uniform(void* p, bool f32, size_t n, uint64_t seed, float amp, hipStream_t st);

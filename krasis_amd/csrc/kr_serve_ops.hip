@@ -853,17 +853,18 @@ __global__ void sv_moe_scan_kernel(const int* __restrict__ counts, int E, int* _
     }
 }
 __global__ void sv_moe_fill_kernel(const int* __restrict__ ids, int n, int top, const int* __restrict__ seg, int* __restrict__ cursor, int* __restrict__ src_row,
-                                   int* __restrict__ row_group, int* __restrict__ pair_pos) {
+                                   int* __restrict__ row_group, int* __restrict__ pair_pos, const float* __restrict__ wts, float* __restrict__ row_w) {
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
     const int e = ids[i];
     const int pos = seg[e] + atomicAdd(&cursor[e], 1);
     src_row[pos] = i / top; row_group[pos] = e; pair_pos[i] = pos;
+    if (row_w) row_w[pos] = wts[i];
 }
 
 // the three launches above as one workgroup, for decode-sized batches (n pairs <= 1024, E counters in LDS)
 __global__ void __launch_bounds__(256) sv_moe_sort_small_kernel(const int* __restrict__ ids, int n, int top, int E, int* __restrict__ seg, int* __restrict__ src_row,
-                                                                int* __restrict__ row_group, int* __restrict__ pair_pos) {
+                                                                int* __restrict__ row_group, int* __restrict__ pair_pos, const float* __restrict__ wts, float* __restrict__ row_w) {
     extern __shared__ int cnt[];             // counts[E] | start[E]
     int* start = cnt + E;
     for (int e = threadIdx.x; e < E; e += 256) cnt[e] = 0;
@@ -880,15 +881,18 @@ __global__ void __launch_bounds__(256) sv_moe_sort_small_kernel(const int* __res
         const int e = ids[i];
         const int pos = start[e] + atomicAdd(&cnt[e], 1);
         src_row[pos] = i / top; row_group[pos] = e; pair_pos[i] = pos;
+        if (row_w) row_w[pos] = wts[i];
     }
 }
 
 template <typename T>
-__global__ void sv_act_kernel(const float* __restrict__ gu, int ld, T* __restrict__ y, int M, int F, int kind, float limit, float alpha) {
+__global__ void sv_act_kernel(const float* __restrict__ gu, int ld, T* __restrict__ y, int M, int F, int kind, float limit, float alpha,
+                              const float* __restrict__ row_w) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (size_t)M * F) return;
     const size_t r = i / F; const int c = (int)(i - r * F);
     float g = gu[r * ld + c], u = kind == KR_SV_ACT_RELU2 ? 0.0f : gu[r * ld + F + c], v;
+    if (row_w) { g *= row_w[r]; u *= row_w[r]; }
     if (kind == KR_SV_ACT_RELU2) {
         g = fmaxf(g, 0.0f); v = g * g;
     } else if (kind == KR_SV_ACT_GELU_TANH) {
@@ -925,7 +929,7 @@ __global__ void __launch_bounds__(NT) sv_residual_norm_kernel(const KrSvResidual
         }
     }
     const bool staged = rows && top <= 64;
-    if (staged && threadIdx.x < top) { pp_s[threadIdx.x] = a.pair_pos[t * top + threadIdx.x]; w_s[threadIdx.x] = a.wts[t * top + threadIdx.x]; }
+    if (staged && threadIdx.x < top) { pp_s[threadIdx.x] = a.pair_pos[t * top + threadIdx.x]; w_s[threadIdx.x] = a.wts ? a.wts[t * top + threadIdx.x] : 1.0f; }
     if (rows) __syncthreads();
     auto gate_at = [&](int c) {
         const float z = a.gate[t * a.ld_gate + c] + (a.gate_b ? a.gate_b[c] : 0.0f);
@@ -940,7 +944,7 @@ __global__ void __launch_bounds__(NT) sv_residual_norm_kernel(const KrSvResidual
 #pragma unroll 4
                 for (int s = 0; s < top; s++) ff = __builtin_fmaf(w_s[s], rows[(size_t)pp_s[s] * width + c], ff);
             } else {
-                for (int s = 0; s < top; s++) ff = __builtin_fmaf(a.wts[t * top + s], rows[(size_t)a.pair_pos[t * top + s] * width + c], ff);
+                for (int s = 0; s < top; s++) ff = __builtin_fmaf(a.wts ? a.wts[t * top + s] : 1.0f, rows[(size_t)a.pair_pos[t * top + s] * width + c], ff);
             }
             any = true;
         }
@@ -999,47 +1003,64 @@ __global__ void __launch_bounds__(NT) sv_residual_norm_kernel(const KrSvResidual
 }
 
 // ---- latent mixer
+// the rotated part of a key or query: thread `tid` of `nt` turns its pairs of z [rot] into dst
+template <typename T>
+__device__ __forceinline__ void sv_latent_turn(const float* z, const float2* cs, int rot, int interleaved, T* dst, int tid, int nt) {
+    const int half = rot / 2;
+    for (int i = tid; i < half; i += nt) {
+        const int i0 = interleaved ? 2 * i : i, i1 = interleaved ? 2 * i + 1 : i + half;
+        const float u = z[i0], v = z[i1];
+        const float2 c = cs[i];
+        sv_st(dst + i0, u * c.x - v * c.y); sv_st(dst + i1, v * c.x + u * c.y);
+    }
+}
+// dst = z / rms(z) * w over n elements, by a workgroup of 256
+template <typename T>
+__device__ __forceinline__ void sv_latent_rms(const float* z, const float* w, int n, float eps, T* dst, float* red) {
+    float q = 0.0f;
+    for (int c = threadIdx.x; c < n; c += 256) q = __builtin_fmaf(z[c], z[c], q);
+    const float inv = 1.0f / sqrtf(sv_block_sum<4>(q, red) / (float)n + eps);
+    for (int c = threadIdx.x; c < n; c += 256) sv_st(dst + c, z[c] * inv * w[c]);
+}
+// the cache row of token t: [normed latent | turned shared key part]
+template <typename T>
+__device__ __forceinline__ void sv_latent_kv_row(const KrSvLatent& a, int t, int off, float* red) {
+    const float* z = a.dz + (size_t)t * a.ld + off;
+    const int p = a.pos[t];
+    const size_t page = (size_t)a.page_table[(size_t)a.slot[t] * a.table_ld + p / a.page_tokens];
+    T* dst = (T*)a.pool + (page * a.page_tokens + (p % a.page_tokens)) * (size_t)(a.kv_rank + a.rot);
+    sv_latent_rms(z, a.dkv_norm_w, a.kv_rank, a.eps, dst, red);
+    sv_latent_turn(z + a.kv_rank, a.cs + (size_t)t * (a.rot / 2), a.rot, a.rot_interleaved, dst + a.kv_rank, threadIdx.x, 256);
+}
+// head h of token t, by one wave: the plain part in the storage type, the turned part into the latent-wide query
+template <typename T>
+__device__ __forceinline__ void sv_latent_q_head(const KrSvLatent& a, const float* q, int t, int h, T* qn, float* qe, int lane) {
+    T* n = qn + ((size_t)t * a.heads + h) * a.dim;
+    for (int d = lane; d < a.dim; d += 64) sv_st(n + d, q[d]);
+    sv_latent_turn(q + a.dim, a.cs + (size_t)t * (a.rot / 2), a.rot, a.rot_interleaved, qe + ((size_t)t * a.heads + h) * (a.kv_rank + a.rot) + a.kv_rank, lane, 64);
+}
 // one workgroup per (token, part): part 0 norms the query latent, part 1 norms the key / value latent into the cache row and turns the shared key part
 template <typename T>
 __global__ void __launch_bounds__(256) sv_latent_prep_kernel(const KrSvLatent a) {
     __shared__ float red[4];
-    const int t = blockIdx.x, part = blockIdx.y;
-    const float* z = a.dz + (size_t)t * a.ld + (part ? a.q_rank : 0);
-    const int n = part ? a.kv_rank : a.q_rank;
-    const float* w = part ? a.dkv_norm_w : a.dq_norm_w;
-    T* dst;
-    if (part) {
-        const int p = a.pos[t];
-        const size_t page = (size_t)a.page_table[(size_t)a.slot[t] * a.table_ld + p / a.page_tokens];
-        dst = (T*)a.pool + (page * a.page_tokens + (p % a.page_tokens)) * (size_t)(a.kv_rank + a.rot);
-    } else dst = (T*)a.cq + (size_t)t * a.q_rank;
-    float q = 0.0f;
-    for (int c = threadIdx.x; c < n; c += 256) q = __builtin_fmaf(z[c], z[c], q);
-    const float inv = 1.0f / sqrtf(sv_block_sum<4>(q, red) / (float)n + a.eps);
-    for (int c = threadIdx.x; c < n; c += 256) sv_st(dst + c, z[c] * inv * w[c]);
-    if (part) {
-        const float2* cs = a.cs + (size_t)t * (a.rot / 2);
-        for (int i = threadIdx.x; i < a.rot / 2; i += 256) {
-            const float u = z[n + 2 * i], v = z[n + 2 * i + 1];
-            const float2 c = cs[i];
-            sv_st(dst + n + 2 * i, u * c.x - v * c.y); sv_st(dst + n + 2 * i + 1, v * c.x + u * c.y);
-        }
-    }
+    const int t = blockIdx.x;
+    if (blockIdx.y) sv_latent_kv_row<T>(a, t, a.q_rank, red);
+    else sv_latent_rms(a.dz + (size_t)t * a.ld, a.dq_norm_w, a.q_rank, a.eps, (T*)a.cq + (size_t)t * a.q_rank, red);
 }
 // one wave per (token, head)
 template <typename T>
 __global__ void __launch_bounds__(64) sv_latent_q_kernel(const KrSvLatent a, const float* __restrict__ q2, T* __restrict__ qn, float* __restrict__ qe) {
-    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
-    const float* q = q2 + ((size_t)t * a.heads + h) * (a.dim + a.rot);
-    T* n = qn + ((size_t)t * a.heads + h) * a.dim;
-    for (int d = lane; d < a.dim; d += 64) sv_st(n + d, q[d]);
-    float* e = qe + ((size_t)t * a.heads + h) * (a.kv_rank + a.rot) + a.kv_rank;
-    const float2* cs = a.cs + (size_t)t * (a.rot / 2);
-    for (int i = lane; i < a.rot / 2; i += 64) {
-        const float u = q[a.dim + 2 * i], v = q[a.dim + 2 * i + 1];
-        const float2 c = cs[i];
-        e[2 * i] = u * c.x - v * c.y; e[2 * i + 1] = v * c.x + u * c.y;
-    }
+    const int t = blockIdx.x, h = blockIdx.y;
+    sv_latent_q_head(a, q2 + ((size_t)t * a.heads + h) * (a.dim + a.rot), t, h, qn, qe, threadIdx.x);
+}
+// queries without a latent of their own: parts 0 .. ceil(heads / 4) - 1 take four heads each, a wave per head; the last part (own_kv) writes the cache row
+template <typename T>
+__global__ void __launch_bounds__(256) sv_latent_direct_kernel(const KrSvLatent a, T* __restrict__ qn, float* __restrict__ qe) {
+    __shared__ float red[4];
+    const int t = blockIdx.x, n = a.heads * (a.dim + a.rot);
+    if ((int)blockIdx.y == (a.heads + 3) / 4) { sv_latent_kv_row<T>(a, t, n, red); return; }
+    const int h = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (h < a.heads) sv_latent_q_head(a, a.dz + (size_t)t * a.ld + (size_t)h * (a.dim + a.rot), t, h, qn, qe, threadIdx.x & 63);
 }
 __global__ void sv_head_rows_kernel(int T, int heads, int* __restrict__ seg, int* __restrict__ rows, int* __restrict__ group) {
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
@@ -1934,25 +1955,26 @@ void kr_sv_router_select(const float* z, int ld, int parts, const float* bias, i
     hipLaunchKernelGGL(sv_router_select_kernel, dim3(T), dim3(64), lds, st, z, ld, parts, bias, bias_mode, score_kind, group_kind, E, top, groups, keep, renorm, ids, wts);
 }
 
-void kr_sv_moe_sort(const int* ids, int T, int top, int E, int* counts, int* seg, int* cursor, int* src_row, int* row_group, int* pair_pos, hipStream_t st) {
+void kr_sv_moe_sort(const int* ids, int T, int top, int E, int* counts, int* seg, int* cursor, int* src_row, int* row_group, int* pair_pos, const float* wts, float* row_w,
+                    hipStream_t st) {
     const int n = T * top;
     if (n <= 0) return;
     if (n <= 1024 && E <= 4096) {
-        hipLaunchKernelGGL(sv_moe_sort_small_kernel, dim3(1), dim3(256), (size_t)2 * E * sizeof(int), st, ids, n, top, E, seg, src_row, row_group, pair_pos);
+        hipLaunchKernelGGL(sv_moe_sort_small_kernel, dim3(1), dim3(256), (size_t)2 * E * sizeof(int), st, ids, n, top, E, seg, src_row, row_group, pair_pos, wts, row_w);
         return;
     }
     hipLaunchKernelGGL(sv_fill_int_kernel, dim3((E + 255) / 256), dim3(256), 0, st, counts, E, 0);
     hipLaunchKernelGGL(sv_moe_count_kernel, dim3((n + 255) / 256), dim3(256), 0, st, ids, n, counts);
     hipLaunchKernelGGL(sv_moe_scan_kernel, dim3(1), dim3(64), 0, st, counts, E, seg, cursor);
-    hipLaunchKernelGGL(sv_moe_fill_kernel, dim3((n + 255) / 256), dim3(256), 0, st, ids, n, top, seg, cursor, src_row, row_group, pair_pos);
+    hipLaunchKernelGGL(sv_moe_fill_kernel, dim3((n + 255) / 256), dim3(256), 0, st, ids, n, top, seg, cursor, src_row, row_group, pair_pos, wts, row_w);
 }
 
-void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, hipStream_t st) {
+void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, const float* row_w, hipStream_t st) {
     const size_t n = (size_t)M * F;
     if (n == 0) return;
     const dim3 grid((unsigned)((n + 255) / 256));
-    if (f32) hipLaunchKernelGGL(sv_act_kernel<float>, grid, dim3(256), 0, st, gu, ld, (float*)y, M, F, kind, limit, alpha);
-    else hipLaunchKernelGGL(sv_act_kernel<uint16_t>, grid, dim3(256), 0, st, gu, ld, (uint16_t*)y, M, F, kind, limit, alpha);
+    if (f32) hipLaunchKernelGGL(sv_act_kernel<float>, grid, dim3(256), 0, st, gu, ld, (float*)y, M, F, kind, limit, alpha, row_w);
+    else hipLaunchKernelGGL(sv_act_kernel<uint16_t>, grid, dim3(256), 0, st, gu, ld, (uint16_t*)y, M, F, kind, limit, alpha, row_w);
 }
 
 void kr_sv_residual_norm(const KrSvResidual& r, bool out_f32, hipStream_t st) {
@@ -1974,6 +1996,12 @@ void kr_sv_latent_q(const KrSvLatent& a, const float* q2, void* qn, float* qe, b
     if (a.T <= 0) return;
     if (f32) hipLaunchKernelGGL(sv_latent_q_kernel<float>, dim3(a.T, a.heads), dim3(64), 0, st, a, q2, (float*)qn, qe);
     else hipLaunchKernelGGL(sv_latent_q_kernel<uint16_t>, dim3(a.T, a.heads), dim3(64), 0, st, a, q2, (uint16_t*)qn, qe);
+}
+void kr_sv_latent_direct(const KrSvLatent& a, void* qn, float* qe, bool f32, hipStream_t st) {
+    if (a.T <= 0) return;
+    const dim3 grid(a.T, (a.heads + 3) / 4 + (a.own_kv ? 1 : 0));
+    if (f32) hipLaunchKernelGGL(sv_latent_direct_kernel<float>, grid, dim3(256), 0, st, a, (float*)qn, qe);
+    else hipLaunchKernelGGL(sv_latent_direct_kernel<uint16_t>, grid, dim3(256), 0, st, a, (uint16_t*)qn, qe);
 }
 void kr_sv_head_rows(int T, int heads, int* seg, int* rows, int* group, hipStream_t st) {
     const int n = T * heads > heads + 1 ? T * heads : heads + 1;

@@ -468,6 +468,78 @@ def lufozen_fit_checkpoint(spec: ServeModelSpec, shape_of: Callable[[str], Tuple
 register_architecture("Lufozen", lufozen_spec)
 
 
+# ---- Ripupel: sequential layers with a weight-only layer norm before and after each sublayer, x <- x + n1b(mixer(n1(x))), x <- x + n2b(ff(n2(x))).  Two mixers.
+# 'rglru': a convolution branch u and a gated branch y; per channel S <- d S + sqrt(1 - d^2) i u with log d = -8 r softplus(lam), the gates r and i
+# block-diagonal in u; output from S * gelu(y).  'latent_attention': queries straight from the input, keys and values through a normed latent, a rotated key
+# part shared by the heads (half-split pairs), a learned sink, an element-wise sigmoid gate on the heads' outputs; a layer may attend to an earlier layer's
+# latents with projections of its own.  Feed-forward: SiLU-gated dense, or SiLU-gated experts behind a sigmoid router whose weight multiplies the expert's
+# INPUT, not renormalised.  The vocabulary projection is the embedding table.
+def _ripupel_tensors(spec: ServeModelSpec) -> Iterator[Tuple[int, str, int, str]]:
+    yield -1, "embed", 0, "embed"
+    yield -1, "final_norm_w", 0, "final.norm"
+    yield -1, "head", 0, "embed"
+    for i, l in enumerate(spec.layers):
+        p = f"l{i}"
+        yield i, "norm_w", 0, f"{p}.norm1"
+        yield i, "post1_w", 0, f"{p}.norm1b"
+        if l.mixer_kind == S.MIX_RGLRU:
+            for r, n in (("rg_y", "y"), ("rg_y_b", "y.b"), ("rg_x", "x"), ("rg_x_b", "x.b"), ("rg_conv", "conv"), ("rg_conv_b", "conv.b"), ("rg_ra", "ra"), ("rg_ra_b", "ra.b"),
+                         ("rg_ri", "ri"), ("rg_ri_b", "ri.b"), ("rg_lam", "lam"), ("o", "o")):
+                yield i, r, 0, f"{p}.mix.{n}"
+        else:
+            yield i, "q", 0, f"{p}.mix.q"
+            if l.kv_from < 0:
+                yield i, "dkv", 0, f"{p}.mix.dkv"
+                yield i, "dkv_norm", 0, f"{p}.mix.dkv.norm"
+            for r, n in (("uk", "uk"), ("uv", "uv"), ("sink", "sink"), ("out_gate", "g"), ("o", "o")):
+                yield i, r, 0, f"{p}.mix.{n}"
+        if l.mlp_kind != S.MLP_NONE:
+            yield i, "norm2_w", 0, f"{p}.norm2"
+            yield i, "post2_w", 0, f"{p}.norm2b"
+        if l.mlp_kind == S.MLP_DENSE:
+            for r in ("gate", "up", "down"):
+                yield i, r, 0, f"{p}.mlp.{r}"
+        elif l.mlp_kind == S.MLP_MOE:
+            yield i, "router", 0, f"{p}.mlp.router"
+            for e in range(l.experts):
+                for r in ("gate", "up", "down"):
+                    yield i, f"expert_{r}", e, f"{p}.mlp.e{e}.{r}"
+
+
+def ripupel_spec(cfg: dict) -> ServeModelSpec:
+    layers: List[S.LayerSpec] = []
+    for i, lc in enumerate(cfg["layers"]):
+        kind, m = lc.get("type"), lc["mixer"]
+        if kind == "rglru":
+            l = S.LayerSpec(heads=1, kv_heads=1, dim=1, vdim=1, mixer_kind=S.MIX_RGLRU, rg_width=int(m["width"]), rg_blocks=int(m["blocks"]), rg_conv=int(m.get("conv") or 1), rg_rate=8.0)
+        elif kind == "latent_attention":
+            rot = m.get("rot") or {}
+            if int(rot.get("dims", m["rot_dim"])) != int(m["rot_dim"]):
+                raise ValueError(f"layer {i}: the rotated part has {m['rot_dim']} coordinates, the rotation {rot['dims']}")
+            l = S.LayerSpec(heads=int(m["heads"]), kv_heads=1, dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), mixer_kind=S.MIX_LATENT, q_rank=0, kv_rank=int(m["kv_rank"]),
+                            rot_dims=int(m["rot_dim"]), rot_interleaved=0, rot_base=float(rot.get("base", 10000.0)), scale=float(m["scale"]), has_sink=S.SINK_TENSOR,
+                            out_gate=S.OGATE_ELEM_SIGMOID, kv_from=-1 if m.get("kv_from") is None else int(m["kv_from"]))
+        else:
+            raise ValueError(f"layer {i}: mixer type {kind!r} is not part of this design")
+        mlp = lc.get("mlp")
+        if mlp is not None:
+            if mlp.get("kind") == "dense":
+                l.mlp_kind, l.ff, l.dense_act = S.MLP_DENSE, int(mlp["ff"]), S.ACT_SILU
+            elif mlp.get("kind") == "moe":
+                r, ex = mlp["router"], mlp["expert"]
+                l.mlp_kind, l.experts, l.top, l.router_score, l.expert_in_weight = S.MLP_MOE, int(r["experts"]), int(r["top"]), S.RSCORE_SIGMOID, 1
+                l.expert_ff, l.expert_act = int(ex["ff"]), S.ACT_SILU
+            else:
+                raise ValueError(f"layer {i}: feed-forward kind {mlp.get('kind')!r}")
+        layers.append(l)
+    return ServeModelSpec(vocab=int(cfg["vocab"]), width=int(cfg["width"]), norm_kind=S.NORM_LAYER, norm_eps=float(cfg["norm"]["eps"]), layers=layers,
+                          tensors=_ripupel_tensors, block_kind=S.BLOCK_SEQUENTIAL, pre_norm=1, post_norm=1, norm_bias=0,
+                          embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
+
+
+register_architecture("Ripupel", ripupel_spec)
+
+
 def read_config(model_dir: str) -> dict:
     with open(os.path.join(model_dir, "config.json")) as f:
         return json.load(f)

@@ -17,7 +17,7 @@ NORM_LAYER, NORM_RMS = 0, 1
 MLP_NONE, MLP_DENSE, MLP_MOE = 0, 1, 2
 ACT_GELU_TANH, ACT_CLAMPED_SWIGLU, ACT_SILU, ACT_RELU2 = 0, 1, 2, 3
 BLOCK_PARALLEL, BLOCK_SEQUENTIAL = 0, 1
-MIX_ATTENTION, MIX_LATENT, MIX_RETENTION, MIX_MLSTM, MIX_GLA, MIX_SSD = 0, 1, 2, 3, 4, 5
+MIX_ATTENTION, MIX_LATENT, MIX_RETENTION, MIX_MLSTM, MIX_GLA, MIX_SSD, MIX_RGLRU = 0, 1, 2, 3, 4, 5, 6
 QKNORM_NONE, QKNORM_AFTER_ROT, QKNORM_WEIGHTED, QKNORM_WHOLE = 0, 1, 2, 3
 RBIAS_NONE, RBIAS_LOGIT, RBIAS_CHOICE = 0, 1, 2
 RSCORE_SOFTMAX, RSCORE_SIGMOID = 0, 1
@@ -34,7 +34,8 @@ ROLES = {n: i for i, n in enumerate(["embed", "final_norm_w", "final_norm_b", "h
                                      "q_bias", "k_bias", "o_bias", "out_gate", "canon", "res_gate1", "res_gate1_b", "res_gate2", "res_gate2_b",
                                      "lin_norm", "lin_decay", "igate", "igate_b", "fgate", "fgate_b",
                                      "embed_norm", "bigram", "pre_add", "v_bias", "q_conv", "k_conv", "v_conv", "decay_a1", "decay_a2", "decay_a2_b",
-                                     "ssd_in", "ssd_conv", "ssd_conv_b", "ssd_dt_bias", "ssd_a_log", "ssd_d", "ssd_norm", "ssd_o"])}
+                                     "ssd_in", "ssd_conv", "ssd_conv_b", "ssd_dt_bias", "ssd_a_log", "ssd_d", "ssd_norm", "ssd_o",
+                                     "rg_y", "rg_y_b", "rg_x", "rg_x_b", "rg_conv", "rg_conv_b", "rg_ra", "rg_ra_b", "rg_ri", "rg_ri_b", "rg_lam"])}
 
 
 @dataclass
@@ -102,6 +103,11 @@ class LayerSpec:
     ssd_norm_groups: int = 0
     mix_scale: float = 0.0               # weights of the two mixers' outputs (0 reads as 1)
     side_scale: float = 0.0
+    expert_in_weight: int = 0            # 1: the router's weight multiplies the expert's input instead of its output
+    rg_width: int = 0                    # real-gated linear recurrence: channels, equal parts of the block-diagonal gates, taps of its convolution, decay rate
+    rg_blocks: int = 0
+    rg_conv: int = 0
+    rg_rate: float = 0.0
 
 
 class ServeStore:
@@ -139,7 +145,7 @@ class ServeStore:
 
     # ---- weights
     def set_tensor(self, layer: int, role: str, array: np.ndarray, index: int = 0) -> None:
-        """array: uint16 (bf16 bit patterns) or float32, [rows, cols] or a vector"""
+        """array: uint16 (bf16 bit patterns) or float32, [rows, cols] or a vector; a stack of matrices counts as its matrices one below the other"""
         a = np.ascontiguousarray(array)
         if a.dtype == np.uint16:
             src = BF16
@@ -147,7 +153,7 @@ class ServeStore:
             src = F32
         else:
             raise ValueError(f"tensor dtype {a.dtype}: bf16 bit patterns (uint16) or float32")
-        rows, cols = (1, a.size) if a.ndim <= 1 else a.shape
+        rows, cols = (1, a.size) if a.ndim <= 1 else (a.size // a.shape[-1], a.shape[-1])
         check_serve(self._lib.kr_serve_set_tensor(self._h, layer, ROLES[role], index, a.ctypes.data, src, rows, cols))
 
     def fill_synthetic(self, seed: int = 1, amp: float = 1.0) -> None:
