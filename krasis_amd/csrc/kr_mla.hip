@@ -43,7 +43,9 @@ template <bool FP8> __device__ __forceinline__ float kr_stage_val(const unsigned
     _Float16 hv; __builtin_memcpy(&hv, row + 2 * i, 2);
     return (float)hv;
 }
+// v is rounded to f32 before it is rounded again: left alone, the compiler forms a product and its conversion in ONE instruction (v_fma_mixlo_f16, one rounding)
 template <bool FP8> __device__ __forceinline__ void kr_mla_st(void* base, size_t i, float v) {
+    asm volatile("" : "+v"(v));
     if (FP8) reinterpret_cast<uint8_t*>(base)[i] = kr_f32_to_e4m3(v);
     else reinterpret_cast<uint16_t*>(base)[i] = __half_as_ushort(__float2half_rn(v));
 }
