@@ -347,9 +347,9 @@ def parse():
                          "sizes -- prompt pass and decode throughput, kernel-family times -- beside the closest model of the decode graph (GQA + softmax top-k MoE, INT4) at "
                          "the same sizes; prints its own JSON line")
     ap.add_argument("--arch-sizes", default="small,large", help="sizes of --arch-compare (ARCH_SIZES)")
-    ap.add_argument("--arch-design", default="lomutar", choices=["lomutar", "pamulix", "midisun", "lufozen"],
+    ap.add_argument("--arch-design", default="lomutar", choices=["lomutar", "pamulix", "midisun", "lufozen", "ripupel"],
                     help="which layer-described design --arch-compare measures: lomutar (beside the decode graph's GQA + MoE model), pamulix or midisun (beside "
-                         "Lomutar), lufozen (beside Midisun with a dense feed-forward) -- both on the batched serving store, at the same layer sizes")
+                         "Lomutar), lufozen (beside Midisun with a dense feed-forward), ripupel (beside Pamulix's latent layers and Midisun's retention) -- both on the batched serving store, at the same layer sizes")
     return ap.parse_args()
 
 
@@ -780,6 +780,91 @@ def arch_compare_lufozen(args):
                                        "gemm_family_frac_of_hbm_peak": (byts - st_b) / (d["family_ms"][1] * 1e-3) / 1e9 / HBM_PEAK_GBS, "state_bytes_per_step": st_b}
             res["midisun_" + label] = r
             del eng; gc.collect()
+        out["sizes"][name] = res
+    flush_native_stdout()
+    print(json.dumps(out), flush=True)
+    return out
+
+
+def ripupel_serve_engine(z, kinds):
+    """A Ripupel model with random bf16 weights on the batched serving store at the layer sizes z (ARCH_SIZES); kinds: one letter per layer, G = gated linear
+    recurrence (as wide as the model, blocks of 256 channels, four taps), L = attention through latents (kv_rank 512 + 64 rotated, the size's heads with
+    128 plain dimensions), B = the same with the latents of the L layer before it.  Every layer: SiLU experts behind a sigmoid router whose weight multiplies the
+    expert's input, the size's expert counts."""
+    from krasis_amd import model_registry as R, scheduler as SCH, serve_store as S
+    W, H, D, E, k, F, V, P = (z[c] for c in ("width", "heads", "dim", "experts", "top", "ff", "vocab", "prompt"))
+    moe = dict(mlp_kind=S.MLP_MOE, experts=E, top=k, groups=1, keep=1, router_score=S.RSCORE_SIGMOID, expert_in_weight=1, expert_ff=F, expert_act=S.ACT_SILU)
+    layers, lender = [], -1
+    for i, kd in enumerate(kinds):
+        if kd == "G":
+            layers.append(S.LayerSpec(heads=1, kv_heads=1, dim=1, vdim=1, mixer_kind=S.MIX_RGLRU, rg_width=W, rg_blocks=W // 256, rg_conv=4, rg_rate=8.0, **moe))
+        else:
+            layers.append(S.LayerSpec(heads=H, kv_heads=1, dim=D, vdim=D, mixer_kind=S.MIX_LATENT, q_rank=0, kv_rank=512, rot_dims=64, rot_interleaved=0, rot_base=1e6,
+                                      scale=(D + 64) ** -0.5, has_sink=S.SINK_TENSOR, out_gate=S.OGATE_ELEM_SIGMOID, kv_from=lender if kd == "B" else -1, **moe))
+            lender = i if kd == "L" else lender
+    spec = R.ServeModelSpec(V, W, S.NORM_LAYER, 1e-5, layers, None, block_kind=S.BLOCK_SEQUENTIAL, pre_norm=1, post_norm=1, norm_bias=0, embed_scale=0.5)
+    eng = SCH.BatchEngine(spec, dtype="bfloat16", max_tokens=4 * (P + 256), max_slots=4)
+    eng.load_synthetic(seed=7, amp=1.0)
+    return eng
+
+
+def arch_compare_ripupel(args):
+    """The Ripupel design beside the two designs of the store that come closest, all with random bf16 weights and the same experts at the layer sizes of
+    ARCH_SIZES: Pamulix's latent layers (the same cache row of 512 + 64; its queries pass a latent of width * 3 / 8) for the attention, Midisun's retention
+    for the recurrence.  Three Ripupel models per size: the mixed order latent, recurrence, borrowed latents, recurrence, ... (the throughput), and one mixer
+    kind alone each (what its kernels reach).  The gated recurrence is priced against the HBM peak: its branches in (8 bytes per token and channel), its
+    output out (2 bytes) and the gates' matrices are what must move."""
+    import numpy as np
+    out = {"metric": "arch_compare_ripupel_vs_pamulix_and_midisun", "unit": "tok/s", "sizes": {}}
+    for name in [x for x in args.arch_sizes.split(",") if x]:
+        z = ARCH_SIZES[name]; W, H, G, D, E, k, F, L, V, P = (z[c] for c in ("width", "heads", "kv_heads", "dim", "experts", "top", "ff", "layers", "vocab", "prompt"))
+        Rk, Rr, Qr = 512, 64, W * 3 // 8
+        res = {"shape": dict(z, kv_rank=Rk, rot_dim=Rr, rg_width=W, rg_block=256)}
+        lat_flops = 2.0 * H * (2 * Rk + Rr) * sum(i + 1 for i in range(P))                 # per latent layer: keys 576 wide, values 512
+        rec_bytes = P * W * 10.0 + 2.0 * 2 * W * 256                                          # per recurrent layer and prompt
+        ret_flops = 4.0 * P * H * D * D
+        w_exp, w_moe = 3 * W * F, E * W                                                       # one expert; the router
+        w_kv = (Rk + Rr) * W
+        w_lat = H * (D + Rr) * W + H * D * W + H * D * Rk * 2 + W * H * D                     # q, gate, W_uk and W_uv, output (W_dkv apart)
+        w_plat = Qr * W + H * (D + Rr) * Qr + H * D * Rk * 2 + W * H * D + w_kv
+        w_rg = 3 * W * W + 2 * W * 256
+        w_ret = 5 * H * D * W + 2 * W * W                                                     # q, k, v, gate, output and the two residual gates
+
+        def price(eng, macs_mix, mix_bytes_gemm, kinds, batches, mixer):
+            m = serve_measure(eng, V, P, np.random.default_rng(3), decode_batches=batches)
+            fam = m["prefill_family_ms"]
+            macs = macs_mix + len(kinds) * (k * w_exp + w_moe)
+            r = {"prefill": {"tok_s": P / m["prefill_s"], "ms": m["prefill_s"] * 1e3, "tokens": P, "family_ms": {n: round(v, 3) for n, v in zip(SERVE_FAMILIES, fam)},
+                             "gemm_family_frac_of_bf16_peak": 2.0 * P * (macs + V * W / P) / (fam[1] * 1e-3) / 1e12 / F16_PEAK_TFLOPS}}
+            r["prefill"].update(mixer(fam[3]))
+            for B, d in m["decode"].items():
+                byts = 2.0 * (mix_bytes_gemm + len(kinds) * (min(E, B * k) * w_exp + w_moe) + V * W)
+                r["decode_b%d" % B] = {"tok_s": B / d["s_per_step"], "ms_per_step": d["s_per_step"] * 1e3, "weight_bytes_per_step": byts,
+                                       "frac_of_hbm_peak": byts / d["s_per_step"] / 1e9 / HBM_PEAK_GBS, "family_ms": {n: round(v, 4) for n, v in zip(SERVE_FAMILIES, d["family_ms"])},
+                                       "gemm_family_frac_of_hbm_peak": byts / (d["family_ms"][1] * 1e-3) / 1e9 / HBM_PEAK_GBS}
+            return r
+
+        def attention(n):
+            return lambda ms: {"attention_TFLOPs": n * lat_flops / (ms * 1e-3) / 1e12, "attention_frac_of_f32_matrix_peak": n * lat_flops / (ms * 1e-3) / 1e12 / F32_MATRIX_PEAK_TFLOPS}
+        order = "".join("LGBG"[i % 4] for i in range(L))
+        for label, kinds in (("mixed_" + order, order), ("latent_only", "L" * L), ("recurrence_only", "G" * L)):
+            eng = ripupel_serve_engine(z, kinds)
+            nG, nL = kinds.count("G"), len(kinds) - kinds.count("G")
+            mix_w = nG * w_rg + nL * w_lat + kinds.count("L") * w_kv
+            mixer = attention(nL) if not nG else (lambda ms: {"recurrence_bytes_GBs": nG * rec_bytes / (ms * 1e-3) / 1e9, "recurrence_frac_of_hbm_peak":
+                                                              nG * rec_bytes / (ms * 1e-3) / 1e9 / HBM_PEAK_GBS}) if not nL else (lambda ms: {})
+            res["ripupel_" + label] = price(eng, mix_w, mix_w, kinds, (1, 4) if nG and nL else (1,), mixer)
+            del eng; gc.collect()
+        eng = pamulix_serve_engine(z, "L" * L)
+        res["pamulix_latent_only"] = price(eng, L * w_plat, L * w_plat, "L" * L, (1, 4), attention(L))
+        del eng; gc.collect()
+        eng = midisun_serve_engine(z, "R" * L)
+        # the chunked retention moves q, k, v in and o out (f32) and the state of every 64-token block out, in and out again
+        ret_bytes = L * (P * 4.0 * 4 * H * D + P / 64.0 * 3 * 4 * H * D * D)
+        res["midisun_retention_only"] = price(eng, L * w_ret, L * w_ret, "R" * L, (1, 4), lambda ms: {
+            "retention_TFLOPs": L * ret_flops / (ms * 1e-3) / 1e12, "retention_frac_of_f32_matrix_peak": L * ret_flops / (ms * 1e-3) / 1e12 / F32_MATRIX_PEAK_TFLOPS,
+            "retention_bytes_GBs": ret_bytes / (ms * 1e-3) / 1e9, "retention_frac_of_hbm_peak": ret_bytes / (ms * 1e-3) / 1e9 / HBM_PEAK_GBS})
+        del eng; gc.collect()
         out["sizes"][name] = res
     flush_native_stdout()
     print(json.dumps(out), flush=True)
@@ -1744,7 +1829,7 @@ def main_multi(args, torch, dist, world, rank, local_rank):
 def main():
     args = parse()
     if args.arch_compare:
-        return {"pamulix": arch_compare_pamulix, "midisun": arch_compare_midisun, "lufozen": arch_compare_lufozen}.get(args.arch_design, arch_compare)(args)
+        return {"pamulix": arch_compare_pamulix, "midisun": arch_compare_midisun, "lufozen": arch_compare_lufozen, "ripupel": arch_compare_ripupel}.get(args.arch_design, arch_compare)(args)
     import torch
     import torch.distributed as dist
 
