@@ -1,6 +1,6 @@
 // kr_serve_rglru.hip -- the real-gated linear recurrence of the serving store (KrSvRglru, gfx950, wave64).
 //
-// Portions: a chunk is 64 tokens of one request.  sv_rglru_gate_kernel, a workgroup per (chunk, 64 channels of a block): the convolution feeds both gate
+// Portions: a chunk is 64 tokens of one request.  sv_rglru_gate_kernel, a workgroup per (chunk, 128 channels of a block): the convolution feeds both gate
 // products from LDS, the lane that holds a channel's gates of 16 tokens in its accumulators forms decay and input there and walks them, and four lanes
 // compose to the chunk: it leaves per token (product of the decays, state from zero) since the chunk's start.  sv_rglru_chain_kernel carries S over the
 // chunks, sv_rglru_out_kernel forms S of every token from its chunk's start, gates it and keeps the convolution's last rows.
@@ -20,13 +20,27 @@ typedef uint32_t rg_u2 __attribute__((ext_vector_type(2)));
 
 __device__ __forceinline__ float rg_ld(const float* p) { return *p; }
 __device__ __forceinline__ float rg_ld(const uint16_t* p) { return kr_bf16_to_f32(*p); }
-__device__ __forceinline__ float rg_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float rg_gelu(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
-// decay and input of one token and channel from the gates' logits: 1 - d^2 = -expm1(2 log d) keeps its digits when d is next to one
+// sigmoid on the hardware's exponential and reciprocal (one unit in the last place each)
+__device__ __forceinline__ float rg_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
+// tanh form of gelu: (1 + tanh w) / 2 = sigmoid(2 w)
+__device__ __forceinline__ float rg_gelu(float z) { return z * rg_sigmoid(2.0f * 0.7978845608028654f * (z + 0.044715f * z * z * z)); }
+// decay d = exp(x) and input sqrt(1 - d^2) i u of one token and channel from the gates' logits.  Near one d and 1 - d^2 both come from m = exp(x) - 1 as a
+// polynomial in x (terms to x^6: 5e-8 of m at x = -1/4), so neither loses digits; below, from the exponential itself
 __device__ __forceinline__ void rg_decay_input(float zr, float zi, float rate, float u, float& d, float& b) {
-    const float ld = rate * rg_sigmoid(zr);
-    d = expf(ld);
-    b = sqrtf(-expm1f(2.0f * ld)) * rg_sigmoid(zi) * u;
+    const float x = rate * rg_sigmoid(zr);
+    float p = __builtin_fmaf(x, 1.0f / 720.0f, 1.0f / 120.0f);
+    p = __builtin_fmaf(x, p, 1.0f / 24.0f); p = __builtin_fmaf(x, p, 1.0f / 6.0f); p = __builtin_fmaf(x, p, 0.5f);
+    const float m = __builtin_fmaf(x * x, p, x), e = __builtin_amdgcn_exp2f(1.4426950408889634f * x);
+    const bool near1 = x > -0.25f;
+    d = near1 ? 1.0f + m : e;
+    const float q = near1 ? -m * (2.0f + m) : __builtin_fmaf(-e, e, 1.0f);
+    b = __builtin_amdgcn_sqrtf(q) * rg_sigmoid(zi) * u;
+}
+// two floats as two bf16 (round to nearest even), the first in the low half
+__device__ __forceinline__ uint32_t rg_pack2(float lo, float hi) {
+    typedef __bf16 b2 __attribute__((ext_vector_type(2)));
+    b2 v; v[0] = (__bf16)lo; v[1] = (__bf16)hi;
+    return __builtin_bit_cast(uint32_t, v);
 }
 
 struct RgChunk { int e, t0, n, row0, p0, slot; };      // entry, first token, tokens, first row and first position of the entry's portion
@@ -49,21 +63,25 @@ __device__ __forceinline__ float rg_x(const KrSvRglru& a, const RgChunk& k, int 
     return p < 0 ? 0.0f : a.ring[((size_t)k.slot * a.taps + p % a.taps) * a.width + c];
 }
 
-#define RG_LDU 72      // LDS row of 64 bf16 (+ 8): 16-byte fragment reads stay aligned and consecutive rows start 4 banks apart
-#define RG_LDF 68      // the same of 64 floats
+#define RG_CH 128      // channels of a workgroup, and of a slab of the reduction
+#define RG_LDU 136     // LDS row of RG_CH bf16 (+ 8): 16-byte fragment reads stay aligned and consecutive rows start 4 banks apart
+#define RG_LDF 132     // the same of RG_CH floats
+// Token 16 a + 4 m + i of a chunk lies in LDS row 16 m + 4 a + i: product m's rows then are token 16 (r / 4) + 4 m + r % 4 for row r -- so that a lane's
+// accumulators are 16 consecutive tokens -- and its fragment reads are 16 consecutive LDS rows, which fall into distinct banks
+__device__ __forceinline__ int rg_row(int t) { return 16 * ((t >> 2) & 3) + 4 * (t >> 4) + (t & 3); }
 // TAPS: the convolution's taps when known, 0 = any number
 template <typename T, int TAPS>
-__global__ void __launch_bounds__(256) sv_rglru_gate_kernel(const KrSvRglru a) {
+__global__ void __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(sizeof(T) == 2 ? 4 : 2))) sv_rglru_gate_kernel(const KrSvRglru a) {
     constexpr bool BF = sizeof(T) == 2;
     constexpr int VEC = 16 / sizeof(T);
     // bf16 store: u as three bf16 terms (8 mantissa bits each: their sum is u); f32 store: u itself
     __shared__ __attribute__((aligned(16))) char lds[BF ? 3 * 64 * RG_LDU * 2 : 64 * RG_LDF * 4];
     uint16_t* up = (uint16_t*)lds; float* uf = (float*)lds;
-    const int size = a.width / a.blocks, nsl = (size + 63) / 64;
+    const int size = a.width / a.blocks, nsl = (size + RG_CH - 1) / RG_CH;
     const int b = blockIdx.y / nsl, ns = blockIdx.y % nsl;
     const RgChunk k = rg_chunk(a, blockIdx.x);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r15 = lane & 15, qd = lane >> 4;
-    const int cl = ns * 64 + wave * 16 + r15;                   // the lane's channel within the block
+    const int cl = ns * RG_CH + wave * 16 + r15;                // the lane's channel within the block
     const bool live = cl < size;
     const int c = b * size + min(cl, size - 1);
     const T* gw = (const T*)a.gw + (size_t)b * 2 * size * size;
@@ -74,17 +92,61 @@ __global__ void __launch_bounds__(256) sv_rglru_gate_kernel(const KrSvRglru a) {
     for (int g = 0; g < 2; g++)
 #pragma unroll
         for (int m = 0; m < 4; m++) acc[g][m] = rg_f4{0.0f, 0.0f, 0.0f, 0.0f};
-    // the 64-channel slabs of the block in turn, this workgroup's own channels last: their u stays in LDS for the recurrence
+    // the slabs of the block in turn, this workgroup's own channels last: their u stays in LDS for the recurrence
     for (int s = 1; s <= nsl; s++) {
-        const int k0 = (ns + s) % nsl * 64;
-        // ---- weights of this slab: 16-byte pieces in the order the products take them, requested before the convolution
-        constexpr int NP = BF ? 2 : 4;
+        const int k0 = (ns + s) % nsl * RG_CH;
+        // ---- u of the slab: a thread forms 8 consecutive tokens of two channels
+        const int kc = k0 + 2 * lane, j0 = wave * 8, cc = b * size + kc;
+        float u[8][2];
+#pragma unroll
+        for (int j = 0; j < 8; j++) u[j][0] = u[j][1] = 0.0f;
+        bool done = kc >= size;
+        if constexpr (TAPS > 0) {
+            if (!done && kc + 1 < size && k.t0 + j0 - (TAPS - 1) >= k.row0 && j0 + 8 <= k.n) {      // both channels exist and every row is one of this step's
+                const float* xp = a.x + (size_t)(k.t0 + j0 - (TAPS - 1)) * a.ld + cc;
+                float xs[7 + TAPS][2], wt[2][TAPS];
+#pragma unroll
+                for (int i = 0; i < 7 + TAPS; i++) __builtin_memcpy(xs[i], xp + (size_t)i * a.ld, 8);
+#pragma unroll
+                for (int q = 0; q < 2; q++) {
+                    const float xb = a.x_b[cc + q], cb = a.conv_b[cc + q];
+#pragma unroll
+                    for (int i = 0; i < TAPS; i++) wt[q][i] = a.conv[(size_t)(cc + q) * TAPS + i];
+#pragma unroll
+                    for (int i = 0; i < 7 + TAPS; i++) xs[i][q] += xb;
+#pragma unroll
+                    for (int j = 0; j < 8; j++) {
+                        float v = cb;
+#pragma unroll
+                        for (int i = 0; i < TAPS; i++) v = __builtin_fmaf(wt[q][i], xs[j + i][q], v);
+                        u[j][q] = v;
+                    }
+                }
+                done = true;
+            }
+        }
+        if (!done) {
+#pragma unroll
+            for (int q = 0; q < 2; q++) {
+                if (kc + q >= size) continue;
+                const float xb = a.x_b[cc + q], cb = a.conv_b[cc + q];
+#pragma unroll
+                for (int j = 0; j < 8; j++) u[j][q] = cb;
+                for (int i = 0; i < a.taps; i++) {
+                    const float wt = a.conv[(size_t)(cc + q) * a.taps + i];
+#pragma unroll
+                    for (int j = 0; j < 8; j++) u[j][q] = __builtin_fmaf(wt, rg_x(a, k, j0 + j - (a.taps - 1) + i, cc + q, xb), u[j][q]);
+                }
+            }
+        }
+        // ---- weights of the slab: 16-byte pieces in the order the products take them
+        constexpr int NP = BF ? 4 : 8;
         rg_u4 wv[2][NP];
 #pragma unroll
         for (int g = 0; g < 2; g++)
 #pragma unroll
             for (int q = 0; q < NP; q++) {
-                const int kk = k0 + (BF ? q * 32 + 8 * qd : 16 * qd + 4 * q);
+                const int kk = k0 + (BF ? q * 32 + 8 * qd : 32 * qd + 4 * q);
                 rg_u4 v = {0u, 0u, 0u, 0u};
                 if (vec) { if (kk < size) v = *reinterpret_cast<const rg_u4*>(wr[g] + kk); }
                 else {
@@ -96,79 +158,39 @@ __global__ void __launch_bounds__(256) sv_rglru_gate_kernel(const KrSvRglru a) {
                 }
                 wv[g][q] = v;
             }
-        // ---- u of the slab: a thread forms 16 consecutive tokens of one channel
-        float u[16];
-        {
-            const int kc = k0 + lane, j0 = wave * 16;
-            if (kc < size) {
-                const int cc = b * size + kc;
-                const float xb = a.x_b[cc], cb = a.conv_b[cc];
-                const float* w = a.conv + (size_t)cc * a.taps;
-                bool done = false;
-                if constexpr (TAPS > 0) {
-                    if (k.t0 + j0 - (TAPS - 1) >= k.row0 && j0 + 16 <= k.n) {      // every row is one of this step's
-                        const float* xp = a.x + (size_t)(k.t0 + j0 - (TAPS - 1)) * a.ld + cc;
-                        float xs[15 + TAPS], wt[TAPS];
-#pragma unroll
-                        for (int i = 0; i < 15 + TAPS; i++) xs[i] = xp[(size_t)i * a.ld] + xb;
-#pragma unroll
-                        for (int i = 0; i < TAPS; i++) wt[i] = w[i];
-#pragma unroll
-                        for (int j = 0; j < 16; j++) {
-                            float v = cb;
-#pragma unroll
-                            for (int i = 0; i < TAPS; i++) v = __builtin_fmaf(wt[i], xs[j + i], v);
-                            u[j] = v;
-                        }
-                        done = true;
-                    }
-                }
-                if (!done) {
-#pragma unroll
-                    for (int j = 0; j < 16; j++) u[j] = cb;
-                    for (int i = 0; i < a.taps; i++) {
-                        const float wt = w[i];
-#pragma unroll
-                        for (int j = 0; j < 16; j++) u[j] = __builtin_fmaf(wt, rg_x(a, k, j0 + j - (a.taps - 1) + i, cc, xb), u[j]);
-                    }
-                }
-            } else {
-#pragma unroll
-                for (int j = 0; j < 16; j++) u[j] = 0.0f;
-            }
-        }
         __syncthreads();                                        // the previous slab's products have read LDS
 #pragma unroll
-        for (int j = 0; j < 16; j++) {
-            const int t = wave * 16 + j;
+        for (int j = 0; j < 8; j++) {
+            const int t = rg_row(j0 + j);
             if constexpr (BF) {
-                const uint16_t hi = kr_f32_to_bf16(u[j]);
-                const float r1 = u[j] - kr_bf16_to_f32(hi);
-                const uint16_t mid = kr_f32_to_bf16(r1);
-                const uint16_t lo = kr_f32_to_bf16(r1 - kr_bf16_to_f32(mid));
-                up[t * RG_LDU + lane] = hi; up[(64 + t) * RG_LDU + lane] = mid; up[(128 + t) * RG_LDU + lane] = lo;
-            } else uf[t * RG_LDF + lane] = u[j];
+                float r0 = u[j][0], r1 = u[j][1];
+#pragma unroll
+                for (int pl = 0; pl < 3; pl++) {
+                    const uint32_t h = rg_pack2(r0, r1);
+                    *reinterpret_cast<uint32_t*>(&up[(pl * 64 + t) * RG_LDU + 2 * lane]) = h;
+                    r0 -= __uint_as_float(h << 16); r1 -= __uint_as_float(h & 0xFFFF0000u);
+                }
+            } else *reinterpret_cast<float2*>(&uf[t * RG_LDF + 2 * lane]) = make_float2(u[j][0], u[j][1]);
         }
         __syncthreads();
-        // ---- both gates' logits.  Row r of product m stands for token 16 (r / 4) + 4 m + r % 4, so that a lane's accumulators are 16 consecutive tokens
-        const int tr = 16 * (r15 >> 2) + (r15 & 3);
+        // ---- both gates' logits
         if constexpr (BF) {
 #pragma unroll
-            for (int q = 0; q < 2; q++)
+            for (int q = 0; q < 4; q++)
 #pragma unroll
                 for (int pl = 2; pl >= 0; pl--)                 // small terms first
 #pragma unroll
                     for (int m = 0; m < 4; m++) {
-                        const rg_b8 av = __builtin_bit_cast(rg_b8, *reinterpret_cast<const rg_u4*>(&up[(pl * 64 + tr + 4 * m) * RG_LDU + q * 32 + 8 * qd]));
+                        const rg_b8 av = __builtin_bit_cast(rg_b8, *reinterpret_cast<const rg_u4*>(&up[(pl * 64 + 16 * m + r15) * RG_LDU + q * 32 + 8 * qd]));
 #pragma unroll
                         for (int g = 0; g < 2; g++) acc[g][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, __builtin_bit_cast(rg_b8, wv[g][q]), acc[g][m], 0, 0, 0);
                     }
         } else {
 #pragma unroll
-            for (int q = 0; q < 4; q++)
+            for (int q = 0; q < 8; q++)
 #pragma unroll
                 for (int m = 0; m < 4; m++) {
-                    const float4 av = *reinterpret_cast<const float4*>(&uf[(tr + 4 * m) * RG_LDF + 16 * qd + 4 * q]);
+                    const float4 av = *reinterpret_cast<const float4*>(&uf[(16 * m + r15) * RG_LDF + 32 * qd + 4 * q]);
                     const float af[4] = {av.x, av.y, av.z, av.w};
 #pragma unroll
                     for (int i = 0; i < 4; i++)
@@ -182,12 +204,11 @@ __global__ void __launch_bounds__(256) sv_rglru_gate_kernel(const KrSvRglru a) {
     float A[16], H[16], ca = 1.0f, ch = 0.0f;
 #pragma unroll
     for (int j = 0; j < 16; j++) {
-        const int t = 16 * qd + j, ul = wave * 16 + r15;
-        float d = 1.0f, in = 0.0f;
-        if (t < k.n) {
-            const float u = BF ? kr_bf16_to_f32(up[t * RG_LDU + ul]) + (kr_bf16_to_f32(up[(64 + t) * RG_LDU + ul]) + kr_bf16_to_f32(up[(128 + t) * RG_LDU + ul])) : uf[t * RG_LDF + ul];
-            rg_decay_input(acc[0][j >> 2][j & 3] + br, acc[1][j >> 2][j & 3] + bi, rate, u, d, in);
-        }
+        const int t = 16 * qd + j, tr = rg_row(t), ul = wave * 16 + r15;
+        const float u = BF ? kr_bf16_to_f32(up[tr * RG_LDU + ul]) + (kr_bf16_to_f32(up[(64 + tr) * RG_LDU + ul]) + kr_bf16_to_f32(up[(128 + tr) * RG_LDU + ul])) : uf[tr * RG_LDF + ul];
+        float d, in;
+        rg_decay_input(acc[0][j >> 2][j & 3] + br, acc[1][j >> 2][j & 3] + bi, rate, u, d, in);
+        if (t >= k.n) { d = 1.0f; in = 0.0f; }                  // rows past the portion
         ca *= d; ch = __builtin_fmaf(d, ch, in);
         A[j] = ca; H[j] = ch;
     }
@@ -273,15 +294,15 @@ __global__ void __launch_bounds__(256) sv_rglru_out_kernel(const KrSvRglru a) {
     }
 }
 
-// One token per entry.  A workgroup per (MB entries, 16 channels of a block): u of the whole block in LDS, a wave multiplies it by both gates' rows of four
+// One token per entry.  A workgroup per (MB entries, 4 CN channels of a block): u of the whole block in LDS, a wave multiplies it by both gates' rows of CN
 // channels (lanes 0 .. 31 the first gate, 32 .. 63 the second), and the lanes that then hold a channel finish it.  The ring has one row more than the
 // convolution looks back, so the row a workgroup writes is none that another one still reads.
-template <typename T, int MB>
+template <typename T, int MB, int CN>
 __global__ void __launch_bounds__(256) sv_rglru_step_kernel(const KrSvRglru a) {
     extern __shared__ float us[];            // [MB][size]
-    constexpr int VEC = 16 / sizeof(T), CN = 4;
-    const int size = a.width / a.blocks, nsl = (size + 15) / 16, e0 = blockIdx.x * MB;
-    const int b = blockIdx.y / nsl, c0 = (blockIdx.y % nsl) * 16 + (threadIdx.x >> 6) * CN;
+    constexpr int VEC = 16 / sizeof(T);
+    const int size = a.width / a.blocks, nsl = (size + 4 * CN - 1) / (4 * CN), e0 = blockIdx.x * MB;
+    const int b = blockIdx.y / nsl, c0 = ((blockIdx.y % nsl) * 4 + (threadIdx.x >> 6)) * CN;
     const int tid = threadIdx.x, lane = tid & 63, g = lane >> 5, l32 = lane & 31;
     const T* gw = (const T*)a.gw + ((size_t)b * 2 + g) * size * size;
     const bool vec = size % VEC == 0 && (uintptr_t)a.gw % 16 == 0;
@@ -374,9 +395,12 @@ bool kr_sv_rglru_fits(int width, int blocks, int taps) {
 void kr_sv_rglru_step(const KrSvRglru& a, bool f32, hipStream_t st) {
     if (a.n_entries <= 0) return;
     const int size = a.width / a.blocks, mb = a.n_entries == 1 ? 1 : 4;
-    const dim3 grid((a.n_entries + mb - 1) / mb, a.blocks * ((size + 15) / 16));
+    // channels per wave: four when that still gives every compute unit two workgroups, else two
+    const int eg = (a.n_entries + mb - 1) / mb, cn = (long)eg * a.width / 16 >= 512 ? 4 : 2;
+    const dim3 grid(eg, a.blocks * ((size + 4 * cn - 1) / (4 * cn)));
     const size_t lds = (size_t)mb * size * sizeof(float);
-#define RG_S(T_, MB_) hipLaunchKernelGGL((sv_rglru_step_kernel<T_, MB_>), grid, dim3(256), lds, st, a)
+#define RG_S(T_, MB_) do { if (cn == 4) hipLaunchKernelGGL((sv_rglru_step_kernel<T_, MB_, 4>), grid, dim3(256), lds, st, a); \
+                           else hipLaunchKernelGGL((sv_rglru_step_kernel<T_, MB_, 2>), grid, dim3(256), lds, st, a); } while (0)
     if (f32) { if (mb == 1) RG_S(float, 1); else RG_S(float, 4); }
     else { if (mb == 1) RG_S(uint16_t, 1); else RG_S(uint16_t, 4); }
 #undef RG_S
@@ -385,8 +409,8 @@ void kr_sv_rglru_step(const KrSvRglru& a, bool f32, hipStream_t st) {
 void kr_sv_rglru_portions(const KrSvRglru& a, bool f32, hipStream_t st) {
     if (a.n_chunks <= 0) return;
     const int size = a.width / a.blocks;
-    const dim3 grid(a.n_chunks, a.blocks * ((size + 63) / 64));
-#define RG_G(T_, N_) hipLaunchKernelGGL((sv_rglru_gate_kernel<T_, N_>), grid, dim3(256), 0, st, a)
+    const dim3 grid(a.n_chunks, a.blocks * ((size + RG_CH - 1) / RG_CH));
+#define RG_G(T_, N_) hipLaunchKernelGGL((sv_rglru_gate_kernel<T_, N_>), grid, dim3(512), 0, st, a)
     if (f32) { if (a.taps == 4) RG_G(float, 4); else RG_G(float, 0); }
     else { if (a.taps == 4) RG_G(uint16_t, 4); else RG_G(uint16_t, 0); }
 #undef RG_G
