@@ -399,6 +399,10 @@ typedef struct {
      * bigram [bigram_buckets + 1, width]; a request's first token takes the last row.  The previous token is part of a request's state */
     int bigram_buckets, bigram_mul_prev, bigram_mul_cur;
     float logit_scale;          /* 0 or 1: the logits as they are; else logits * logit_scale */
+    int pos_rows;               /* > 0: a learned row per position joins the embedding row (tensor pos [pos_rows, width], unscaled); a request holds at most
+                                 * pos_rows positions.  Not together with the pair embedding */
+    int token_side;             /* > 0: every layer ends with x += mult * rms(W_proj (gelu_tanh(W_gate x) * e)) * w, e = the layer's token_side columns of the
+                                 * token's row in tensor side_embed [vocab, n_layers * token_side]; tensors side_gate, side_proj, side_norm.  RMS-normed designs only */
 } kr_serve_config;
 typedef struct {
     /* mixer: attention over the paged cache; the feed-forward follows it or runs beside it (kr_serve_config.block_kind) */
@@ -430,7 +434,8 @@ typedef struct {
     int v_mix;                         /* KR_SERVE_VMIX_*: values blended with the values an earlier layer formed for the same token, before they are cached */
     int router_bias;                   /* KR_SERVE_RBIAS_*: bias[expert] joins the logits before everything, or the scores for the choice only */
     /* ---- attention */
-    int proj_bias;                     /* 1: q, k and the output projection carry biases (tensors q_bias, k_bias, o_bias); 2: v too (v_bias) */
+    int proj_bias;                     /* 1: q, k and the output projection carry biases (tensors q_bias, k_bias, o_bias); 2: v too (v_bias); 3: q, k and v, the output
+                                        * projection does not */
     int v_from_k;                      /* the values are the keys as projected (with their bias, before any norm); no v projection; vdim == dim */
     float softcap;                     /* > 0: score <- softcap * tanh(score / softcap), after the scale, before the distance bias */
     int out_gate;                      /* KR_SERVE_OGATE_*: the mixer's output is gated by a projection of the mixer's input (tensor out_gate) before W_o */
@@ -467,7 +472,22 @@ typedef struct {
      * the current token's); in each of rg_blocks equal parts of u: r = sigmoid(A u + a), i = sigmoid(B u + b); log d = -rg_rate r softplus(lam),
      * S_t = d S_(t-1) + sqrt(1 - d^2) i u, per channel, f32; mixer output W_o (S * y).  S and the last rg_conv - 1 rows W_x h + b_x are a request's state. */
     int rg_width, rg_blocks, rg_conv; float rg_rate;
+    /* ---- attention, further */
+    int keep_first;                    /* with window: position i also sees the first keep_first positions of its request */
+    /* ---- feed-forward */
+    int ff_bias;                       /* 1: the dense feed-forward's three projections carry biases (tensors gate_b, up_b, down_b) */
+    /* ---- KR_SERVE_MIX_LIGHTNING, alone (mixer_kind) or beside an attention mixer on the same input (side_mixer): lt_heads heads, q = silu(W_q h), k = silu(W_k h)
+     * (lt_dim each), v = silu(W_v h) (lt_vdim); S_t = decay_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; the heads laid side by side rms-normed as one row, times a weight,
+     * times sigmoid(W_g h), then its own output projection.  Beside attention weighted by mix_scale / side_scale like the state-space mixer */
+    int lt_heads, lt_dim, lt_vdim;
 } kr_serve_layer;
+/* KR_SERVE_MIX_WKV: heads x dim (vdim == dim, kv_heads == heads).  Five inputs h + (h' - h) * mu_i, h' = the previous token's h (part of the state, zeros before position
+ * 0); r, k, v, g are projections (q, k, v, out_gate) of the first four, and the fifth forms a log decay per key channel, -exp(W_2 tanh(W_1 z) + w_0) (decay_a1
+ * [decay_rank, width], decay_a2, decay_a2_b).  o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t, S_t = diag(w_t) S_(t-1) + k_t v_t^T; o rms-normed per head, times a weight
+ * (lin_norm_weight 1), times silu(g).
+ * KR_SERVE_MIX_DELTA: kv_heads queries and keys of dim, heads values of vdim; q, k, v pass a convolution of proj_conv taps, then silu; q and k are unit vectors per head
+ * (x / sqrt(sum x^2 + 1e-6)), q times dim^(-1/2); b = sigmoid(W_b h), a = exp(-exp(A_log) softplus(W_a h + dt_bias)) per head (tensors delta_b, delta_a, ssd_a_log, ssd_dt_bias);
+ * S <- a S, u = b (v - S^T k), S <- S + k u^T, o = S^T q; o rms-normed per head, times a weight shared by the heads (lin_norm_weight 2), times silu(W_g h). */
 #define KR_SERVE_BLOCK_PARALLEL 0
 #define KR_SERVE_BLOCK_SEQUENTIAL 1
 #define KR_SERVE_MIX_ATTENTION 0
@@ -476,6 +496,9 @@ typedef struct {
 #define KR_SERVE_MIX_GLA 4             /* a decay per key channel, formed from the input through a low-rank projection (fields decay_*) */
 #define KR_SERVE_MIX_SSD 5             /* selective state space with one decay per head and token (fields ssd_*) */
 #define KR_SERVE_MIX_RGLRU 6           /* real-gated linear recurrence over channels between a convolution and a gated branch (fields rg_*) */
+#define KR_SERVE_MIX_WKV 7             /* token-shifted inputs, a decay per key channel, a bonus for the current token */
+#define KR_SERVE_MIX_DELTA 8           /* gated delta rule: the state is corrected towards the value at its key */
+#define KR_SERVE_MIX_LIGHTNING 9       /* linear attention with a fixed decay per head on silu'd q, k, v, one norm over all heads (fields lt_*) */
 #define KR_SERVE_MIX_MLSTM 3           /* exponential input gate and sigmoid forget gate in log space with a running maximum m (m_0 = 0), normaliser state n;
                                         * q scaled by dim^(-1/2); o = S^T q / (max(|n.q|, exp(-m)) + 1e-6); o / rms(o) per head, times a weight, times sigmoid(W_g h) */
 #define KR_SERVE_QKNORM_NONE 0
@@ -520,9 +543,12 @@ enum { KR_SV_EMBED = 0, KR_SV_FINAL_NORM_W, KR_SV_FINAL_NORM_B, KR_SV_HEAD, KR_S
        KR_SV_SSD_IN, KR_SV_SSD_CONV, KR_SV_SSD_CONV_B, KR_SV_SSD_DT_BIAS, KR_SV_SSD_A_LOG, KR_SV_SSD_D, KR_SV_SSD_NORM, KR_SV_SSD_O,
        KR_SV_RG_Y, KR_SV_RG_Y_B, KR_SV_RG_X, KR_SV_RG_X_B, KR_SV_RG_CONV, KR_SV_RG_CONV_B,
        KR_SV_RG_RA /* [rg_blocks * size, size] */, KR_SV_RG_RA_B /* [rg_blocks, size] */, KR_SV_RG_RI, KR_SV_RG_RI_B, KR_SV_RG_LAM,
+       KR_SV_POS, KR_SV_SIDE_EMBED /* layer = -1 */, KR_SV_SIDE_GATE, KR_SV_SIDE_PROJ, KR_SV_SIDE_NORM, KR_SV_GATE_B, KR_SV_UP_B, KR_SV_DOWN_B,
+       KR_SV_WKV_MU /* index 0 - 4: r, k, v, g, w */, KR_SV_WKV_U /* [heads, dim] */, KR_SV_DELTA_B, KR_SV_DELTA_A /* [heads, width] each */,
+       KR_SV_LT_Q, KR_SV_LT_K, KR_SV_LT_V, KR_SV_LT_G, KR_SV_LT_NORM /* [lt_heads * lt_vdim] */, KR_SV_LT_O, KR_SV_LT_DECAY /* [lt_heads] f32 */,
        KR_SV_N_ROLES };
 /* layout version of kr_serve_config / kr_serve_layer: a caller built against another one must not use the library */
-#define KR_SERVE_ABI 5
+#define KR_SERVE_ABI 6
 int kr_serve_abi(void);
 int kr_serve_create(int device_ordinal, const kr_serve_config* cfg, const kr_serve_layer* layers, kr_serve** out);
 void kr_serve_destroy(kr_serve* s);

@@ -51,7 +51,7 @@ class ServeConfigC(C.Structure):
                 ("block_kind", C.c_int), ("pre_norm", C.c_int), ("post_norm", C.c_int), ("norm_bias", C.c_int), ("residual_mult", C.c_float),
                 ("norm_groups", C.c_int), ("embed_scale", C.c_float), ("canon_taps", C.c_int), ("res_gate", C.c_int),
                 ("norm_weight_offset", C.c_float), ("embed_norm", C.c_int), ("bigram_buckets", C.c_int), ("bigram_mul_prev", C.c_int), ("bigram_mul_cur", C.c_int),
-                ("logit_scale", C.c_float)]
+                ("logit_scale", C.c_float), ("pos_rows", C.c_int), ("token_side", C.c_int)]
 
 
 class ServeLayerC(C.Structure):
@@ -67,10 +67,11 @@ class ServeLayerC(C.Structure):
                 ("weights_of", C.c_int), ("pre_add", C.c_int), ("proj_conv", C.c_int), ("decay_rank", C.c_int), ("decay_tau", C.c_float), ("side_mixer", C.c_int),
                 ("ssd_heads", C.c_int), ("ssd_vdim", C.c_int), ("ssd_state", C.c_int), ("ssd_groups", C.c_int), ("ssd_conv", C.c_int), ("ssd_norm_groups", C.c_int),
                 ("mix_scale", C.c_float), ("side_scale", C.c_float),
-                ("expert_in_weight", C.c_int), ("rg_width", C.c_int), ("rg_blocks", C.c_int), ("rg_conv", C.c_int), ("rg_rate", C.c_float)]
+                ("expert_in_weight", C.c_int), ("rg_width", C.c_int), ("rg_blocks", C.c_int), ("rg_conv", C.c_int), ("rg_rate", C.c_float),
+                ("keep_first", C.c_int), ("ff_bias", C.c_int), ("lt_heads", C.c_int), ("lt_dim", C.c_int), ("lt_vdim", C.c_int)]
 
 
-SERVE_ABI = 5      # layout version of the two structures above (KR_SERVE_ABI in include/krasis_hip.h)
+SERVE_ABI = 6      # layout version of the two structures above (KR_SERVE_ABI in include/krasis_hip.h)
 
 
 _lib = None

@@ -37,16 +37,37 @@ struct SvLayer {
     size_t ssd_state_stride = 0;
     // real-gated linear recurrence: branch biases, convolution taps and bias, both gates' block matrices and biases, -rate softplus(lam); per slot S and the convolution's ring
     DevBuf rg_yb, rg_xb, rg_conv, rg_convb, rg_w, rg_b, rg_rate, rg_state, rg_ring;
+    // wkv: the projections of the shifted inputs as one grouped matrix [r | k | v | g, heads * dim rows each | the decay's first projection], shift weights [5, width], bonus;
+    // the previous token's input row of every slot.  Gated delta: the ring of projected rows, taps of them per slot
+    DevBuf wk, mu, bonus, shift_state, delta_ring;
+    // biases of hw's rows (the feed-forward's; zero elsewhere) and of the down projection; the per-layer token input; lightning attention: decays, norm weight, per-slot state
+    DevBuf h_bias, down_b, side_gate, side_proj, side_norm, lt_decay, lt_norm, lt_state;
+    size_t lt_state_stride = 0;
+    char have_mu[5] = {0, 0, 0, 0, 0};
     int wsrc = 0;                // the layer whose tensors this one uses (itself, or d.weights_of - 1); cache pools and state are always the layer's own
     // row blocks of hw: mixer [q | k | v | out gate | i | f | state-space in-projection], or the recurrence's branches [y | x] (n_qkv rows in all), then [router | gate | up | residual gate of the feed-forward]
-    int rope_id = 0, n_qkv = 0, off_ogate = 0, off_if = 0, off_ssd = 0, off_router = 0, n_router = 0, off_gu = 0, n_gu = 0, off_rg2 = 0, n_h = 0;
+    int rope_id = 0, n_qkv = 0, off_ogate = 0, off_if = 0, off_ba = 0, off_ssd = 0, off_lt = 0, off_router = 0, n_router = 0, off_gu = 0, n_gu = 0, off_rg2 = 0, n_h = 0;
     bool latent() const { return d.mixer_kind == KR_SERVE_MIX_LATENT; }
     bool gla() const { return d.mixer_kind == KR_SERVE_MIX_GLA; }
-    bool recurrent() const { return d.mixer_kind == KR_SERVE_MIX_RETENTION || d.mixer_kind == KR_SERVE_MIX_MLSTM || gla(); }
+    bool wkv() const { return d.mixer_kind == KR_SERVE_MIX_WKV; }
+    bool delta() const { return d.mixer_kind == KR_SERVE_MIX_DELTA; }
+    bool recurrent() const { return d.mixer_kind == KR_SERVE_MIX_RETENTION || d.mixer_kind == KR_SERVE_MIX_MLSTM || gla() || wkv() || delta(); }
     bool chunkable() const { return d.mixer_kind == KR_SERVE_MIX_RETENTION || d.mixer_kind == KR_SERVE_MIX_MLSTM; }      // the block form of the recurrence
     bool ssd_alone() const { return d.mixer_kind == KR_SERVE_MIX_SSD; }
     bool rglru() const { return d.mixer_kind == KR_SERVE_MIX_RGLRU; }
-    bool no_heads() const { return ssd_alone() || rglru(); }       // neither attention nor a matrix state per head
+    bool lt_alone() const { return d.mixer_kind == KR_SERVE_MIX_LIGHTNING; }
+    bool has_lt() const { return lt_alone() || d.side_mixer == KR_SERVE_MIX_LIGHTNING; }
+    int lt_inner() const { return d.lt_heads * d.lt_vdim; }
+    int lt_cols() const { return 2 * d.lt_heads * d.lt_dim + lt_inner(); }      // q | k | v
+    bool side_alone() const { return ssd_alone() || lt_alone(); }
+    bool has_side() const { return has_ssd() || has_lt(); }
+    int side_inner() const { return has_ssd() ? ssd_inner() : has_lt() ? lt_inner() : 0; }
+    bool no_heads() const { return side_alone() || rglru(); }       // neither attention nor a matrix state per head of the layer's own description
+    int q_rows() const { return (delta() ? d.kv_heads : d.heads) * d.dim; }
+    int k_rows() const { return d.kv_heads * d.dim; }
+    int v_rows() const { return (delta() ? d.heads : d.kv_heads) * d.vdim; }
+    int wk_rows() const { return 4 * d.heads * d.dim + d.decay_rank; }
+    int decay_out_rows() const { return (d.decay_rank + d.heads * d.dim - 1) / (d.heads * d.dim); }      // rows of heads * dim floats that hold the decay's low-rank vector
     bool lat_direct() const { return latent() && d.q_rank == 0; }
     int lat_q_rows() const { return d.q_rank ? d.q_rank : d.heads * (d.dim + d.rot_dims); }      // first row block of a latent mixer
     int lat_kv_rows() const { return d.kv_from < 0 ? d.kv_rank + d.rot_dims : 0; }
@@ -54,9 +75,9 @@ struct SvLayer {
     int ssd_inner() const { return d.ssd_heads * d.ssd_vdim; }
     int ssd_conv_c() const { return ssd_inner() + 2 * d.ssd_groups * d.ssd_state; }
     int ssd_in_rows() const { return 2 * ssd_inner() + 2 * d.ssd_groups * d.ssd_state + d.ssd_heads; }
-    int att_out_cols() const { return ssd_alone() ? 0 : rglru() ? d.rg_width : d.heads * d.vdim; }                   // the output projection reads [first mixer | state-space mixer]
-    int o_cols() const { return att_out_cols() + (has_ssd() ? ssd_inner() : 0); }
-    int pconv_c() const { return d.heads * d.dim + d.kv_heads * (d.dim + d.vdim); }
+    int att_out_cols() const { return side_alone() ? 0 : rglru() ? d.rg_width : d.heads * d.vdim; }                   // the output projection reads [first mixer | state-space mixer]
+    int o_cols() const { return att_out_cols() + side_inner(); }
+    int pconv_c() const { return q_rows() + k_rows() + v_rows(); }
     bool ungated_ff() const { return d.dense_act == KR_SERVE_ACT_RELU2; }
     bool has_cache() const { return !recurrent() && !no_heads() && d.kv_from < 0; }
     int att_heads_kv() const { return latent() ? 1 : d.kv_heads; }
@@ -78,8 +99,8 @@ struct kr_serve {
     hipStream_t st = nullptr;
     std::vector<SvLayer> L;
     std::vector<SvRope> ropes;
-    DevBuf embed, head, fnorm_w, fnorm_b, enorm_w, bigram;
-    bool have_embed = false, have_head = false, have_fw = false, have_fb = false, have_enorm = false, have_bigram = false;
+    DevBuf embed, head, fnorm_w, fnorm_b, enorm_w, bigram, pos, side_embed;
+    bool have_embed = false, have_head = false, have_fw = false, have_fb = false, have_enorm = false, have_bigram = false, have_pos = false, have_side = false;
     // cache
     int n_pages = 0;
     std::vector<int> free_pages;
@@ -94,6 +115,7 @@ struct kr_serve {
     DevBuf ssd_z;                                         // the state-space mixer's rows in the block recurrence's layout [q | k | v] per head (prompt portions)
     DevBuf rg_ab, rg_agg, rg_start;                       // real-gated linear recurrence, portions: per token and per chunk of 64
     DevBuf qkv2, sconv, ga1, gz;                          // convolved q | k | v; convolved x | B | C; the gla decay's low-rank input (storage type) and logits
+    DevBuf mixes, sgate;                                 // wkv: the shifted inputs [5][T][width]; the token input's gate logits
     DevBuf v_first;                                      // [T, kv_heads * vdim] f32: the values of the first value-mixing layer
     DevBuf lq_c, lq_2, lq_n, lq_e, att2, head_i;         // latent mixer: query latent, W_uq output, plain query parts, folded queries, per-head values, head row tables
     void* h_meta = nullptr; size_t h_meta_bytes = 0;     // pinned staging of the per-step arrays
@@ -176,7 +198,13 @@ int upload_norm_w(kr_serve* s, DevBuf& dst, const void* host, int src_dtype, siz
 int check_layer(const kr_serve_config& c, const kr_serve_layer* all, int i) {
     const kr_serve_layer& d = all[i];
     const bool ssd1 = d.mixer_kind == KR_SERVE_MIX_SSD, ssd = ssd1 || d.side_mixer == KR_SERVE_MIX_SSD;
-    if (d.side_mixer != 0 && d.side_mixer != KR_SERVE_MIX_SSD) return kr_fail(KR_ERR_VALUE, "layer %d: side mixer %d", i, d.side_mixer);
+    const bool lt1 = d.mixer_kind == KR_SERVE_MIX_LIGHTNING, lt = lt1 || d.side_mixer == KR_SERVE_MIX_LIGHTNING;
+    if (lt && (d.lt_heads < 1 || d.lt_dim < 1 || d.lt_dim > 512 || d.lt_vdim < 1 || d.lt_vdim > 512)) return kr_fail(KR_ERR_VALUE, "layer %d: lightning sizes (heads %d, %d / %d)", i, d.lt_heads, d.lt_dim, d.lt_vdim);
+    if (!lt && (d.lt_heads || d.lt_dim || d.lt_vdim)) return kr_fail(KR_ERR_VALUE, "layer %d: lt_* fields belong to lightning attention", i);
+    if (d.ff_bias && d.mlp_kind != KR_SERVE_MLP_DENSE) return kr_fail(KR_ERR_VALUE, "layer %d: biases belong to a dense feed-forward", i);
+    if (d.keep_first < 0 || (d.keep_first && d.mixer_kind != KR_SERVE_MIX_ATTENTION && d.mixer_kind != KR_SERVE_MIX_LATENT)) return kr_fail(KR_ERR_VALUE, "layer %d: keep_first %d", i, d.keep_first);
+    if (d.keep_first && d.chunk) return kr_fail(KR_ERR_VALUE, "layer %d: kept first tokens stand beside a window, not a chunk", i);
+    if (d.side_mixer != 0 && d.side_mixer != KR_SERVE_MIX_SSD && d.side_mixer != KR_SERVE_MIX_LIGHTNING) return kr_fail(KR_ERR_VALUE, "layer %d: side mixer %d", i, d.side_mixer);
     if (d.side_mixer && d.mixer_kind != KR_SERVE_MIX_ATTENTION) return kr_fail(KR_ERR_VALUE, "layer %d: a side mixer stands beside an attention mixer", i);
     if (ssd) {
         if (d.ssd_heads < 1 || d.ssd_vdim < 1 || d.ssd_vdim > 512 || d.ssd_state < 1 || d.ssd_state > 512 || d.ssd_groups < 1 || d.ssd_heads % d.ssd_groups || d.ssd_conv < 1 || d.ssd_conv > 64 ||
@@ -200,7 +228,7 @@ int check_layer(const kr_serve_config& c, const kr_serve_layer* all, int i) {
     if (rg && (!kr_sv_rglru_fits(d.rg_width, d.rg_blocks, d.rg_conv) || !(d.rg_rate > 0.0f)))
         return kr_fail(KR_ERR_VALUE, "layer %d: recurrence sizes (width %d, blocks %d, taps %d, rate %g)", i, d.rg_width, d.rg_blocks, d.rg_conv, (double)d.rg_rate);
     if (!rg && (d.rg_width || d.rg_blocks || d.rg_conv || d.rg_rate != 0.0f)) return kr_fail(KR_ERR_VALUE, "layer %d: rg_* fields belong to the gated linear recurrence", i);
-    if (ssd1 || rg) {
+    if (ssd1 || lt1 || rg) {
         if (d.kv_from >= 0 || d.v_mix || d.qk_unit_norm || d.window || d.chunk || d.has_sink || d.dist_bias || d.proj_bias || d.v_from_k || d.out_gate || d.softcap != 0.0f || d.rot_dims ||
             d.proj_conv || d.gate_cap != 0.0f || d.lin_norm_weight)
             return kr_fail(KR_ERR_VALUE, "layer %d: an attention-only mechanism is switched on for a mixer without heads", i);
@@ -208,15 +236,19 @@ int check_layer(const kr_serve_config& c, const kr_serve_layer* all, int i) {
     if (d.heads < 1 || d.kv_heads < 1 || d.heads % d.kv_heads) return kr_fail(KR_ERR_VALUE, "layer %d: heads %d / kv_heads %d", i, d.heads, d.kv_heads);
     if (d.dim < 1 || d.vdim < 1 || d.vdim > 512 || d.dim > 512) return kr_fail(KR_ERR_VALUE, "layer %d: head sizes %d / %d (at most 512)", i, d.dim, d.vdim);
     const bool lat = d.mixer_kind == KR_SERVE_MIX_LATENT;
-    const bool rec = d.mixer_kind == KR_SERVE_MIX_RETENTION || d.mixer_kind == KR_SERVE_MIX_MLSTM || d.mixer_kind == KR_SERVE_MIX_GLA;
+    const bool wkv = d.mixer_kind == KR_SERVE_MIX_WKV, delta = d.mixer_kind == KR_SERVE_MIX_DELTA;
+    const bool rec = d.mixer_kind == KR_SERVE_MIX_RETENTION || d.mixer_kind == KR_SERVE_MIX_MLSTM || d.mixer_kind == KR_SERVE_MIX_GLA || wkv || delta;
+    if (wkv && (d.vdim != d.dim || d.decay_rank < 1 || d.lin_norm_weight != 1 || !c.pre_norm || c.canon_taps > 1 || d.pre_add || d.weights_of))
+        return kr_fail(KR_ERR_VALUE, "layer %d: wkv needs vdim == dim, decay_rank, a norm weight per channel and a plain pre-normed input", i);
+    if (delta && (d.lin_norm_weight != 2 || d.proj_conv < 1)) return kr_fail(KR_ERR_VALUE, "layer %d: the delta rule needs a convolution on q, k, v and a norm weight shared by the heads", i);
     if (d.mixer_kind != KR_SERVE_MIX_ATTENTION && !lat && !rec) return kr_fail(KR_ERR_VALUE, "layer %d: mixer kind %d", i, d.mixer_kind);
     if (d.mixer_kind == KR_SERVE_MIX_GLA && (d.decay_rank < 1 || !(d.decay_tau > 0.0f) || d.lin_norm_weight != 2)) return kr_fail(KR_ERR_VALUE, "layer %d: gla needs decay_rank, decay_tau and a shared norm weight", i);
-    if (d.mixer_kind != KR_SERVE_MIX_GLA && (d.decay_rank || d.decay_tau != 0.0f)) return kr_fail(KR_ERR_VALUE, "layer %d: decay_rank / decay_tau belong to the gla mixer", i);
-    if (d.proj_conv < 0 || d.proj_conv > 64 || (d.proj_conv && (d.mixer_kind != KR_SERVE_MIX_ATTENTION || d.kv_from >= 0 || d.v_from_k || d.v_mix || d.qk_unit_norm == KR_SERVE_QKNORM_WHOLE)))
+    if ((d.mixer_kind != KR_SERVE_MIX_GLA && !wkv && d.decay_rank) || (d.mixer_kind != KR_SERVE_MIX_GLA && d.decay_tau != 0.0f)) return kr_fail(KR_ERR_VALUE, "layer %d: decay_rank / decay_tau belong to the gla mixer", i);
+    if (d.proj_conv < 0 || d.proj_conv > 64 || (d.proj_conv && !delta && (d.mixer_kind != KR_SERVE_MIX_ATTENTION || d.kv_from >= 0 || d.v_from_k || d.v_mix || d.qk_unit_norm == KR_SERVE_QKNORM_WHOLE)))
         return kr_fail(KR_ERR_VALUE, "layer %d: the convolution on q / k / v needs an attention mixer with projections and a cache of its own, per-head norms, no value mixing", i);
-    if (d.proj_bias < 0 || d.proj_bias > 2 || (d.proj_bias == 2 && (d.v_from_k || d.kv_from >= 0))) return kr_fail(KR_ERR_VALUE, "layer %d: projection biases %d", i, d.proj_bias);
+    if (d.proj_bias < 0 || d.proj_bias > 3 || (d.proj_bias >= 2 && (d.v_from_k || d.kv_from >= 0))) return kr_fail(KR_ERR_VALUE, "layer %d: projection biases %d", i, d.proj_bias);
     if (rec) {
-        if (d.kv_heads != d.heads) return kr_fail(KR_ERR_VALUE, "layer %d: a recurrent mixer has one key / value head per query head", i);
+        if (!delta && d.kv_heads != d.heads) return kr_fail(KR_ERR_VALUE, "layer %d: a recurrent mixer has one key / value head per query head", i);
         if (d.kv_from >= 0 || d.v_mix || d.qk_unit_norm || d.window || d.chunk || d.has_sink || d.dist_bias || d.proj_bias || d.v_from_k || d.out_gate || d.softcap != 0.0f)
             return kr_fail(KR_ERR_VALUE, "layer %d: an attention-only mechanism is switched on for a recurrent mixer", i);
         if (d.rot_dims && (d.rot_interleaved || d.mixer_kind != KR_SERVE_MIX_RETENTION)) return kr_fail(KR_ERR_VALUE, "layer %d: recurrent mixers rotate half-split pairs, retention only", i);
@@ -298,6 +330,8 @@ int kr_serve_create(int device_ordinal, const kr_serve_config* cfg, const kr_ser
     if ((cfg->canon_taps || cfg->res_gate) && !(cfg->block_kind == KR_SERVE_BLOCK_SEQUENTIAL && cfg->pre_norm && !cfg->post_norm))
         return kr_fail(KR_ERR_VALUE, "input convolution / gated residual need a sequential pre-normed block without output norms");
     if (cfg->embed_norm && !cfg->pre_norm) return kr_fail(KR_ERR_VALUE, "a normed embedding needs pre-normed blocks");
+    if (cfg->pos_rows < 0 || (cfg->pos_rows && cfg->bigram_buckets)) return kr_fail(KR_ERR_VALUE, "position rows %d (one second table joins the embedding)", cfg->pos_rows);
+    if (cfg->token_side < 0 || (cfg->token_side && (cfg->norm_kind != KR_SERVE_NORM_RMS || cfg->norm_groups > 1))) return kr_fail(KR_ERR_VALUE, "per-layer token input of %d needs plain RMS norms", cfg->token_side);
     if (cfg->bigram_buckets < 0) return kr_fail(KR_ERR_VALUE, "bigram buckets %d", cfg->bigram_buckets);
     for (int i = 0; i < cfg->n_layers; i++) { const int rc = check_layer(*cfg, layers, i); if (rc) return rc; }
     int n_dev = 0;
@@ -317,13 +351,17 @@ int kr_serve_create(int device_ordinal, const kr_serve_config* cfg, const kr_ser
         const kr_serve_layer& d = l.d;
         l.have.assign(KR_SV_N_ROLES, 0);
         l.wsrc = d.weights_of ? d.weights_of - 1 : i;
-        l.n_qkv = l.ssd_alone() ? 0 : l.rglru() ? 2 * d.rg_width : l.latent() ? l.lat_q_rows() + l.lat_kv_rows() : d.heads * d.dim + (d.kv_from < 0 ? d.kv_heads * (d.dim + (d.v_from_k ? 0 : d.vdim)) : 0);
+        l.n_qkv = (l.side_alone() || l.wkv()) ? 0 : l.delta() ? l.pconv_c() : l.rglru() ? 2 * d.rg_width : l.latent() ? l.lat_q_rows() + l.lat_kv_rows() : d.heads * d.dim + (d.kv_from < 0 ? d.kv_heads * (d.dim + (d.v_from_k ? 0 : d.vdim)) : 0);
         l.off_ogate = l.n_qkv;
-        if (l.recurrent()) l.n_qkv += d.heads * d.vdim; else if (d.out_gate == KR_SERVE_OGATE_HEAD_SIGMOID) l.n_qkv += d.heads; else if (d.out_gate) l.n_qkv += d.heads * d.vdim;
+        if (l.wkv()) {} else if (l.recurrent()) l.n_qkv += d.heads * d.vdim; else if (d.out_gate == KR_SERVE_OGATE_HEAD_SIGMOID) l.n_qkv += d.heads; else if (d.out_gate) l.n_qkv += d.heads * d.vdim;
         l.off_if = l.n_qkv;
         if (d.mixer_kind == KR_SERVE_MIX_MLSTM) l.n_qkv += 2 * d.heads;
+        l.off_ba = l.n_qkv;
+        if (l.delta()) l.n_qkv += 2 * d.heads;
         l.off_ssd = l.n_qkv;
         if (l.has_ssd()) l.n_qkv += l.ssd_in_rows();
+        l.off_lt = l.n_qkv;
+        if (l.has_lt()) l.n_qkv += l.lt_cols() + l.lt_inner();
         l.n_router = d.mlp_kind == KR_SERVE_MLP_MOE ? d.experts * (s->f32 ? 1 : 2) : 0;
         l.n_gu = d.mlp_kind == KR_SERVE_MLP_DENSE ? (l.ungated_ff() ? 1 : 2) * d.ff : (d.mlp_kind == KR_SERVE_MLP_MOE ? 2 * d.shared_ff : 0);
         l.off_router = l.n_qkv; l.off_gu = l.off_router + l.n_router; l.off_rg2 = l.off_gu + l.n_gu;
@@ -380,7 +418,24 @@ int kr_serve_create(int device_ordinal, const kr_serve_config* cfg, const kr_ser
             const size_t b = (size_t)cfg->max_slots * (cfg->canon_taps - 1) * cfg->width * 4;
             if (l.canon_state.ensure(b) || hipMemset(l.canon_state.p, 0, b) != hipSuccess) { kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "input convolution state"); }
         }
-        if (d.proj_conv > 1) {
+        if (l.wkv()) {
+            const size_t b = (size_t)cfg->max_slots * cfg->width * 4;
+            if (l.shift_state.ensure(b) || hipMemset(l.shift_state.p, 0, b) != hipSuccess) { kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "token shift state"); }
+        }
+        if (l.delta()) {
+            const size_t b = (size_t)cfg->max_slots * d.proj_conv * l.pconv_c() * 4;
+            if (l.delta_ring.ensure(b) || hipMemset(l.delta_ring.p, 0, b) != hipSuccess) { kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "convolution state"); }
+        }
+        if (d.ff_bias && !d.weights_of) {
+            const size_t b = (size_t)l.n_h * 4;
+            if (l.h_bias.ensure(b) || hipMemset(l.h_bias.p, 0, b) != hipSuccess) { kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "feed-forward biases"); }
+        }
+        if (l.has_lt()) {
+            l.lt_state_stride = (size_t)d.lt_heads * d.lt_vdim * d.lt_dim;
+            const size_t b = l.lt_state_stride * cfg->max_slots * 4;
+            if (l.lt_state.ensure(b) || hipMemset(l.lt_state.p, 0, b) != hipSuccess) { kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "lightning state of %zu bytes", b); }
+        }
+        if (d.proj_conv > 1 && !l.delta()) {
             const size_t b = (size_t)cfg->max_slots * (d.proj_conv - 1) * l.pconv_c() * 4;
             if (l.pconv_state.ensure(b) || hipMemset(l.pconv_state.p, 0, b) != hipSuccess) { kr_serve_destroy(s); return kr_fail(KR_ERR_HIP, "projection convolution state"); }
         }
@@ -447,13 +502,17 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
             SHAPE(1, W); s->have_enorm = true; return upload_norm_w(s, s->enorm_w, host, src_dtype, n);
         case KR_SV_BIGRAM: if (s->c.bigram_buckets < 1) return kr_fail(KR_ERR_VALUE, "the design has no pair embedding");
             SHAPE(s->c.bigram_buckets + 1, W); s->have_bigram = true; return upload(s, s->bigram, n, 0, host, src_dtype, n, false);
+        case KR_SV_POS: if (s->c.pos_rows < 1) return kr_fail(KR_ERR_VALUE, "the design has no position rows");
+            SHAPE(s->c.pos_rows, W); s->have_pos = true; return upload(s, s->pos, n, 0, host, src_dtype, n, false);
+        case KR_SV_SIDE_EMBED: if (s->c.token_side < 1) return kr_fail(KR_ERR_VALUE, "the design has no per-layer token input");
+            SHAPE(V, s->c.n_layers * s->c.token_side); s->have_side = true; return upload(s, s->side_embed, n, 0, host, src_dtype, n, false);
         case KR_SV_FINAL_NORM_B: SHAPE(1, W); s->have_fb = true; return upload(s, s->fnorm_b, n, 0, host, src_dtype, n, true);
         default: return kr_fail(KR_ERR_VALUE, "role %d is not a model-level tensor", role);
         }
     }
     if (layer >= s->c.n_layers) return kr_fail(KR_ERR_VALUE, "layer %d of %d", layer, s->c.n_layers);
     SvLayer& l = s->L[layer]; const kr_serve_layer& d = l.d;
-    const int nq = d.heads * d.dim, nk = d.kv_heads * d.dim, nv = d.kv_heads * d.vdim;
+    const int nq = l.q_rows(), nk = l.k_rows(), nv = l.v_rows();
     if (role < 0 || role >= KR_SV_N_ROLES) return kr_fail(KR_ERR_VALUE, "role %d", role);
     const bool moe = d.mlp_kind == KR_SERVE_MLP_MOE;
     const bool lat = l.latent();
@@ -463,20 +522,26 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     int rc = KR_OK;
     if (l.wsrc != layer && role != KR_SV_PRE_ADD) return kr_fail(KR_ERR_VALUE, "layer %d uses the tensors of layer %d", layer, l.wsrc);
     const int inner = l.ssd_inner(), sgn = d.ssd_groups * d.ssd_state;
-    if (role >= KR_SV_SSD_IN && role <= KR_SV_SSD_O && !l.has_ssd()) return kr_fail(KR_ERR_VALUE, "layer %d has no state-space mixer", layer);
-    if (role >= KR_SV_DECAY_A1 && role <= KR_SV_DECAY_A2_B && !l.gla()) return kr_fail(KR_ERR_VALUE, "layer %d has no gla mixer", layer);
+    if (role >= KR_SV_SSD_IN && role <= KR_SV_SSD_O && !l.has_ssd() && !(l.delta() && (role == KR_SV_SSD_DT_BIAS || role == KR_SV_SSD_A_LOG))) return kr_fail(KR_ERR_VALUE, "layer %d has no state-space mixer", layer);
+    if (role >= KR_SV_DECAY_A1 && role <= KR_SV_DECAY_A2_B && !l.gla() && !l.wkv()) return kr_fail(KR_ERR_VALUE, "layer %d has no gla mixer", layer);
     if (lat && !d.q_rank && (role == KR_SV_DQ || role == KR_SV_DQ_NORM || role == KR_SV_UQ)) return kr_fail(KR_ERR_VALUE, "layer %d projects its queries without a latent", layer);
     if (lat && d.kv_from >= 0 && (role == KR_SV_DKV || role == KR_SV_DKV_NORM)) return kr_fail(KR_ERR_VALUE, "layer %d borrows its latents", layer);
     if ((role >= KR_SV_RG_Y && role <= KR_SV_RG_LAM) != l.rglru() && ((role >= KR_SV_RG_Y && role <= KR_SV_RG_LAM) || role == KR_SV_Q || role == KR_SV_K || role == KR_SV_V))
         return kr_fail(KR_ERR_VALUE, "layer %d: role %d does not fit its mixer", layer, role);
     const int rgs = l.rglru() ? d.rg_width / d.rg_blocks : 0;
-    if (l.ssd_alone() && (role == KR_SV_Q || role == KR_SV_K || role == KR_SV_V || role == KR_SV_O)) return kr_fail(KR_ERR_VALUE, "layer %d has a state-space mixer only", layer);
+    if (role >= KR_SV_LT_Q && role <= KR_SV_LT_DECAY && !l.has_lt()) return kr_fail(KR_ERR_VALUE, "layer %d has no lightning attention", layer);
+    if ((role == KR_SV_WKV_MU || role == KR_SV_WKV_U) && !l.wkv()) return kr_fail(KR_ERR_VALUE, "layer %d has no wkv mixer", layer);
+    if ((role == KR_SV_DELTA_B || role == KR_SV_DELTA_A) && !l.delta()) return kr_fail(KR_ERR_VALUE, "layer %d has no delta rule", layer);
+    if (role >= KR_SV_SIDE_GATE && role <= KR_SV_SIDE_NORM && s->c.token_side < 1) return kr_fail(KR_ERR_VALUE, "the design has no per-layer token input");
+    if (role >= KR_SV_GATE_B && role <= KR_SV_DOWN_B && !d.ff_bias) return kr_fail(KR_ERR_VALUE, "layer %d: its feed-forward has no biases", layer);
+    const int ltq = d.lt_heads * d.lt_dim, lti = l.lt_inner();
+    if (l.side_alone() && (role == KR_SV_Q || role == KR_SV_K || role == KR_SV_V || role == KR_SV_O)) return kr_fail(KR_ERR_VALUE, "layer %d has no attention beside its mixer", layer);
     switch (role) {
     case KR_SV_PRE_ADD:
         if (!d.pre_add) return kr_fail(KR_ERR_VALUE, "layer %d takes no vector before it", layer);
         SHAPE(1, W); rc = upload(s, l.pre_add, n, 0, host, src_dtype, n, true); break;
     case KR_SV_V_BIAS:
-        if (d.proj_bias != 2) return kr_fail(KR_ERR_VALUE, "layer %d has no value bias", layer);
+        if (d.proj_bias < 2) return kr_fail(KR_ERR_VALUE, "layer %d has no value bias", layer);
         SHAPE(1, nv);
         rc = upload(s, l.v_bias, n, 0, host, src_dtype, n, true);
         if (!rc && d.proj_conv) rc = upload(s, l.pconv_bias, l.pconv_c(), (size_t)nq + nk, host, src_dtype, n, true);
@@ -485,14 +550,35 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
         if (!d.proj_conv) return kr_fail(KR_ERR_VALUE, "layer %d has no convolution on its projections", layer);
         SHAPE(role == KR_SV_Q_CONV ? nq : role == KR_SV_K_CONV ? nk : nv, d.proj_conv);
         rc = upload(s, l.pconv_w, (size_t)l.pconv_c() * d.proj_conv, (size_t)(role == KR_SV_Q_CONV ? 0 : role == KR_SV_K_CONV ? nq : nq + nk) * d.proj_conv, host, src_dtype, n, true); break;
-    case KR_SV_DECAY_A1: SHAPE(d.decay_rank, W); rc = upload(s, l.a1, n, 0, host, src_dtype, n, false); break;
+    case KR_SV_WKV_MU:
+        if (index < 0 || index > 4) return kr_fail(KR_ERR_VALUE, "shifted input %d of 5", index);
+        SHAPE(1, W); rc = upload(s, l.mu, (size_t)5 * W, (size_t)index * W, host, src_dtype, n, true); l.have_mu[index] = 1; break;
+    case KR_SV_WKV_U: SHAPE(d.heads, d.dim); rc = upload(s, l.bonus, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_DELTA_B: case KR_SV_DELTA_A:
+        SHAPE(d.heads, W); rc = upload(s, l.hw, (size_t)l.n_h * W, ((size_t)l.off_ba + (role == KR_SV_DELTA_A ? d.heads : 0)) * W, host, src_dtype, n, false); break;
+    case KR_SV_LT_Q: case KR_SV_LT_K: case KR_SV_LT_V: case KR_SV_LT_G:
+        SHAPE(role == KR_SV_LT_Q || role == KR_SV_LT_K ? ltq : lti, W);
+        rc = upload(s, l.hw, (size_t)l.n_h * W, ((size_t)l.off_lt + (role == KR_SV_LT_Q ? 0 : role == KR_SV_LT_K ? ltq : role == KR_SV_LT_V ? 2 * ltq : 2 * ltq + lti)) * W, host, src_dtype, n, false); break;
+    case KR_SV_LT_NORM: SHAPE(1, lti); rc = upload(s, l.lt_norm, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_LT_DECAY: SHAPE(1, d.lt_heads); rc = upload(s, l.lt_decay, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_LT_O: SHAPE(W, lti); rc = upload_cols(s, l.o, W, l.o_cols(), l.att_out_cols(), host, src_dtype, lti); break;
+    case KR_SV_SIDE_GATE: SHAPE(s->c.token_side, W); rc = upload(s, l.side_gate, n, 0, host, src_dtype, n, false); break;
+    case KR_SV_SIDE_PROJ: SHAPE(W, s->c.token_side); rc = upload(s, l.side_proj, n, 0, host, src_dtype, n, false); break;
+    case KR_SV_SIDE_NORM: SHAPE(1, W); rc = upload(s, l.side_norm, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_GATE_B: case KR_SV_UP_B:
+        if (role == KR_SV_GATE_B && l.ungated_ff()) return kr_fail(KR_ERR_VALUE, "layer %d: an un-gated feed-forward", layer);
+        SHAPE(1, d.ff); rc = upload(s, l.h_bias, l.n_h, (size_t)l.off_gu + ((role == KR_SV_UP_B && !l.ungated_ff()) ? d.ff : 0), host, src_dtype, n, true); break;
+    case KR_SV_DOWN_B: SHAPE(1, W); rc = upload(s, l.down_b, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_DECAY_A1:
+        if (l.wkv()) { SHAPE(d.decay_rank, W); rc = upload(s, l.wk, (size_t)l.wk_rows() * W, (size_t)4 * nq * W, host, src_dtype, n, false); break; }
+        SHAPE(d.decay_rank, W); rc = upload(s, l.a1, n, 0, host, src_dtype, n, false); break;
     case KR_SV_DECAY_A2: SHAPE(nq, d.decay_rank); rc = upload(s, l.a2, n, 0, host, src_dtype, n, false); break;
     case KR_SV_DECAY_A2_B: SHAPE(1, nq); rc = upload(s, l.a2_b, n, 0, host, src_dtype, n, true); break;
     case KR_SV_SSD_IN: SHAPE(l.ssd_in_rows(), W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)l.off_ssd * W, host, src_dtype, n, false); break;
     case KR_SV_SSD_CONV: SHAPE(inner + 2 * sgn, d.ssd_conv); rc = upload(s, l.sconv_w, n, 0, host, src_dtype, n, true); break;
     case KR_SV_SSD_CONV_B: SHAPE(1, inner + 2 * sgn); rc = upload(s, l.sconv_b, n, 0, host, src_dtype, n, true); break;
-    case KR_SV_SSD_DT_BIAS: SHAPE(1, d.ssd_heads); rc = upload(s, l.dt_bias, n, 0, host, src_dtype, n, true); break;
-    case KR_SV_SSD_A_LOG: SHAPE(1, d.ssd_heads); rc = upload(s, l.a_log, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_SSD_DT_BIAS: SHAPE(1, l.delta() ? d.heads : d.ssd_heads); rc = upload(s, l.dt_bias, n, 0, host, src_dtype, n, true); break;
+    case KR_SV_SSD_A_LOG: SHAPE(1, l.delta() ? d.heads : d.ssd_heads); rc = upload(s, l.a_log, n, 0, host, src_dtype, n, true); break;
     case KR_SV_SSD_D: SHAPE(1, d.ssd_heads); rc = upload(s, l.ssd_d, n, 0, host, src_dtype, n, true); break;
     case KR_SV_SSD_NORM: SHAPE(1, inner); rc = upload(s, l.ssd_norm, n, 0, host, src_dtype, n, true); break;
     case KR_SV_SSD_O: SHAPE(W, inner); rc = upload_cols(s, l.o, W, l.o_cols(), l.att_out_cols(), host, src_dtype, inner); break;
@@ -518,13 +604,14 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
         rc = upload(s, l.rg_rate, n, 0, r.data(), KR_SERVE_F32, n, true); break;
     }
     case KR_SV_Q_BIAS: case KR_SV_K_BIAS: case KR_SV_O_BIAS:
-        if (!d.proj_bias) return kr_fail(KR_ERR_VALUE, "layer %d has no projection biases", layer);
+        if (!d.proj_bias || (role == KR_SV_O_BIAS && d.proj_bias == 3)) return kr_fail(KR_ERR_VALUE, "layer %d has no projection biases", layer);
         SHAPE(1, role == KR_SV_Q_BIAS ? nq : role == KR_SV_K_BIAS ? nk : W);
         rc = upload(s, role == KR_SV_Q_BIAS ? l.q_bias : role == KR_SV_K_BIAS ? l.k_bias : l.o_bias, n, 0, host, src_dtype, n, true);
         if (!rc && d.proj_conv && role != KR_SV_O_BIAS) rc = upload(s, l.pconv_bias, l.pconv_c(), role == KR_SV_Q_BIAS ? 0 : (size_t)nq, host, src_dtype, n, true);
         break;
     case KR_SV_OUT_GATE:
         if (!rec && !d.out_gate) return kr_fail(KR_ERR_VALUE, "layer %d has no output gate", layer);
+        if (l.wkv()) { SHAPE(nq, W); rc = upload(s, l.wk, (size_t)l.wk_rows() * W, (size_t)3 * nq * W, host, src_dtype, n, false); break; }
         SHAPE((rec || d.out_gate == KR_SERVE_OGATE_ELEM_SIGMOID) ? d.heads * d.vdim : d.heads, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)l.off_ogate * W, host, src_dtype, n, false); break;
     case KR_SV_IGATE: case KR_SV_FGATE:
         if (d.mixer_kind != KR_SERVE_MIX_MLSTM) return kr_fail(KR_ERR_VALUE, "layer %d has no input / forget gates", layer);
@@ -582,13 +669,17 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     }
     case KR_SV_NORM_W: SHAPE(1, W); rc = upload_norm_w(s, l.norm_w, host, src_dtype, n); break;
     case KR_SV_NORM_B: SHAPE(1, W); rc = upload(s, l.norm_b, n, 0, host, src_dtype, n, true); break;
-    case KR_SV_Q: SHAPE(lat ? l.lat_q_rows() : nq, W); rc = upload(s, l.hw, (size_t)l.n_h * W, 0, host, src_dtype, n, false); break;
-    case KR_SV_K: if (d.kv_from >= 0) return kr_fail(KR_ERR_VALUE, "layer %d borrows its keys", layer);
-        SHAPE(nk, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)nq * W, host, src_dtype, n, false); break;
-    case KR_SV_V: if (d.kv_from >= 0 || d.v_from_k) return kr_fail(KR_ERR_VALUE, "layer %d has no value projection", layer);
+    case KR_SV_Q: case KR_SV_K: case KR_SV_V:
+        if (l.wkv()) { SHAPE(nq, W); rc = upload(s, l.wk, (size_t)l.wk_rows() * W, (size_t)(role == KR_SV_Q ? 0 : role == KR_SV_K ? 1 : 2) * nq * W, host, src_dtype, n, false); break; }
+        if (role == KR_SV_Q) { SHAPE(lat ? l.lat_q_rows() : nq, W); rc = upload(s, l.hw, (size_t)l.n_h * W, 0, host, src_dtype, n, false); break; }
+        if (role == KR_SV_K) {
+            if (d.kv_from >= 0) return kr_fail(KR_ERR_VALUE, "layer %d borrows its keys", layer);
+            SHAPE(nk, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)nq * W, host, src_dtype, n, false); break;
+        }
+        if (d.kv_from >= 0 || d.v_from_k) return kr_fail(KR_ERR_VALUE, "layer %d has no value projection", layer);
         SHAPE(nv, W); rc = upload(s, l.hw, (size_t)l.n_h * W, (size_t)(nq + nk) * W, host, src_dtype, n, false); break;
     case KR_SV_O: SHAPE(W, l.att_out_cols());
-        if (l.has_ssd()) rc = upload_cols(s, l.o, W, l.o_cols(), 0, host, src_dtype, l.att_out_cols());
+        if (l.has_side()) rc = upload_cols(s, l.o, W, l.o_cols(), 0, host, src_dtype, l.att_out_cols());
         else rc = upload(s, l.o, n, 0, host, src_dtype, n, false);
         break;
     case KR_SV_SINK: if (d.has_sink != KR_SERVE_SINK_TENSOR) return kr_fail(KR_ERR_VALUE, "layer %d has no sink tensor", layer);
@@ -656,6 +747,8 @@ int kr_serve_fill_synthetic(kr_serve* s, uint64_t seed, float amp) {
     s->have_embed = s->have_head = s->have_fw = s->have_fb = true;
     if (s->c.embed_norm) { bad |= vec(s->enorm_w, W, true); s->have_enorm = true; }
     if (s->c.bigram_buckets > 0) { bad |= mat(s->bigram, (size_t)(s->c.bigram_buckets + 1) * W, 1); s->have_bigram = true; }
+    if (s->c.pos_rows > 0) { bad |= mat(s->pos, (size_t)s->c.pos_rows * W, 1); s->have_pos = true; }
+    if (s->c.token_side > 0) { bad |= mat(s->side_embed, (size_t)V * s->c.n_layers * s->c.token_side, 1); s->have_side = true; }
     // a vector of n f32 values uniform in +-amp_v around mid
     auto vecu = [&](DevBuf& b, size_t n, float mid, float amp_v) -> int {
         if (vec(b, n, false)) return 1;
@@ -673,12 +766,27 @@ int kr_serve_fill_synthetic(kr_serve* s, uint64_t seed, float amp) {
         const kr_serve_layer& d = l.d;
         if (d.pre_add) bad |= vecu(l.pre_add, W, 0.0f, 0.1f);
         if (l.wsrc != (int)(&l - s->L.data())) { std::fill(l.have.begin(), l.have.end(), 1); continue; }      // the tensors are another layer's
-        bad |= mat(l.hw, (size_t)l.n_h * W, W) | mat(l.o, (size_t)W * l.o_cols(), l.o_cols());
-        if (d.proj_bias == 2) bad |= vec(l.v_bias, (size_t)d.kv_heads * d.vdim, false);
+        if (l.n_h > 0) bad |= mat(l.hw, (size_t)l.n_h * W, W);
+        bad |= mat(l.o, (size_t)W * l.o_cols(), l.o_cols());
+        if (d.proj_bias >= 2) bad |= vec(l.v_bias, (size_t)d.kv_heads * d.vdim, false);
         if (d.proj_conv) {           // taps of about 1 / taps: the convolved projection stays at the projection's scale
             bad |= vecu(l.pconv_w, (size_t)l.pconv_c() * d.proj_conv, 1.0f / (float)d.proj_conv, 0.5f / (float)d.proj_conv);
         }
         if (l.gla()) bad |= mat(l.a1, (size_t)d.decay_rank * W, W) | mat(l.a2, (size_t)d.heads * d.dim * d.decay_rank, d.decay_rank) | vecu(l.a2_b, (size_t)d.heads * d.dim, 3.0f, 1.0f);
+        if (l.wkv()) {               // log decays around -exp(-2): a memory of a few to a few dozen tokens
+            bad |= mat(l.wk, (size_t)l.wk_rows() * W, W) | mat(l.a2, (size_t)d.heads * d.dim * d.decay_rank, d.decay_rank) | vecu(l.a2_b, (size_t)d.heads * d.dim, -2.0f, 2.0f) |
+                   vecu(l.mu, (size_t)5 * W, 0.5f, 0.5f) | vecu(l.bonus, (size_t)d.heads * d.dim, 0.0f, 0.5f);
+        }
+        if (l.delta()) bad |= vecu(l.dt_bias, d.heads, -2.0f, 1.0f) | vecu(l.a_log, d.heads, 0.0f, 1.0f);
+        if (l.has_lt()) {
+            bad |= vec(l.lt_norm, l.lt_inner(), true) | vec(l.lt_decay, d.lt_heads, true);
+            std::vector<float> dc(d.lt_heads);
+            for (int h = 0; h < d.lt_heads; h++) dc[h] = 1.0f - std::exp2(-5.0f - (float)(h % 8));
+            if (!bad) bad |= hipMemcpy(l.lt_decay.p, dc.data(), dc.size() * 4, hipMemcpyHostToDevice) != hipSuccess;
+        }
+        if (d.ff_bias) bad |= vec(l.h_bias, l.n_h, false) | vec(l.down_b, W, false);
+        if (s->c.token_side > 0) bad |= mat(l.side_gate, (size_t)s->c.token_side * W, W) | mat(l.side_proj, (size_t)W * s->c.token_side, s->c.token_side) | vec(l.side_norm, W, true);
+        std::fill(l.have_mu, l.have_mu + 5, (char)1);
         if (l.has_ssd()) {
             bad |= vecu(l.sconv_w, (size_t)l.ssd_conv_c() * d.ssd_conv, 1.0f / (float)d.ssd_conv, 0.5f / (float)d.ssd_conv) | vec(l.sconv_b, l.ssd_conv_c(), false) |
                    vecu(l.dt_bias, d.ssd_heads, -2.0f, 1.0f) | vecu(l.a_log, d.ssd_heads, 0.0f, 1.0f) | vec(l.ssd_d, d.ssd_heads, true) | vec(l.ssd_norm, l.ssd_inner(), true);
@@ -740,6 +848,8 @@ int kr_serve_finalize(kr_serve* s) {
     if (s->c.norm_bias && !s->have_fb) return kr_fail(KR_ERR_STATE, "final norm bias missing");
     if (s->c.embed_norm && !s->have_enorm) return kr_fail(KR_ERR_STATE, "embedding norm missing");
     if (s->c.bigram_buckets > 0 && !s->have_bigram) return kr_fail(KR_ERR_STATE, "pair embedding missing");
+    if (s->c.pos_rows > 0 && !s->have_pos) return kr_fail(KR_ERR_STATE, "position rows missing");
+    if (s->c.token_side > 0 && !s->have_side) return kr_fail(KR_ERR_STATE, "per-layer token table missing");
     const bool seq = s->c.block_kind == KR_SERVE_BLOCK_SEQUENTIAL, nb = s->c.norm_bias != 0;
     for (int i = 0; i < s->c.n_layers; i++) {
         SvLayer& l = s->L[i]; const kr_serve_layer& d = l.d;
@@ -747,7 +857,7 @@ int kr_serve_finalize(kr_serve* s) {
         if (d.pre_add && !l.have[KR_SV_PRE_ADD]) return kr_fail(KR_ERR_STATE, "layer %d: the vector before the layer is missing", i);
         if (l.wsrc != i) continue;
         std::vector<int> need;
-        if (!l.ssd_alone()) need.push_back(KR_SV_O);
+        if (!l.side_alone()) need.push_back(KR_SV_O);
         if (s->c.pre_norm) { need.push_back(KR_SV_NORM_W); if (nb) need.push_back(KR_SV_NORM_B); }
         if (s->c.pre_norm && seq && has_ff) { need.push_back(KR_SV_NORM2_W); if (nb) need.push_back(KR_SV_NORM2_B); }
         if (s->c.post_norm) { need.push_back(KR_SV_POST1_W); if (nb) need.push_back(KR_SV_POST1_B); }
@@ -762,10 +872,15 @@ int kr_serve_finalize(kr_serve* s) {
             if (d.kv_from < 0) { need.push_back(KR_SV_K); if (!d.v_from_k) need.push_back(KR_SV_V); }
         }
         if (d.qk_unit_norm == KR_SERVE_QKNORM_WEIGHTED || d.qk_unit_norm == KR_SERVE_QKNORM_WHOLE) { need.push_back(KR_SV_Q_NORM); if (d.kv_from < 0) need.push_back(KR_SV_K_NORM); }
-        if (d.proj_bias) { need.push_back(KR_SV_Q_BIAS); need.push_back(KR_SV_O_BIAS); if (d.kv_from < 0) need.push_back(KR_SV_K_BIAS); }
-        if (d.proj_bias == 2) need.push_back(KR_SV_V_BIAS);
+        if (d.proj_bias) { need.push_back(KR_SV_Q_BIAS); if (d.proj_bias != 3) need.push_back(KR_SV_O_BIAS); if (d.kv_from < 0) need.push_back(KR_SV_K_BIAS); }
+        if (d.proj_bias >= 2) need.push_back(KR_SV_V_BIAS);
         if (d.proj_conv) for (int r : {KR_SV_Q_CONV, KR_SV_K_CONV, KR_SV_V_CONV}) need.push_back(r);
-        if (l.gla()) for (int r : {KR_SV_DECAY_A1, KR_SV_DECAY_A2, KR_SV_DECAY_A2_B}) need.push_back(r);
+        if (l.gla() || l.wkv()) for (int r : {KR_SV_DECAY_A1, KR_SV_DECAY_A2, KR_SV_DECAY_A2_B}) need.push_back(r);
+        if (l.wkv()) { need.push_back(KR_SV_WKV_U); for (int m = 0; m < 5; m++) if (!l.have_mu[m]) return kr_fail(KR_ERR_STATE, "layer %d: weights of shifted input %d missing", i, m); }
+        if (l.delta()) for (int r : {KR_SV_DELTA_B, KR_SV_DELTA_A, KR_SV_SSD_A_LOG, KR_SV_SSD_DT_BIAS}) need.push_back(r);
+        if (l.has_lt()) for (int r = KR_SV_LT_Q; r <= KR_SV_LT_DECAY; r++) need.push_back(r);
+        if (d.ff_bias) { if (!l.ungated_ff()) need.push_back(KR_SV_GATE_B); need.push_back(KR_SV_UP_B); need.push_back(KR_SV_DOWN_B); }
+        if (s->c.token_side > 0) for (int r : {KR_SV_SIDE_GATE, KR_SV_SIDE_PROJ, KR_SV_SIDE_NORM}) need.push_back(r);
         if (l.has_ssd()) for (int r = KR_SV_SSD_IN; r <= KR_SV_SSD_O; r++) need.push_back(r);
         if (d.out_gate || l.recurrent()) need.push_back(KR_SV_OUT_GATE);
         if (l.recurrent() && d.lin_norm_weight) need.push_back(KR_SV_LIN_NORM);
@@ -841,6 +956,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         for (int f = 0; f < e; f++) if (slots[f] == sl) return kr_fail(KR_ERR_VALUE, "slot %d appears twice in one step", sl);
         if (counts[e] < 1) return kr_fail(KR_ERR_VALUE, "entry %d: %d tokens", e, counts[e]);
         const SvSlot& q = s->slots[sl];
+        if (c.pos_rows > 0 && q.len + counts[e] > c.pos_rows) return kr_fail(KR_ERR_VALUE, "entry %d: %d positions, the design has %d", e, q.len + counts[e], c.pos_rows);
         need_pages += (q.len + counts[e] + PT - 1) / PT - (int)q.pages.size();
         T64 += counts[e];
     }
@@ -898,7 +1014,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     const bool lin_chunked = max_count >= 32;
     // the gated linear recurrence: one launch when every entry brings one token, else chunks of 64 tokens
     const bool rg_step = max_count == 1;
-    size_t max_rg = 0;
+    size_t max_rg = 0; bool any_wkv = false;
     for (const SvLayer& l : s->L) {
         const kr_serve_layer& d = l.d;
         if (d.proj_conv) max_pconv = std::max(max_pconv, (size_t)l.pconv_c());
@@ -907,6 +1023,17 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             if (lin_chunked && kr_sv_lin_chunked_fits(d.ssd_state, d.ssd_vdim)) {
                 lin_tok = std::max(lin_tok, (size_t)d.ssd_heads); lin_sb = std::max(lin_sb, (size_t)d.ssd_heads * d.ssd_state * d.ssd_vdim); lin_nb = std::max(lin_nb, (size_t)d.ssd_heads * d.ssd_state);
                 max_ssdz = std::max(max_ssdz, (size_t)d.ssd_heads * (2 * d.ssd_state + d.ssd_vdim));
+            }
+        }
+        if (l.delta()) lin_tok = std::max(lin_tok, (size_t)d.heads);
+        if (l.wkv()) {
+            any_wkv = true; max_gz = std::max(max_gz, (size_t)d.heads * d.dim); head_i = std::max(head_i, (size_t)5);
+            max_pconv = std::max(max_pconv, (size_t)(4 + l.decay_out_rows()) * d.heads * d.dim);
+        }
+        if (l.has_lt()) {
+            max_lin = std::max(max_lin, (size_t)l.lt_inner());
+            if (lin_chunked && kr_sv_lin_chunked_fits(d.lt_dim, d.lt_vdim)) {
+                lin_tok = std::max(lin_tok, (size_t)d.lt_heads); lin_sb = std::max(lin_sb, (size_t)d.lt_heads * d.lt_dim * d.lt_vdim); lin_nb = std::max(lin_nb, (size_t)d.lt_heads * d.lt_dim);
             }
         }
         if (l.gla()) { max_ga1 = std::max(max_ga1, (size_t)d.decay_rank); max_gz = std::max(max_gz, (size_t)d.heads * d.dim); }
@@ -924,6 +1051,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             lq_c = std::max(lq_c, (size_t)d.q_rank); lq_2 = std::max(lq_2, (size_t)d.heads * (d.dim + d.rot_dims)); lq_n = std::max(lq_n, (size_t)d.heads * d.dim);
             lq_e = std::max(lq_e, (size_t)d.heads * l.att_dim()); att2 = std::max(att2, (size_t)d.heads * d.vdim); head_i = std::max(head_i, (size_t)d.heads);
         }
+        if (c.token_side > 0) max_y = std::max(max_y, (size_t)c.token_side);
         if (d.mlp_kind == KR_SERVE_MLP_DENSE) { max_gu = std::max(max_gu, (size_t)2 * d.ff); max_y = std::max(max_y, (size_t)d.ff); }
         if (d.mlp_kind == KR_SERVE_MLP_MOE) {
             max_gu = std::max(max_gu, std::max((size_t)d.top * 2 * d.expert_ff, (size_t)2 * d.shared_ff));
@@ -941,11 +1069,12 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         (head_i && (s->lq_c.ensure(Ts * lq_c * s->esz) || s->lq_2.ensure(Ts * lq_2 * 4) || s->lq_n.ensure(Ts * lq_n * s->esz) || s->lq_e.ensure(Ts * lq_e * 4) ||
                     s->att2.ensure(Ts * att2 * s->esz) || s->head_i.ensure((2 * Ts * head_i + head_i + 1) * 4))))
         return kr_fail(KR_ERR_HIP, "mixer scratch for %d tokens", T);
-    if ((c.canon_taps > 1 && (s->h32.ensure(Ts * W * 4) || s->hc.ensure(Ts * W * s->esz))) || (c.res_gate && s->rg.ensure(Ts * W * 4)) || (whole_norm && s->qk_rms.ensure(Ts * 2 * 4)) ||
+    if ((any_wkv && (s->h32.ensure(Ts * W * 4) || s->mixes.ensure(5 * Ts * W * s->esz))) || (c.token_side > 0 && s->sgate.ensure(Ts * c.token_side * 4)) ||
+        (c.canon_taps > 1 && (s->h32.ensure(Ts * W * 4) || s->hc.ensure(Ts * W * s->esz))) || (c.res_gate && s->rg.ensure(Ts * W * 4)) || (whole_norm && s->qk_rms.ensure(Ts * 2 * 4)) ||
         (max_lin && s->lin_o.ensure(Ts * max_lin * 4)) ||
         (lin_tok && (s->lin_tok.ensure(Ts * lin_tok * 16) || s->lin_sbuf.ensure((size_t)n_chunks * lin_sb * 4) || s->lin_nbuf.ensure((size_t)n_chunks * lin_nb * 4) || s->lin_cm.ensure((size_t)n_chunks * lin_tok * 16))))
         return kr_fail(KR_ERR_HIP, "block scratch for %d tokens", T);
-    if ((max_pconv && s->qkv2.ensure(Ts * max_pconv * 4)) || (max_sconv && s->sconv.ensure(Ts * max_sconv * 4)) || (max_ga1 && (s->ga1.ensure(Ts * max_ga1 * s->esz) || s->gz.ensure(Ts * max_gz * 4))))
+    if ((max_pconv && s->qkv2.ensure(Ts * max_pconv * 4)) || (max_sconv && s->sconv.ensure(Ts * max_sconv * 4)) || (max_ga1 && s->ga1.ensure(Ts * max_ga1 * s->esz)) || (max_gz && s->gz.ensure(Ts * max_gz * 4)))
         return kr_fail(KR_ERR_HIP, "convolution / decay scratch for %d tokens", T);
     if (max_rg && (s->rg_ab.ensure(Ts * max_rg * 8) || s->rg_agg.ensure((size_t)n_chunks * max_rg * 8) || s->rg_start.ensure((size_t)n_chunks * max_rg * 4)))
         return kr_fail(KR_ERR_HIP, "recurrence scratch for %d tokens", T);
@@ -956,7 +1085,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     for (int li = 0; li < c.n_layers; li++) {
         const SvLayer& l = s->L[li]; const kr_serve_layer& d = l.d;
         if (l.recurrent() || l.no_heads()) continue;
-        const int visible = d.window > 0 ? std::min(max_pos + 1, d.window) : (d.chunk > 0 ? std::min(max_pos + 1, d.chunk) : max_pos + 1);
+        const int visible = d.window > 0 ? std::min(max_pos + 1, d.window + d.keep_first) : (d.chunk > 0 ? std::min(max_pos + 1, d.chunk) : max_pos + 1);
         const int ldk = l.latent() ? l.att_dim() : d.kv_heads * d.dim, ldv = l.latent() ? l.att_dim() : d.kv_heads * d.vdim;
         nsplit[li] = kr_sv_attention_splits(T, d.heads, l.att_heads_kv(), l.att_dim(), l.att_vdim(), ldk, ldv, s->f32, visible);
         if (nsplit[li] > 1 && (s->part_ml.ensure(Ts * d.heads * nsplit[li] * 8) || s->part_acc.ensure(Ts * d.heads * nsplit[li] * l.att_vdim() * 4)))
@@ -968,8 +1097,8 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     float* x = (float*)s->x.p;
     {
         Timer tm(s, 7);
-        kr_sv_embed(s->embed.p, s->f32, d_tok, x, c.pre_norm ? nullptr : s->h.p, T, W, c.embed_scale != 0.0f ? c.embed_scale : 1.0f, c.bigram_buckets > 0 ? s->bigram.p : nullptr, d_brow,
-                    st);     // without input norms the first sublayer reads the embedding row itself
+        kr_sv_embed(s->embed.p, s->f32, d_tok, x, c.pre_norm ? nullptr : s->h.p, T, W, c.embed_scale != 0.0f ? c.embed_scale : 1.0f, c.pos_rows > 0 ? s->pos.p : c.bigram_buckets > 0 ? s->bigram.p : nullptr,
+                    c.pos_rows > 0 ? d_pos : d_brow, st);     // without input norms the first sublayer reads the embedding row itself
     }
     if (c.embed_norm) { Timer tm(s, 0); kr_sv_stream_norm(x, nullptr, (const float*)s->enorm_w.p, nullptr, true, nullptr, s->f32, T, W, c.norm_eps, c.norm_kind, c.norm_groups > 1 ? c.norm_groups : 1, st); }
     {
@@ -980,7 +1109,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     // down projection of a gated feed-forward: decode-sized problems form the activation inside the projection's launch, larger ones write it once
     auto down_proj = [&](KrSvGemm g, const float* gu, int ld, int rows_m, int F, int kind, float limit, float alpha, const float* row_w = nullptr) {
         if (kr_sv_gemm_small(g)) { g.act_row_w = row_w; g.act_gu = gu; g.act_ld = ld; g.act_kind = kind; g.act_limit = limit; g.act_alpha = alpha; g.A = nullptr; Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); return; }
-        { Timer tm(s, 5); kr_sv_act(gu, ld, s->y.p, s->f32, rows_m, F, kind, limit, alpha, row_w, st); }
+        { Timer tm(s, 5); kr_sv_act(gu, ld, s->y.p, s->f32, rows_m, F, kind, limit, alpha, row_w, st, g.up_tab, g.up_rows, g.up_ld, g.up_off); }
         g.A = s->y.p; g.lda = F;
         { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
     };
@@ -990,7 +1119,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     const bool canon = c.canon_taps > 1;
     // gate: 0 none, 1 the mixer's (logits in rg, the output projection's bias, and the input convolution's rows of this layer are kept), 2 the feed-forward's
     // (logits in the last row block of hz).  to_mixer: the handed-on row feeds a mixer (an f32 copy goes along for its input convolution)
-    const SvLayer* res_layer = nullptr; const SvLayer* res_run = nullptr; int res_gate_kind = 0; bool res_to_mixer = false;
+    const SvLayer* res_layer = nullptr; const SvLayer* res_run = nullptr; int res_gate_kind = 0; bool res_to_mixer = false, res_next32 = false;
     auto residual = [&](const float* mixp, const float* dense, const float* shared, const float* rows, const int* pair_pos, int top, const DevBuf* post_w, const DevBuf* post_b,
                         bool hand_on, const DevBuf* next_w, const DevBuf* next_b) {
         Timer tm(s, 6);
@@ -998,13 +1127,14 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         r.groups = NG;
         if (res_layer) {
             const SvLayer& rl = *res_layer;
-            if (mixp && rl.d.proj_bias) r.mix_bias = (const float*)rl.o_bias.p;
+            if (mixp && (rl.d.proj_bias == 1 || rl.d.proj_bias == 2)) r.mix_bias = (const float*)rl.o_bias.p;
             if (res_gate_kind == 1) {
                 if (c.res_gate) { r.gate = (const float*)s->rg.p; r.ld_gate = W; r.gate_b = (const float*)rl.rg1_b.p; }
                 if (canon) { r.h32_in = (const float*)s->h32.p; r.canon_state = (float*)res_run->canon_state.p; r.canon_keep = c.canon_taps - 1; r.slot = d_slot; r.pos = d_pos; }
+                if (rl.wkv()) { r.h32_in = (const float*)s->h32.p; r.canon_state = (float*)res_run->shift_state.p; r.canon_keep = 1; r.slot = d_slot; r.pos = d_pos; }
             } else if (res_gate_kind == 2 && c.res_gate) { r.gate = (const float*)s->qkv.p + rl.off_rg2; r.ld_gate = rl.n_h; r.gate_b = (const float*)rl.rg2_b.p; }
         }
-        if (canon && hand_on && res_to_mixer) r.h32_out = (float*)s->h32.p;
+        if ((canon || res_next32) && hand_on && res_to_mixer) r.h32_out = (float*)s->h32.p;
         r.x = x; r.mix = mixp; r.dense = dense; r.shared = shared; r.rows = rows; r.pair_pos = pair_pos; r.wts = (res_layer && res_layer->d.expert_in_weight) ? nullptr : (const float*)s->wts.p; r.top = top;
         r.post_w = post_w ? (const float*)post_w->p : nullptr; r.post_b = (post_w && c.norm_bias && post_b) ? (const float*)post_b->p : nullptr; r.mult = c.residual_mult;
         r.norm_w = (hand_on && next_w) ? (const float*)next_w->p : nullptr; r.norm_b = (hand_on && next_w && c.norm_bias && next_b) ? (const float*)next_b->p : nullptr;
@@ -1014,7 +1144,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     if (c.pre_norm && !s->L[0].d.pre_add) {
         Timer tm(s, 0);
         kr_sv_norm(x, nullptr, (const float*)s->L[0].norm_w.p, c.norm_bias ? (const float*)s->L[0].norm_b.p : nullptr, s->h.p, s->f32, T, W, c.norm_eps, c.norm_kind, NG,
-                   canon ? (float*)s->h32.p : nullptr, st);
+                   (canon || s->L[0].wkv()) ? (float*)s->h32.p : nullptr, st);
     }
     int head_rows_for = 0;               // the head row tables in head_i are valid for this head count
     for (int li = 0; li < c.n_layers; li++) {
@@ -1022,8 +1152,9 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         SvLayer& l = s->L[run.wsrc]; const kr_serve_layer& d = l.d;       // tensors and layout: the layer that owns them
         const SvLayer* nxrun = li + 1 < c.n_layers ? &s->L[li + 1] : nullptr;
         const SvLayer* nx = nxrun ? &s->L[nxrun->wsrc] : nullptr;
-        const bool hand = nxrun && !nxrun->d.pre_add;     // a layer with a vector before it forms its own input from the stream
+        const bool hand = nxrun && !nxrun->d.pre_add, side = c.token_side > 0;     // a layer with a vector before it forms its own input from the stream
         const bool has_ff = d.mlp_kind != KR_SERVE_MLP_NONE;
+        res_next32 = nx && nx->wkv();                     // its mixer reads the normed row in f32
         if (run.d.pre_add) {
             Timer tm(s, 0);
             kr_sv_stream_norm(x, (const float*)run.pre_add.p, (const float*)l.norm_w.p, c.norm_bias ? (const float*)l.norm_b.p : nullptr, false, s->h.p, s->f32, T, W, c.norm_eps, c.norm_kind, NG, st);
@@ -1043,11 +1174,12 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             Timer tm(s, 1); kr_sv_gemm(gg, s->f32, st);
         }
         g.A = mixer_in; g.lda = W; g.W = l.hw.p; g.C = hz; g.ldc = l.n_h; g.M = T; g.N = seq ? l.n_qkv : l.n_h; g.K = W;
-        { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
+        g.bias = d.ff_bias ? (const float*)l.h_bias.p : nullptr;
+        if (g.N > 0) { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
         const SvLayer& kvl = d.kv_from >= 0 ? s->L[d.kv_from] : run;
         KrSvAttn a{};
         a.heads = d.heads; a.kv_heads = l.att_heads_kv(); a.dim = l.att_dim(); a.vdim = l.att_vdim();
-        a.eps = c.norm_eps; a.scale = d.scale; a.window = d.window; a.chunk = d.chunk; a.slopes = d.dist_bias ? (const float*)l.slopes.p : nullptr;
+        a.eps = c.norm_eps; a.scale = d.scale; a.window = d.window; a.keep = d.window > 0 ? d.keep_first : 0; a.chunk = d.chunk; a.slopes = d.dist_bias ? (const float*)l.slopes.p : nullptr;
         a.sink = d.has_sink ? (const float*)l.sink.p : nullptr;
         a.kpool = kvl.kpool.p; a.page_table = d_tab; a.table_ld = s->n_pages; a.slot = d_slot; a.pos = d_pos; a.page_tokens = PT; a.T = T;
         a.out = s->att.p;
@@ -1072,6 +1204,30 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
                 q.gz = (const float*)s->gz.p; q.gz_ld = d.heads * d.dim; q.gz_bias = (const float*)l.a2_b.p; q.inv_tau = 1.0f / d.decay_tau;
                 q.q_scale = isd; q.k_scale = 1.0f;
             }
+            if (l.wkv()) {
+                // five shifted inputs, one grouped GEMM ([r | k | v | g] side by side per token, the decay's low-rank vector behind all of them), then the log decays
+                const int hd = d.heads * d.dim;
+                int* hseg = (int*)s->head_i.p; int* hrows = hseg + 6; int* hgroup = hrows + (size_t)5 * T;
+                head_rows_for = 0;
+                KrSvShift sh{}; sh.h32 = (const float*)s->h32.p; sh.mu = (const float*)l.mu.p; sh.n = 5; sh.state = (const float*)run.shift_state.p; sh.slot = d_slot; sh.pos = d_pos; sh.T = T; sh.width = W;
+                sh.out = s->mixes.p; sh.seg = hseg; sh.c_rows = hrows; sh.group = hgroup; sh.last_rows = l.decay_out_rows();
+                { Timer tm(s, 2); kr_sv_shift(sh, s->f32, st); }
+                KrSvGemm gw{}; gw.A = s->mixes.p; gw.lda = W; gw.W = l.wk.p; gw.w_stride = (size_t)hd * W; gw.C = (float*)s->qkv2.p; gw.ldc = hd; gw.c_rows = hrows; gw.M = 5 * T; gw.K = W;
+                gw.N = std::max(hd, d.decay_rank); gw.n_first = hd; gw.n_last = d.decay_rank; gw.seg = hseg; gw.row_group = hgroup; gw.n_groups = 5;
+                { Timer tm(s, 1); kr_sv_gemm(gw, s->f32, st); }
+                { Timer tm(s, 2); kr_sv_wkv_decay((const float*)s->qkv2.p + (size_t)4 * T * hd, l.decay_out_rows() * hd, l.a2.p, s->f32, (const float*)l.a2_b.p, T, d.decay_rank, hd, (float*)s->gz.p, st); }
+                q.z = (float*)s->qkv2.p; q.ld = 4 * hd; q.qsrc = q.z; q.ksrc = q.z + hd; q.vsrc = q.z + 2 * hd; q.src_ld = q.ld; q.qk_group = 1; q.gz = (const float*)s->gz.p; q.gz_ld = hd;
+                q.bonus = (const float*)l.bonus.p; q.q_scale = q.k_scale = 1.0f; q.gate = q.z + 3 * hd; q.gate_ld = q.ld; q.gate_act = 1;
+            }
+            if (l.delta()) {
+                KrSvDelta dl{};
+                dl.z = hz; dl.ld = l.n_h; dl.bz = hz + l.off_ba; dl.az = dl.bz + d.heads; dl.heads = d.heads; dl.kv_heads = d.kv_heads; dl.dim = d.dim; dl.vdim = d.vdim; dl.taps = d.proj_conv;
+                dl.conv = (const float*)l.pconv_w.p; dl.a_log = (const float*)l.a_log.p; dl.dt_bias = (const float*)l.dt_bias.p; dl.ring = (float*)run.delta_ring.p; dl.slot = d_slot; dl.pos = d_pos;
+                dl.T = T; dl.ent_off = d_eoff; dl.n_entries = n_entries; dl.single = rg_step; dl.out = (float*)s->qkv2.p; dl.tok = (float4*)s->lin_tok.p;
+                { Timer tm(s, 2); kr_sv_delta_prep(dl, st); }
+                q.z = (float*)s->qkv2.p; q.ld = l.pconv_c(); q.qsrc = q.z; q.ksrc = q.z + l.q_rows(); q.vsrc = q.ksrc + l.k_rows(); q.src_ld = q.ld; q.qk_group = d.heads / d.kv_heads;
+                q.q_scale = q.k_scale = 1.0f; q.gate = hz + l.off_ogate; q.gate_ld = l.n_h; q.gate_act = 1;
+            }
             q.ent_chunk0 = d_echunk; q.n_chunks = n_chunks; q.tok = (float4*)s->lin_tok.p; q.sbuf = (float*)s->lin_sbuf.p; q.nbuf = (float*)s->lin_nbuf.p; q.cmeta = (float*)s->lin_cm.p;
             {
                 Timer tm(s, 3);
@@ -1089,8 +1245,8 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             q.ab = (float2*)s->rg_ab.p; q.agg = (float2*)s->rg_agg.p; q.start = (float*)s->rg_start.p;
             Timer tm(s, 3);
             if (rg_step) kr_sv_rglru_step(q, s->f32, st); else kr_sv_rglru_portions(q, s->f32, st);
-        } else if (l.ssd_alone()) {
-            // no first mixer: the state-space mixer below is the layer's only one
+        } else if (l.side_alone()) {
+            // no first mixer: the mixer below is the layer's only one
         } else if (!l.latent()) {
             a.qkv = hz; a.ldq = l.n_h; a.rot_dims = d.rot_dims; a.rot_interleaved = d.rot_interleaved; a.unit_norm = d.qk_unit_norm; a.own_kv = d.kv_from < 0;
             a.q_norm_w = (const float*)l.q_norm.p; a.k_norm_w = (const float*)l.k_norm.p;
@@ -1100,8 +1256,8 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             a.q_bias = d.proj_bias ? (const float*)l.q_bias.p : nullptr; a.k_bias = (d.proj_bias && d.kv_from < 0) ? (const float*)l.k_bias.p : nullptr;
             a.inv_rms = a.inv_rms_out = (float*)s->qk_rms.p; a.v_from_k = d.v_from_k; a.softcap = d.softcap;
             if (d.out_gate) { a.out_gate = hz + l.off_ogate; a.ld_gate = l.n_h; a.gate_elem = d.out_gate == KR_SERVE_OGATE_ELEM_SIGMOID; }
-            a.v_bias = d.proj_bias == 2 ? (const float*)l.v_bias.p : nullptr;
-            if (l.has_ssd()) { a.out_ld = l.o_cols(); a.out_scale = d.mix_scale; }
+            a.v_bias = d.proj_bias >= 2 ? (const float*)l.v_bias.p : nullptr;
+            if (l.has_side()) { a.out_ld = l.o_cols(); a.out_scale = d.mix_scale; }
             if (d.proj_conv) {
                 // q | k | v with their biases pass the short convolution; the preparation below reads the convolved rows and adds no bias again
                 KrSvChanConv cv{}; cv.in = hz; cv.ld_in = l.n_h; cv.in_bias = d.proj_bias ? (const float*)l.pconv_bias.p : nullptr; cv.w = (const float*)l.pconv_w.p; cv.taps = d.proj_conv;
@@ -1183,23 +1339,43 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             so.out = (char*)s->att.p + (size_t)l.att_out_cols() * s->esz; so.out_ld = l.o_cols(); so.T = T;
             { Timer tm(s, 2); kr_sv_ssd_out(so, s->f32, st); }
         }
+        if (l.has_lt()) {
+            // [q | k | v | g] came out of the layer's one GEMM; a retention on silu'd rows, then one norm over the heads laid side by side
+            float* zin = hz + l.off_lt;
+            KrSvLin q{};
+            q.kind = KR_SERVE_MIX_RETENTION; q.z = zin; q.ld = l.n_h; q.heads = d.lt_heads; q.dim = d.lt_dim; q.vdim = d.lt_vdim; q.q_scale = q.k_scale = 1.0f; q.decay = (const float*)l.lt_decay.p;
+            q.qkv_act = 1; q.state = (float*)run.lt_state.p; q.state_stride = l.lt_state_stride; q.ent_off = d_eoff; q.ent_slot = d_eslot; q.n_entries = n_entries; q.pos = d_pos; q.T = T;
+            q.o = (float*)s->lin_o.p; q.ent_chunk0 = d_echunk; q.n_chunks = n_chunks; q.tok = (float4*)s->lin_tok.p; q.sbuf = (float*)s->lin_sbuf.p; q.nbuf = (float*)s->lin_nbuf.p; q.cmeta = (float*)s->lin_cm.p;
+            {
+                Timer tm(s, 3);
+                if (lin_chunked && kr_sv_lin_chunked_fits(d.lt_dim, d.lt_vdim)) {
+                    kr_sv_lt_prep(zin, l.n_h, l.lt_cols(), q.decay, d.lt_heads, q.tok, T, st);
+                    q.prepped = 1; kr_sv_lin_chunked(q, st);
+                } else kr_sv_lin_scan(q, st);
+            }
+            Timer tm(s, 2);
+            kr_sv_row_out((const float*)s->lin_o.p, l.lt_inner(), (const float*)l.lt_norm.p, zin + l.lt_cols(), l.n_h, c.norm_eps, (d.side_mixer && d.side_scale != 0.0f) ? d.side_scale : 1.0f,
+                          (char*)s->att.p + (size_t)l.att_out_cols() * s->esz, l.o_cols(), s->f32, T, st);
+        }
         g = KrSvGemm{};
         g.A = o_in; g.lda = l.latent() ? d.heads * d.vdim : l.o_cols(); g.W = l.o.p; g.C = (float*)s->mix.p; g.ldc = W; g.M = T; g.N = W; g.K = g.lda;
         { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
         if (seq) {
             // the mixer's sublayer ends here; the new x, normed or as it is, is the feed-forward's input (or the next layer's when there is none)
-            res_layer = &l; res_run = &run; res_gate_kind = 1; res_to_mixer = !has_ff;
+            res_layer = &l; res_run = &run; res_gate_kind = 1; res_to_mixer = !has_ff && !side;
             if (has_ff) residual((const float*)s->mix.p, nullptr, nullptr, nullptr, nullptr, 0, c.post_norm ? &l.post1_w : nullptr, &l.post1_b, true, c.pre_norm ? &l.norm2_w : nullptr, &l.norm2_b);
-            else residual((const float*)s->mix.p, nullptr, nullptr, nullptr, nullptr, 0, c.post_norm ? &l.post1_w : nullptr, &l.post1_b, hand, (nx && c.pre_norm) ? &nx->norm_w : nullptr,
+            else residual((const float*)s->mix.p, nullptr, nullptr, nullptr, nullptr, 0, c.post_norm ? &l.post1_w : nullptr, &l.post1_b, hand || side, (nx && c.pre_norm && !side) ? &nx->norm_w : nullptr,
                           nx ? &nx->norm_b : nullptr);
             if (has_ff && l.n_h > l.off_router) {
                 g = KrSvGemm{}; g.A = s->h.p; g.lda = W; g.W = (const char*)l.hw.p + (size_t)l.off_router * W * s->esz; g.C = hz + l.off_router; g.ldc = l.n_h; g.M = T; g.N = l.n_h - l.off_router; g.K = W;
+                g.bias = d.ff_bias ? (const float*)l.h_bias.p + l.off_router : nullptr;
                 Timer tm(s, 1); kr_sv_gemm(g, s->f32, st);
             }
         }
         const float *dense = nullptr, *shared = nullptr, *rows = nullptr; const int* pair_pos = nullptr;
         if (d.mlp_kind == KR_SERVE_MLP_DENSE) {
             g = KrSvGemm{}; g.W = l.down.p; g.C = (float*)s->ffout.p; g.ldc = W; g.M = T; g.N = W; g.K = d.ff;
+            g.bias = d.ff_bias ? (const float*)l.down_b.p : nullptr;
             down_proj(g, hz + l.off_gu, l.n_h, T, d.ff, d.dense_act, 0.0f, 1.0f);
             dense = (const float*)s->ffout.p;
         } else if (d.mlp_kind == KR_SERVE_MLP_MOE) {
@@ -1227,10 +1403,21 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             }
         }
         // x += the layer's sublayers (parallel block) or the feed-forward alone (sequential), and the next layer's input from the same launch
-        res_layer = &l; res_run = &run; res_gate_kind = seq ? 2 : 0; res_to_mixer = true;
-        if (!seq) residual((const float*)s->mix.p, dense, shared, rows, pair_pos, d.top, nullptr, nullptr, hand, (nx && c.pre_norm) ? &nx->norm_w : nullptr, nx ? &nx->norm_b : nullptr);
-        else if (has_ff) residual(nullptr, dense, shared, rows, pair_pos, d.top, c.post_norm ? &l.post2_w : nullptr, &l.post2_b, hand, (nx && c.pre_norm) ? &nx->norm_w : nullptr,
+        res_layer = &l; res_run = &run; res_gate_kind = seq ? 2 : l.wkv() ? 1 : 0; res_to_mixer = !side;
+        if (!seq) residual((const float*)s->mix.p, dense, shared, rows, pair_pos, d.top, nullptr, nullptr, hand || side, (nx && c.pre_norm && !side) ? &nx->norm_w : nullptr, nx ? &nx->norm_b : nullptr);
+        else if (has_ff) residual(nullptr, dense, shared, rows, pair_pos, d.top, c.post_norm ? &l.post2_w : nullptr, &l.post2_b, hand || side, (nx && c.pre_norm && !side) ? &nx->norm_w : nullptr,
                                   nx ? &nx->norm_b : nullptr);
+        if (side) {
+            // the token's own row for this layer: gate from the stream as it stands, times the row, projected, normed, added; the next layer's input from the same launch
+            const int ns = c.token_side;
+            g = KrSvGemm{}; g.A = s->h.p; g.lda = W; g.W = l.side_gate.p; g.C = (float*)s->sgate.p; g.ldc = ns; g.M = T; g.N = ns; g.K = W;
+            { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
+            g = KrSvGemm{}; g.W = l.side_proj.p; g.C = (float*)s->mix.p; g.ldc = W; g.M = T; g.N = W; g.K = ns;
+            g.up_tab = s->side_embed.p; g.up_rows = d_tok; g.up_ld = c.n_layers * ns; g.up_off = li * ns;
+            down_proj(g, (const float*)s->sgate.p, ns, T, ns, KR_SV_ACT_GELU_TANH, 0.0f, 1.0f);
+            res_layer = nullptr; res_run = nullptr; res_gate_kind = 0; res_to_mixer = true;
+            residual((const float*)s->mix.p, nullptr, nullptr, nullptr, nullptr, 0, &l.side_norm, nullptr, hand, (nx && c.pre_norm) ? &nx->norm_w : nullptr, nx ? &nx->norm_b : nullptr);
+        }
         if (s->capture) KR_HIP(hipMemcpyAsync((float*)s->cap.p + (size_t)li * Ts * W, x, Ts * W * 4, hipMemcpyDeviceToDevice, st));
     }
     if (n_want > 0) {
@@ -1252,7 +1439,8 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         mixin((uint64_t)T); mixin((uint64_t)n_want); mixin(want_amax);
         for (int v : nsplit) mixin((uint64_t)v);
         for (const DevBuf* b : {&s->meta, &s->x, &s->h, &s->qkv, &s->att, &s->mix, &s->gu, &s->y, &s->rows, &s->ffout, &s->ids, &s->wts, &s->rz, &s->moe_i, &s->hw, &s->logits,
-                                &s->amax, &s->part_ml, &s->part_acc, &s->v_first, &s->lq_c, &s->lq_2, &s->lq_n, &s->lq_e, &s->att2, &s->head_i, &s->h32, &s->hc, &s->rg, &s->qk_rms, &s->lin_o, &s->qkv2, &s->sconv, &s->ga1, &s->gz, &s->rg_ab, &s->rg_agg, &s->rg_start}) mixin((uint64_t)(uintptr_t)b->p);
+                                &s->amax, &s->part_ml, &s->part_acc, &s->v_first, &s->lq_c, &s->lq_2, &s->lq_n, &s->lq_e, &s->att2, &s->head_i, &s->h32, &s->hc, &s->rg, &s->qk_rms, &s->lin_o, &s->qkv2, &s->sconv, &s->ga1, &s->gz, &s->rg_ab, &s->rg_agg, &s->rg_start,
+                                &s->mixes, &s->sgate, &s->lin_tok}) mixin((uint64_t)(uintptr_t)b->p);
         for (const SvRope& r : s->ropes) mixin((uint64_t)(uintptr_t)r.cs.p);
         hipGraphExec_t exec = nullptr;
         for (auto& g : s->graphs) if (g.key == key) exec = g.exec;

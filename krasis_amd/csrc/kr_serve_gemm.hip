@@ -24,10 +24,14 @@ template <bool BF>
 __device__ __forceinline__ void gm_store(const KrSvGemm& g, int m, int n, float v) {
     const int row = g.c_rows ? g.c_rows[m] : m;
     const size_t i = (size_t)row * g.ldc + n;
+    if (g.bias) v += g.bias[n];
     if (g.o_gate) v *= 1.0f / (1.0f + expf(-g.o_gate[(size_t)(row / g.o_gate_div) * g.o_gate_ld + (size_t)(row % g.o_gate_div) * g.N + n]));
     if (BF && g.c_storage) ((uint16_t*)g.C)[i] = kr_f32_to_bf16(v);
     else g.C[i] = v;
 }
+
+// columns of group `group`: all N, or what the group's own matrix has
+__device__ __forceinline__ int gm_cols(const KrSvGemm& g, int group) { return g.n_last > 0 ? (group == g.n_groups - 1 ? g.n_last : g.n_first) : g.N; }
 
 // row tile `tile` of a grouped problem: walks the segment table; returns false past the last tile
 __device__ __forceinline__ bool gm_find_tile(const int* seg, int n_groups, int tile, int BM, int& group, int& m0, int& mend) {
@@ -58,14 +62,18 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
     constexpr int VEC = 16 / sizeof(T);
     const int lane = threadIdx.x & 63, n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * CN;
     if (n0 >= g.N) return;
-    int m0 = mbase, mcnt;
+    int m0 = mbase, mcnt, N = g.N;
     const T* W = (const T*)g.W;
-    if (g.row_group) { m0 = blockIdx.y; mcnt = 1; W += (size_t)g.row_group[m0] * g.w_stride; }
-    else mcnt = min(MB, g.M - m0);
+    if (g.row_group) {
+        m0 = blockIdx.y; mcnt = 1;
+        const int group = g.row_group[m0];
+        W += (size_t)group * g.w_stride; N = gm_cols(g, group);
+        if (n0 >= N) return;
+    } else mcnt = min(MB, g.M - m0);
     const T* wr[CN];
 #pragma unroll
-    for (int c = 0; c < CN; c++) wr[c] = W + (size_t)min(n0 + c, g.N - 1) * g.K;       // columns past N repeat the last one and are not stored
-    const T* ar[MB]; const float* gr[MB]; float gw[MB];
+    for (int c = 0; c < CN; c++) wr[c] = W + (size_t)min(n0 + c, N - 1) * g.K;       // columns past N repeat the last one and are not stored
+    const T* ar[MB]; const float* gr[MB]; float gw[MB]; const T* ur[MB];      // ur: rows of the table that holds the up factors
 #pragma unroll
     for (int m = 0; m < MB; m++) {
         const int r = min(m0 + m, g.M - 1);
@@ -73,8 +81,9 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
         ar[m] = ACT ? nullptr : (const T*)g.A + (size_t)src * g.lda;
         gr[m] = ACT ? g.act_gu + (size_t)src * g.act_ld : nullptr;
         gw[m] = ACT && g.act_row_w ? g.act_row_w[r] : 1.0f;
+        ur[m] = ACT && g.up_tab ? (const T*)g.up_tab + (size_t)g.up_rows[r] * g.up_ld + g.up_off : nullptr;
     }
-    const int uoff = g.act_kind == KR_SV_ACT_RELU2 ? 0 : g.K;     // an un-gated activation has no up columns: the second read repeats the first
+    const int uoff = g.act_kind == KR_SV_ACT_RELU2 || (ACT && g.up_tab) ? 0 : g.K;     // no up columns (un-gated, or taken from a table): the second read repeats the first
     float acc[MB][CN];
 #pragma unroll
     for (int m = 0; m < MB; m++)
@@ -94,7 +103,9 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
                     if constexpr (ACT) {
 #pragma unroll
                         for (int q = 0; q < VEC / 4; q++) {
-                            const float4 gg = *reinterpret_cast<const float4*>(gr[m] + k + 4 * q), uu = *reinterpret_cast<const float4*>(gr[m] + uoff + k + 4 * q);
+                            const float4 gg = *reinterpret_cast<const float4*>(gr[m] + k + 4 * q);
+                            float4 uu = *reinterpret_cast<const float4*>(gr[m] + uoff + k + 4 * q);
+                            if (ur[m]) uu = make_float4(gm_ld(ur[m] + k + 4 * q), gm_ld(ur[m] + k + 4 * q + 1), gm_ld(ur[m] + k + 4 * q + 2), gm_ld(ur[m] + k + 4 * q + 3));
                             af[4 * q] = gm_round<T>(gm_act(gg.x * gw[m], uu.x * gw[m], g.act_kind, g.act_limit, g.act_alpha)); af[4 * q + 1] = gm_round<T>(gm_act(gg.y * gw[m], uu.y * gw[m], g.act_kind, g.act_limit, g.act_alpha));
                             af[4 * q + 2] = gm_round<T>(gm_act(gg.z * gw[m], uu.z * gw[m], g.act_kind, g.act_limit, g.act_alpha)); af[4 * q + 3] = gm_round<T>(gm_act(gg.w * gw[m], uu.w * gw[m], g.act_kind, g.act_limit, g.act_alpha));
                         }
@@ -133,7 +144,7 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
             for (int m = 0; m < MB; m++) {
                 if (m < mcnt) {
                     float av;
-                    if constexpr (ACT) av = gm_round<T>(gm_act(gr[m][k] * gw[m], gr[m][uoff + k] * gw[m], g.act_kind, g.act_limit, g.act_alpha));
+                    if constexpr (ACT) av = gm_round<T>(gm_act(gr[m][k] * gw[m], (ur[m] ? gm_ld(ur[m] + k) : gr[m][uoff + k]) * gw[m], g.act_kind, g.act_limit, g.act_alpha));
                     else av = gm_ld(ar[m] + k);
 #pragma unroll
                     for (int c = 0; c < CN; c++) acc[m][c] = __builtin_fmaf(av, w[c], acc[m][c]);
@@ -148,7 +159,7 @@ __global__ void __launch_bounds__(256) sv_gemv_kernel(const KrSvGemm g, int mbas
             float v = acc[m][c];
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
-            if (lane == 0 && m < mcnt && n0 + c < g.N) gm_store<sizeof(T) == 2>(g, m0 + m, n0 + c, v);
+            if (lane == 0 && m < mcnt && n0 + c < N) gm_store<sizeof(T) == 2>(g, m0 + m, n0 + c, v);
         }
 }
 
@@ -158,7 +169,8 @@ __global__ void __launch_bounds__(256) sv_gemm_f32_kernel(const KrSvGemm g) {
     __shared__ float As[BK][BM + 4], Bs[BK][BN + 4];
     int group = 0, m0 = blockIdx.y * BM, mend = g.M;
     if (g.seg && !gm_find_tile(g.seg, g.n_groups, blockIdx.y, BM, group, m0, mend)) return;
-    const int n0 = blockIdx.x * BN;
+    const int n0 = blockIdx.x * BN, N = gm_cols(g, group);
+    if (n0 >= N) return;
     const float* A = (const float*)g.A;
     const float* W = (const float*)g.W + (size_t)group * g.w_stride;
     const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
@@ -166,7 +178,7 @@ __global__ void __launch_bounds__(256) sv_gemm_f32_kernel(const KrSvGemm g) {
     const int lr = tid >> 2, lk = (tid & 3) * 4;
     const int am = m0 + lr;
     const float* arow = am < mend ? A + (size_t)(g.a_rows ? g.a_rows[am] : am) * g.lda : nullptr;
-    const float* wrow = n0 + lr < g.N ? W + (size_t)(n0 + lr) * g.K : nullptr;
+    const float* wrow = n0 + lr < N ? W + (size_t)(n0 + lr) * g.K : nullptr;
     float acc[4][4];
 #pragma unroll
     for (int i = 0; i < 4; i++)
@@ -199,7 +211,7 @@ __global__ void __launch_bounds__(256) sv_gemm_f32_kernel(const KrSvGemm g) {
 #pragma unroll
         for (int j = 0; j < 4; j++) {
             const int n = n0 + tx * 4 + j;
-            if (n < g.N) gm_store<false>(g, m, n, acc[i][j]);
+            if (n < N) gm_store<false>(g, m, n, acc[i][j]);
         }
     }
 }
@@ -216,7 +228,8 @@ __global__ void __launch_bounds__(256) sv_gemm_bf16_kernel(const KrSvGemm g) {
     __shared__ __attribute__((aligned(16))) uint16_t Bs[BN * GM_LD];
     int group = 0, m0 = blockIdx.y * BM, mend = g.M;
     if (g.seg && !gm_find_tile(g.seg, g.n_groups, blockIdx.y, BM, group, m0, mend)) return;
-    const int n0 = blockIdx.x * BN;
+    const int n0 = blockIdx.x * BN, N = gm_cols(g, group);
+    if (n0 >= N) return;
     const uint16_t* A = (const uint16_t*)g.A;
     const uint16_t* W = (const uint16_t*)g.W + (size_t)group * g.w_stride;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 31, h = lane >> 5;
@@ -235,7 +248,7 @@ __global__ void __launch_bounds__(256) sv_gemm_bf16_kernel(const KrSvGemm g) {
     for (int i = 0; i < BCH; i++) {
         const int c = tid + i * 256, row = c / GM_KCH;
         bkc[i] = (c % GM_KCH) * 8;
-        bp[i] = n0 + row < g.N ? W + (size_t)(n0 + row) * g.K : nullptr;
+        bp[i] = n0 + row < N ? W + (size_t)(n0 + row) * g.K : nullptr;
     }
     auto load16 = [&](const uint16_t* p, int k) -> gu4 {
         gu4 v = {0u, 0u, 0u, 0u};
@@ -288,7 +301,7 @@ __global__ void __launch_bounds__(256) sv_gemm_bf16_kernel(const KrSvGemm g) {
 #pragma unroll
         for (int b = 0; b < 2; b++) {
             const int n = n0 + wc * 64 + b * 32 + r;
-            if (n >= g.N) continue;
+            if (n >= N) continue;
 #pragma unroll
             for (int i = 0; i < 16; i++) {
                 const int m = m0 + wr * (BM / 2) + a * 32 + (i & 3) + 8 * (i >> 2) + 4 * h;

@@ -27,6 +27,11 @@ struct KrSvGemm {
     const float* act_row_w;          // with act_gu: [M] or null, multiplies the gate and up columns of problem row r before the activation (a weight on the expert's input)
     // [*, o_gate_ld] f32 or null: an element of C is multiplied by sigmoid(o_gate[row / o_gate_div][(row % o_gate_div) * N + n]) before it is stored, row = its row in C
     const float* o_gate; int o_gate_ld, o_gate_div;
+    const float* bias;               // [N] f32 or null: joins every row of C before it is stored (or gated)
+    int n_last;                      // grouped, > 0: the last group's matrix has n_last rows (columns of C) instead of N; N is then the larger of the two
+    int n_first;                     //   ... and the other groups' matrices have n_first
+    // with act_gu: the up columns come from a table instead: element k of problem row r is up_tab[up_rows[r] * up_ld + up_off + k] (storage type)
+    const void* up_tab; const int* up_rows; int up_ld, up_off;
 };
 void kr_sv_gemm(const KrSvGemm& g, bool f32, hipStream_t st);
 bool kr_sv_gemm_small(const KrSvGemm& g);      // true: kr_sv_gemm takes the wave-per-column form for this problem (and honours act_gu)
@@ -85,6 +90,7 @@ struct KrSvAttn {
     const float* q_norm_w; const float* k_norm_w;   // [dim] each: unit_norm == 2 (weighted, before the rotation)
     float eps, scale;
     int window;                      // 0 = every earlier position
+    int keep;                        // > 0, with window: the first `keep` positions of the request are visible too
     int chunk;                       // > 0: only the keys of the query's own block of `chunk` positions (counted from position 0 of the request)
     const float* slopes;             // [heads] or null: score -= slopes[h] * (query position - key position)
     int v_mix; const float* v_lambda; float* v_first;   // 1: values also kept in v_first [T, kv_heads * vdim]; 2: v <- (1 - *v_lambda) v + *v_lambda v_first
@@ -131,7 +137,9 @@ void kr_sv_router_select(const float* z, int ld, int parts, const float* bias, i
 void kr_sv_moe_sort(const int* ids, int T, int top, int E, int* counts, int* seg, int* cursor, int* src_row, int* row_group, int* pair_pos, const float* wts, float* row_w,
                     hipStream_t st);
 // gu rows `ld` floats apart (gate at [0, F), up at [F, 2F)) -> y [M, F] storage type; row_w [M] or null: multiplies a row's gate and up columns first
-void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, const float* row_w, hipStream_t st);
+// up_tab: the up factor of (row r, column c) is up_tab[up_rows[r] * up_ld + up_off + c] (storage type) instead of gu's second half
+void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, const float* row_w, hipStream_t st, const void* up_tab = nullptr,
+               const int* up_rows = nullptr, int up_ld = 0, int up_off = 0);
 // y[t] = mix[t] + (dense[t] + shared[t] + sum_s wts[t][s] * rows[pair_pos[t][s]]) (null terms are skipped, null wts are ones); with post_w, y <- norm(y) * post_w (+ post_b);
 // x[t] += mult * y[t].  With h_out the NEW row goes there in the storage type by the same launch: normed with norm_w (+ norm_b) -- the next sublayer's
 // input -- or, without norm_w, as it is.
@@ -181,10 +189,15 @@ void kr_sv_head_rows(int T, int heads, int* seg, int* rows, int* group, hipStrea
 //   gla (4):   S_t = diag(a_t) S_(t-1) + k_t v_t^T, a_t = exp(log sigmoid(gz_t + gz_bias) * inv_tau) per key channel (gz [T, gz_ld], heads x dim)
 //   ssd (5):   S_t = exp(-exp(a_log_h) dt_t) S_(t-1) + dt_t k_t v_t^T with dt_t = softplus(dtz_t[h] + dt_bias[h]); q, k of head h are those of group
 //              h / qk_group (C and B), v the head's x; the skip term and everything after it belong to kr_sv_ssd_out
-// Kinds 4 and 5 read q, k, v through qsrc / ksrc / vsrc (rows src_ld floats apart); the scan form only.
+//   wkv (7):   o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T q_t, S_t = diag(exp(gz_t)) S_(t-1) + k_t v_t^T; gz holds log decays per key channel
+//   delta (8): S <- exp(tok_t.x) S_(t-1); u = tok_t.w (v_t - S^T k_t); S_t = S + k_t u^T, o_t = S_t^T q_t
+// Kinds 4, 5, 7 and 8 read q, k, v through qsrc / ksrc / vsrc (rows src_ld floats apart).
 struct KrSvLin {
-    int kind;                        // KR_SERVE_MIX_RETENTION (2) | KR_SERVE_MIX_MLSTM (3) | KR_SERVE_MIX_GLA (4) | KR_SERVE_MIX_SSD (5)
-    const float* qsrc; const float* ksrc; const float* vsrc; int src_ld, qk_group;      // kinds 4, 5
+    int kind;                        // KR_SERVE_MIX_RETENTION (2) | _MLSTM (3) | _GLA (4) | _SSD (5) | _WKV (7) | _DELTA (8)
+    const float* qsrc; const float* ksrc; const float* vsrc; int src_ld, qk_group;      // kinds 4, 5, 7, 8: heads h of a group of qk_group share one q and one k
+    const float* bonus;              // kind 7: [heads * dim]
+    int qkv_act;                     // kind 2: 1 = silu on q, k and v as they are read (kr_sv_lin_scan; the block launches take prepped rows)
+    const float* gate; int gate_ld, gate_act;      // kr_sv_lin_out: gate logits [T, gate_ld] (null: they stand behind v in z); gate_act 0: by kind, 1: silu, 2: sigmoid
     const float* gz; int gz_ld; const float* gz_bias; float inv_tau;                     // kind 4
     const float* dtz; int dtz_ld; const float* dt_bias; const float* a_log;              // kind 5
     int norm_shared;                 // norm_w is [vdim], shared by the heads
@@ -261,6 +274,38 @@ bool kr_sv_rglru_fits(int width, int blocks, int taps);
 void kr_sv_rglru_step(const KrSvRglru& a, bool f32, hipStream_t st);
 // portions of any length: chunk-local recurrences in parallel, a serial launch over the chunks, the outputs in parallel
 void kr_sv_rglru_portions(const KrSvRglru& a, bool f32, hipStream_t st);
+// ---- linear-recurrence mixers around their scans (kr_serve_linear.hip)
+// token shift: n inputs of one row, out[i][t] = h_t + (h_(t-1) - h_t) * mu[i] in the storage type; h of the token before the step's portion comes from state
+// [slots][width], zeros before position 0.  The launch also writes the tables of the grouped problem over the n inputs: seg [n + 1], group and c_rows [n * T];
+// rows of C are n - 1 per token side by side, then, behind (n - 1) T rows, the last input's with last_rows rows of C reserved for each.
+struct KrSvShift {
+    const float* h32; const float* mu; int n; const float* state;
+    const int* slot; const int* pos; int T, width;
+    void* out;
+    int* seg; int* group; int* c_rows; int last_rows;
+};
+void kr_sv_shift(const KrSvShift& a, bool f32, hipStream_t st);
+// out[t][c] = -exp(w0[c] + sum_r w2[c][r] tanh(z[t][r])): log decays, everything f32 (w2 [cols, rank] in the storage type)
+void kr_sv_wkv_decay(const float* z, int ld, const void* w2, bool f32, const float* w0, int T, int rank, int cols, float* out, hipStream_t st);
+// the gated delta rule before its recurrence: convolution and silu on q | k | v, unit vectors (q scaled), and per (token, head) tok = (log decay, 0, 0, write strength)
+struct KrSvDelta {
+    const float* z; int ld;          // [T, ld] f32: q [kv_heads * dim] | k [kv_heads * dim] | v [heads * vdim]
+    const float* bz; const float* az;   // logits of the write strength and of the decay, [T, ld] each
+    int heads, kv_heads, dim, vdim, taps;
+    const float* conv;               // [C, taps], C = 2 kv_heads dim + heads vdim, the last column is the current token's
+    const float* a_log; const float* dt_bias;
+    float* ring;                     // [slots][taps][C]: projected rows by position % taps
+    const int* slot; const int* pos; int T;
+    const int* ent_off; int n_entries;
+    int single;                      // every entry brings one token: the ring row is written by the same launch
+    float* out;                      // [T, C]
+    float4* tok;                     // [T, heads]
+};
+void kr_sv_delta_prep(const KrSvDelta& a, hipStream_t st);
+// lightning attention before the block launches: silu on the row block [q | k | v] in place, tok[t][h].x = log decay
+void kr_sv_lt_prep(float* z, int ld, int cols, const float* decay, int heads, float4* tok, int T, hipStream_t st);
+// out[t][c] = o[t] / rms(o[t]) * w[c] * sigmoid(gate[t][c]) * scale over the whole row of n
+void kr_sv_row_out(const float* o, int n, const float* w, const float* gate, int gate_ld, float eps, float scale, void* out, int out_ld, bool f32, int T, hipStream_t st);
 void kr_sv_argmax(const float* logits, int R, int vocab, int* out, hipStream_t st);
 // uniform values in [-amp, amp) from a counter hash of (seed, element); amp = 0 writes zeros
 void kr_sv_fill_uniform(void* p, bool f32, size_t n, uint64_t seed, float amp, hipStream_t st);

@@ -337,7 +337,10 @@ __global__ void __launch_bounds__(256) sv_attn_group_kernel(const KrSvAttn a) {
     for (int i = tid; i < RM * dim; i += 256) qs[i] = i < nr * dim ? q[i] * a.scale : 0.0f;
     __syncthreads();
     SV_STAMP(1);
-    const int lo = a.window > 0 ? max(0, p - a.window + 1) : (a.chunk > 0 ? p - p % a.chunk : 0);
+    int lo = a.window > 0 ? max(0, p - a.window + 1) : (a.chunk > 0 ? p - p % a.chunk : 0);
+    // kept first keys: their own leading blocks when the window has left them behind, else one contiguous range from 0
+    const int nck = a.keep > 0 && lo > a.keep ? (a.keep + 63) / 64 : 0;
+    if (a.keep > 0 && nck == 0) lo = 0;
     float slope[RM];
 #pragma unroll
     for (int r = 0; r < RM; r++) slope[r] = (a.slopes && r < nr) ? a.slopes[h0 + r] : 0.0f;
@@ -361,17 +364,17 @@ __global__ void __launch_bounds__(256) sv_attn_group_kernel(const KrSvAttn a) {
         }
     };
     // blocks of 64 keys: this workgroup's share [c0, c1) of the token's blocks (all of them when the launch is not split), block c by wave (c - c0) % 4
-    const int nch = (p - lo) / 64 + 1, cps = (nch + a.nsplit - 1) / a.nsplit;
+    const int nch = (p - lo) / 64 + 1 + nck, cps = (nch + a.nsplit - 1) / a.nsplit;
     const int c0 = sp * cps, c1 = min(nch, c0 + cps);
     for (int cb = c0 + wave; cb < c1; cb += 4) {
-        const int j0 = lo + 64 * cb;
+        const int j0 = cb < nck ? 64 * cb : lo + 64 * (cb - nck), jl = cb < nck ? a.keep - 1 : p;
         const int j = j0 + lane;
-        const bool live = j <= p;
-        const int jc = min(j, p);                            // lanes past the last key score it again; their weight is set to 0
+        const bool live = j <= jl;
+        const int jc = min(j, jl);                           // lanes past the last key score it again; their weight is set to 0
         const int prow = table[jc / a.page_tokens] * a.page_tokens + (jc % a.page_tokens);
         const T* k = kp + (size_t)prow * a.ldk + (size_t)g * dim;
         constexpr int U = 16 / VC;                           // keys whose value rows are requested together
-        const int nk = min(64, p - j0 + 1);
+        const int nk = min(64, jl - j0 + 1);
         float va[U][VC], vb[U][VC];
         auto fetch_v = [&](int jb, float (&vv)[U][VC]) {
 #pragma unroll
@@ -574,7 +577,9 @@ __global__ void __launch_bounds__(256) sv_attn_mfma_kernel(const KrSvAttn a) {
         const bool rv = tq_row >= base && tq_row < end;
         const int p_row = rv ? p0 + (tq_row - base) : -1;
         const int lo_row = a.window > 0 ? max(0, p_row - a.window + 1) : (a.chunk > 0 && rv ? p_row - p_row % a.chunk : 0);
-        const int hi = p0 + (end - base - 1), lo = a.window > 0 ? max(0, p0 - a.window + 1) : (a.chunk > 0 ? p0 - p0 % a.chunk : 0);
+        const int hi = p0 + (end - base - 1);
+        int lo = a.window > 0 ? max(0, p0 - a.window + 1) : (a.chunk > 0 ? p0 - p0 % a.chunk : 0);
+        const int keep_row = rv ? a.keep : 0;
         const float slope_row = (a.slopes && rv) ? a.slopes[h_row] : 0.0f;
         const int* table = a.page_table + (size_t)sl * a.table_ld;
         float q[DQ];
@@ -588,15 +593,18 @@ __global__ void __launch_bounds__(256) sv_attn_mfma_kernel(const KrSvAttn a) {
 #pragma unroll
         for (int d = 0; d < DB; d++) acc[d] = sv_f4{0.0f, 0.0f, 0.0f, 0.0f};
         constexpr int KEYS = 16 * NKB;
-        const int nch = (hi - lo) / KEYS + 1, cps = (nch + a.nsplit - 1) / a.nsplit, c0 = sp * cps, c1 = min(nch, c0 + cps);
+        // kept first keys: their own leading blocks when every row's window has left them behind, else one contiguous range from 0
+        const int nck = a.keep > 0 && lo > a.keep ? (a.keep + KEYS - 1) / KEYS : 0;
+        if (a.keep > 0 && nck == 0) lo = 0;
+        const int nch = (hi - lo) / KEYS + 1 + nck, cps = (nch + a.nsplit - 1) / a.nsplit, c0 = sp * cps, c1 = min(nch, c0 + cps);
         for (int cb = c0 + wave; cb < c1; cb += 4) {
-            const int j0 = lo + KEYS * cb;
+            const int j0 = cb < nck ? KEYS * cb : lo + KEYS * (cb - nck), jl = cb < nck ? a.keep - 1 : hi;
             // ---- S^T: NKB blocks of 16 keys
             sv_f4 st[NKB];
             int prow[NKB];
 #pragma unroll
             for (int kb = 0; kb < NKB; kb++) {
-                const int key = min(j0 + kb * 16 + row, hi);         // keys past the last one are fetched again and masked
+                const int key = min(j0 + kb * 16 + row, jl);         // keys past the last one are fetched again and masked
                 prow[kb] = table[key / a.page_tokens] * a.page_tokens + (key % a.page_tokens);
             }
 #pragma unroll
@@ -634,7 +642,7 @@ __global__ void __launch_bounds__(256) sv_attn_mfma_kernel(const KrSvAttn a) {
 #pragma unroll
                 for (int i = 0; i < 4; i++) {
                     const int key = j0 + kb * 16 + 4 * qd + i;
-                    const bool ok = rv && key <= p_row && key >= lo_row;
+                    const bool ok = rv && key <= min(p_row, jl) && (key >= lo_row || key < keep_row);
                     const float sc = a.softcap > 0.0f ? a.softcap * tanhf(st[kb][i] / a.softcap) : st[kb][i];
                     st[kb][i] = ok ? sc - slope_row * (float)(p_row - key) : -INFINITY;
                     cm = fmaxf(cm, st[kb][i]);
@@ -887,11 +895,11 @@ __global__ void __launch_bounds__(256) sv_moe_sort_small_kernel(const int* __res
 
 template <typename T>
 __global__ void sv_act_kernel(const float* __restrict__ gu, int ld, T* __restrict__ y, int M, int F, int kind, float limit, float alpha,
-                              const float* __restrict__ row_w) {
+                              const float* __restrict__ row_w, const T* __restrict__ up_tab, const int* __restrict__ up_rows, int up_ld, int up_off) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (size_t)M * F) return;
     const size_t r = i / F; const int c = (int)(i - r * F);
-    float g = gu[r * ld + c], u = kind == KR_SV_ACT_RELU2 ? 0.0f : gu[r * ld + F + c], v;
+    float g = gu[r * ld + c], u = kind == KR_SV_ACT_RELU2 ? 0.0f : up_tab ? sv_ld(up_tab + (size_t)up_rows[r] * up_ld + up_off + c) : gu[r * ld + F + c], v;
     if (row_w) { g *= row_w[r]; u *= row_w[r]; }
     if (kind == KR_SV_ACT_RELU2) {
         g = fmaxf(g, 0.0f); v = g * g;
@@ -1080,7 +1088,7 @@ template <int KIND, int DP>
 __global__ void __launch_bounds__(64) sv_lin_scan_kernel(const KrSvLin a) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     constexpr int TB = 8;
-    constexpr bool ML = KIND == 3, GLA = KIND == 4, SSD = KIND == 5;
+    constexpr bool ML = KIND == 3, GLA = KIND == 4, SSD = KIND == 5, WKV = KIND == 7, DELTA = KIND == 8;
     const int e = blockIdx.x, h = blockIdx.y, cb = blockIdx.z, lane = threadIdx.x;
     const int part = lane & 3, cl = lane >> 2, col = cb * 16 + cl;
     const int dim = a.dim, vdim = a.vdim, H = a.heads, ncb = (vdim + 15) / 16;
@@ -1099,11 +1107,13 @@ __global__ void __launch_bounds__(64) sv_lin_scan_kernel(const KrSvLin a) {
     }
     float m = (ML && !fresh) ? nmg[dim] : 0.0f;
     const float decay = KIND == 2 ? a.decay[h] : 0.0f;
-    float* qs = lds; float* ks = qs + TB * dimp; float* vs = ks + TB * dimp; float* gs = vs + TB * 16; float* as = gs + TB * 2;      // as [TB * dimp]: per-channel decays (gla)
+    float* qs = lds; float* ks = qs + TB * dimp; float* vs = ks + TB * dimp; float* gs = vs + TB * 16; float* as = gs + TB * 2;      // as [TB * dimp]: per-channel decays (gla, wkv)
+    float* us = as + TB * dimp;              // [dimp]: the current token's bonus (wkv)
+    if constexpr (WKV) for (int d = lane; d < dimp; d += 64) us[d] = d < dim ? a.bonus[(size_t)h * dim + d] : 0.0f;
     const int half = a.rot_dims / 2;
     for (int tb = t0; tb < t1; tb += TB) {
         const int nt = min(TB, t1 - tb);
-        if constexpr (GLA || SSD) {
+        if constexpr (GLA || SSD || WKV || DELTA) {
             const int hq = h / a.qk_group;
             for (int idx = lane; idx < nt * dimp; idx += 64) {
                 const int tt = idx / dimp, d = idx - tt * dimp;
@@ -1118,6 +1128,7 @@ __global__ void __launch_bounds__(64) sv_lin_scan_kernel(const KrSvLin a) {
                     }
                     as[idx] = al;
                 }
+                if constexpr (WKV) as[idx] = d < dim ? expf(a.gz[(size_t)(tb + tt) * a.gz_ld + (size_t)h * dim + d]) : 0.0f;
             }
             for (int idx = lane; idx < nt * 16; idx += 64) {
                 const int tt = idx >> 4, c = cb * 16 + (idx & 15);
@@ -1128,16 +1139,18 @@ __global__ void __launch_bounds__(64) sv_lin_scan_kernel(const KrSvLin a) {
                 const float dt = fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z)));                      // softplus
                 gs[2 * lane] = dt; gs[2 * lane + 1] = -expf(a.a_log[h]) * dt;
             }
+            if (DELTA && lane < nt) { const float4 tk = a.tok[(size_t)(tb + lane) * H + h]; gs[2 * lane] = tk.w; gs[2 * lane + 1] = tk.x; }
         } else {
+        auto in = [&](float v) { return a.qkv_act ? v / (1.0f + expf(-v)) : v; };
         for (int idx = lane; idx < nt * dimp; idx += 64) {
             const int tt = idx / dimp, d = idx - tt * dimp;
             const float* zr = a.z + (size_t)(tb + tt) * a.ld + (size_t)h * dim;
-            qs[idx] = d < dim ? zr[d] * a.q_scale : 0.0f;
-            ks[idx] = d < dim ? zr[(size_t)H * dim + d] * a.k_scale : 0.0f;
+            qs[idx] = d < dim ? in(zr[d]) * a.q_scale : 0.0f;
+            ks[idx] = d < dim ? in(zr[(size_t)H * dim + d]) * a.k_scale : 0.0f;
         }
         for (int idx = lane; idx < nt * 16; idx += 64) {
             const int tt = idx >> 4, c = cb * 16 + (idx & 15);
-            vs[idx] = c < vdim ? a.z[(size_t)(tb + tt) * a.ld + (size_t)2 * H * dim + (size_t)h * vdim + c] : 0.0f;
+            vs[idx] = c < vdim ? in(a.z[(size_t)(tb + tt) * a.ld + (size_t)2 * H * dim + (size_t)h * vdim + c]) : 0.0f;
         }
         if (ML && lane < nt) {
             const float* zg = a.z + (size_t)(tb + lane) * a.ld + (size_t)2 * H * dim + (size_t)2 * H * vdim;
@@ -1167,16 +1180,30 @@ __global__ void __launch_bounds__(64) sv_lin_scan_kernel(const KrSvLin a) {
                 const float ig = gs[2 * tt], fg = gs[2 * tt + 1];
                 const float mn = fmaxf(fg + m, ig);
                 av = expf(fg + m - mn); bv = expf(ig - mn); m = mn;
-            } else if constexpr (SSD) { bv = gs[2 * tt]; av = expf(gs[2 * tt + 1]); }
+            } else if constexpr (SSD || DELTA) { bv = gs[2 * tt]; av = expf(gs[2 * tt + 1]); }
             else { av = decay; bv = 1.0f; }
-            const float* ap = as + tt * dimp + part * dpr;
-            const float bvv = bv * v;
+            const float* ap = as + tt * dimp + part * dpr; const float* up = us + part * dpr;
+            float bvv = bv * v;
             float po = 0.0f, pn = 0.0f;
+            if constexpr (DELTA) {                 // the decayed state's value at k first: what is written is the rest of v
+                float pk = 0.0f;
+#pragma unroll
+                for (int r = 0; r < DP; r++) if (r < dpr) { S[r] *= av; pk = __builtin_fmaf(S[r], kp[r], pk); }
+                pk += __shfl_xor(pk, 1); pk += __shfl_xor(pk, 2);
+                bvv = bv * (v - pk); av = 1.0f;
+            }
 #pragma unroll
             for (int r = 0; r < DP; r++) {
                 if (r < dpr) {
                     const float kr = kp[r], qr = qp[r];
+                    if constexpr (WKV) {           // the read-out comes before the write
+                        const float kv = kr * bvv;
+                        po = __builtin_fmaf(__builtin_fmaf(up[r], kv, S[r]), qr, po);
+                        S[r] = __builtin_fmaf(ap[r], S[r], kv);
+                        continue;
+                    }
                     if constexpr (GLA) S[r] = __builtin_fmaf(kr, bvv, ap[r] * S[r]);
+                    else if constexpr (DELTA) S[r] = __builtin_fmaf(kr, bvv, S[r]);
                     else S[r] = __builtin_fmaf(kr, bvv, av * S[r]);
                     po = __builtin_fmaf(S[r], qr, po);
                     if constexpr (ML) { n[r] = __builtin_fmaf(bv, kr, av * n[r]); pn = __builtin_fmaf(n[r], qr, pn); }
@@ -1712,7 +1739,8 @@ template <typename T>
 __global__ void __launch_bounds__(64) sv_lin_out_kernel(const KrSvLin a, T* __restrict__ out) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x, vdim = a.vdim, H = a.heads;
     const float* o = a.o + ((size_t)t * H + h) * vdim;
-    const float* g = a.z + (size_t)t * a.ld + (size_t)2 * H * a.dim + (size_t)H * vdim + (size_t)h * vdim;
+    const float* g = a.gate ? a.gate + (size_t)t * a.gate_ld + (size_t)h * vdim : a.z + (size_t)t * a.ld + (size_t)2 * H * a.dim + (size_t)H * vdim + (size_t)h * vdim;
+    const bool sig = a.gate_act ? a.gate_act == 2 : a.kind == 3;
     float ss = 0.0f;
     for (int d = lane; d < vdim; d += 64) ss = __builtin_fmaf(o[d], o[d], ss);
     const float inv = 1.0f / sqrtf(sv_wave_sum(ss) / (float)vdim + a.eps);
@@ -1720,7 +1748,7 @@ __global__ void __launch_bounds__(64) sv_lin_out_kernel(const KrSvLin a, T* __re
         const float gz = g[d], sg = 1.0f / (1.0f + expf(-gz));
         float v = o[d] * inv;
         if (a.norm_w) v *= a.norm_w[a.norm_shared ? (size_t)d : (size_t)h * vdim + d];
-        sv_st(out + ((size_t)t * H + h) * vdim + d, v * (a.kind == 3 ? sg : gz * sg));
+        sv_st(out + ((size_t)t * H + h) * vdim + d, v * (sig ? sg : gz * sg));
     }
 }
 
@@ -1969,12 +1997,13 @@ void kr_sv_moe_sort(const int* ids, int T, int top, int E, int* counts, int* seg
     hipLaunchKernelGGL(sv_moe_fill_kernel, dim3((n + 255) / 256), dim3(256), 0, st, ids, n, top, seg, cursor, src_row, row_group, pair_pos, wts, row_w);
 }
 
-void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, const float* row_w, hipStream_t st) {
+void kr_sv_act(const float* gu, int ld, void* y, bool f32, int M, int F, int kind, float limit, float alpha, const float* row_w, hipStream_t st, const void* up_tab,
+               const int* up_rows, int up_ld, int up_off) {
     const size_t n = (size_t)M * F;
     if (n == 0) return;
     const dim3 grid((unsigned)((n + 255) / 256));
-    if (f32) hipLaunchKernelGGL(sv_act_kernel<float>, grid, dim3(256), 0, st, gu, ld, (float*)y, M, F, kind, limit, alpha, row_w);
-    else hipLaunchKernelGGL(sv_act_kernel<uint16_t>, grid, dim3(256), 0, st, gu, ld, (uint16_t*)y, M, F, kind, limit, alpha, row_w);
+    if (f32) hipLaunchKernelGGL(sv_act_kernel<float>, grid, dim3(256), 0, st, gu, ld, (float*)y, M, F, kind, limit, alpha, row_w, (const float*)up_tab, up_rows, up_ld, up_off);
+    else hipLaunchKernelGGL(sv_act_kernel<uint16_t>, grid, dim3(256), 0, st, gu, ld, (uint16_t*)y, M, F, kind, limit, alpha, row_w, (const uint16_t*)up_tab, up_rows, up_ld, up_off);
 }
 
 void kr_sv_residual_norm(const KrSvResidual& r, bool out_f32, hipStream_t st) {
@@ -2013,10 +2042,10 @@ void kr_sv_lin_scan(const KrSvLin& a, hipStream_t st) {
     if (a.T <= 0 || a.n_entries <= 0) return;
     const int dpr = (a.dim + 3) / 4;
     const dim3 grid(a.n_entries, a.heads, (a.vdim + 15) / 16);
-    const size_t lds = (size_t)((a.kind == 4 ? 3 : 2) * 8 * 4 * dpr + 8 * 16 + 8 * 2) * sizeof(float);
+    const size_t lds = (size_t)(((a.kind == 4 || a.kind == 7 ? 3 : 2) * 8 + 1) * 4 * dpr + 8 * 16 + 8 * 2) * sizeof(float);
 #define SV_LIN(K_, DP_) hipLaunchKernelGGL((sv_lin_scan_kernel<K_, DP_>), grid, dim3(64), lds, st, a)
 #define SV_LIN_D(K_) do { if (dpr <= 8) SV_LIN(K_, 8); else if (dpr <= 16) SV_LIN(K_, 16); else if (dpr <= 32) SV_LIN(K_, 32); else if (dpr <= 64) SV_LIN(K_, 64); else SV_LIN(K_, 128); } while (0)
-    if (a.kind == 3) SV_LIN_D(3); else if (a.kind == 4) SV_LIN_D(4); else if (a.kind == 5) SV_LIN_D(5); else SV_LIN_D(2);
+    if (a.kind == 3) SV_LIN_D(3); else if (a.kind == 4) SV_LIN_D(4); else if (a.kind == 5) SV_LIN_D(5); else if (a.kind == 7) SV_LIN_D(7); else if (a.kind == 8) SV_LIN_D(8); else SV_LIN_D(2);
 #undef SV_LIN_D
 #undef SV_LIN
 }

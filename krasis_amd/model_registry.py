@@ -90,6 +90,8 @@ class ServeModelSpec:
     embed_norm: int = 0                  # the embedding row is normed before the first layer
     bigram: Optional[Tuple[int, int, int]] = None      # (buckets, multiplier of the previous token, multiplier of the token): a hashed pair embedding joins the row
     logit_scale: float = 0.0             # 0: the logits as they are
+    pos_rows: int = 0                    # > 0: a learned row per position joins the embedding row; no request is longer
+    token_side: int = 0                  # > 0: every layer ends with a gated, normed projection of the token's own row of that many numbers for the layer
     row_of: Optional[Dict[str, int]] = None            # a design's own bookkeeping: which config layer / which pass a layer run stands for
     fit: Optional[Callable[["ServeModelSpec", Callable[[str], Tuple[int, ...]]], None]] = None      # completes sizes that only tensor shapes give (called with name -> shape before the store is made)
 
@@ -538,6 +540,93 @@ def ripupel_spec(cfg: dict) -> ServeModelSpec:
 
 
 register_architecture("Ripupel", ripupel_spec)
+
+
+# ---- Gasavik: pre-normed parallel layers x <- x + m (mixer(h) + ff(h)), h = RMS norm of x, followed by x <- x + m rms(W_proj (gelu(W_gate x) * e)) w with e the token's own
+# row for the layer.  The embedding is token row + position row, normed.  Three mixers.  'wkv': five inputs mixed with the previous token's, a decay per key channel
+# formed by a low-rank pair, a bonus for the current token.  'delta': grouped unit-vector keys after a short convolution, the gated delta rule.  'parallel': an attention
+# (biased projections, q / k norm, no rotation, window with kept first tokens, a sigmoid gate per head) and lightning attention side by side.  Feed-forward: SiLU-gated, with biases.
+def _gasavik_tensors(spec: ServeModelSpec) -> Iterator[Tuple[int, str, int, str]]:
+    yield -1, "embed", 0, "embed"
+    yield -1, "pos", 0, "pos"
+    yield -1, "embed_norm", 0, "embed.norm"
+    if spec.token_side:
+        yield -1, "side_embed", 0, "side.embed"
+    yield -1, "final_norm_w", 0, "final.norm"
+    yield -1, "head", 0, "head"
+    for i, l in enumerate(spec.layers):
+        p = f"l{i}"
+        yield i, "norm_w", 0, f"{p}.norm1"
+        if l.mixer_kind == S.MIX_WKV:
+            for index, n in enumerate("rkvgw"):
+                yield i, "wkv_mu", index, f"{p}.mix.mu.{n}"
+            for role, n in (("q", "r"), ("k", "k"), ("v", "v"), ("out_gate", "g"), ("decay_a1", "w1"), ("decay_a2", "w2"), ("decay_a2_b", "w0"), ("wkv_u", "u"), ("lin_norm", "norm"), ("o", "o")):
+                yield i, role, 0, f"{p}.mix.{n}"
+        elif l.mixer_kind == S.MIX_DELTA:
+            for role, n in (("q", "q"), ("k", "k"), ("v", "v"), ("q_conv", "q.conv"), ("k_conv", "k.conv"), ("v_conv", "v.conv"), ("delta_b", "b"), ("delta_a", "a"), ("ssd_a_log", "A_log"),
+                            ("ssd_dt_bias", "dt_bias"), ("out_gate", "g"), ("lin_norm", "norm"), ("o", "o")):
+                yield i, role, 0, f"{p}.mix.{n}"
+        else:
+            for role, n in (("q", "q"), ("k", "k"), ("v", "v"), ("q_bias", "q.b"), ("k_bias", "k.b"), ("v_bias", "v.b"), ("q_norm", "q.norm"), ("k_norm", "k.norm"), ("out_gate", "g"), ("o", "o")):
+                yield i, role, 0, f"{p}.mix.left.{n}"
+            for role, n in (("lt_q", "q"), ("lt_k", "k"), ("lt_v", "v"), ("lt_g", "g"), ("lt_norm", "norm"), ("lt_o", "o")):
+                yield i, role, 0, f"{p}.mix.right.{n}"
+            yield i, "lt_decay", 0, f"{p}.mix.right.decay"      # from config.json (spec.extra), not from the checkpoint
+        if l.mlp_kind == S.MLP_DENSE:
+            for r in ("gate", "up", "down"):
+                yield i, r, 0, f"{p}.mlp.{r}"
+                yield i, r + "_b", 0, f"{p}.mlp.{r}.b"
+        if spec.token_side:
+            for r in ("gate", "proj", "norm"):
+                yield i, "side_" + r, 0, f"{p}.side.{r}"
+
+
+def gasavik_spec(cfg: dict) -> ServeModelSpec:
+    layers: List[S.LayerSpec] = []
+    extra: Dict[str, np.ndarray] = {}
+    for i, lc in enumerate(cfg["layers"]):
+        kind, m = lc.get("type"), lc["mixer"]
+        if kind == "wkv":
+            # the rank of the decay's projection pair is the checkpoint's (w1: [rank, width]): gasavik_fit_checkpoint
+            l = S.LayerSpec(heads=int(m["heads"]), kv_heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["dim"]), mixer_kind=S.MIX_WKV, lin_norm_weight=1)
+        elif kind == "delta":
+            l = S.LayerSpec(heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), mixer_kind=S.MIX_DELTA,
+                            lin_norm_weight=2, proj_conv=int(m.get("conv") or 1))
+        elif kind == "parallel":
+            a, b = m["left"], m["right"]
+            mask = a.get("mask") or {}
+            l = S.LayerSpec(heads=int(a["heads"]), kv_heads=int(a.get("kv_heads", a["heads"])), dim=int(a["dim"]), vdim=int(a.get("vdim", a["dim"])), qk_unit_norm=S.QKNORM_WEIGHTED,
+                            scale=float(a["scale"]), window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0), proj_bias=3, out_gate=S.OGATE_HEAD_SIGMOID,
+                            side_mixer=S.MIX_LIGHTNING, lt_heads=int(b["heads"]), lt_dim=int(b["dim"]), lt_vdim=int(b.get("vdim", b["dim"])),
+                            # the store reads a weight of 0 as 1: a mixer weighted by zero gets one that vanishes beside anything
+                            mix_scale=float(m.get("left_scale", 1.0)) or 1e-30, side_scale=float(m.get("right_scale", 1.0)) or 1e-30)
+            dec = np.asarray(b["decay"], np.float32)
+            if dec.shape != (l.lt_heads,):
+                raise ValueError(f"layer {i}: {dec.size} decays for {l.lt_heads} heads")
+            extra[f"l{i}.mix.right.decay"] = dec
+        else:
+            raise ValueError(f"layer {i}: mixer type {kind!r} is not part of this design")
+        mlp = lc.get("mlp")
+        if mlp is not None:
+            if mlp.get("kind") != "dense":
+                raise ValueError(f"layer {i}: feed-forward kind {mlp.get('kind')!r}")
+            l.mlp_kind, l.ff, l.dense_act, l.ff_bias = S.MLP_DENSE, int(mlp["ff"]), S.ACT_SILU, 1
+        layers.append(l)
+    return ServeModelSpec(vocab=int(cfg["vocab"]), width=int(cfg["width"]), norm_kind=S.NORM_RMS, norm_eps=float(cfg["norm"]["eps"]), layers=layers, tensors=_gasavik_tensors,
+                          block_kind=S.BLOCK_PARALLEL, pre_norm=1, post_norm=0, norm_bias=0, residual_mult=float(cfg.get("residual_mult", 1.0)), extra=extra, embed_norm=1,
+                          pos_rows=int(cfg.get("max_positions") or 0), token_side=int((cfg.get("token_side") or {}).get("dim", 0)), fit=gasavik_fit_checkpoint)
+
+
+def gasavik_fit_checkpoint(spec: ServeModelSpec, shape_of: Callable[[str], Tuple[int, ...]]) -> None:
+    """sizes that only the checkpoint gives: the rank of a wkv layer's decay projections, the number of position rows when config.json does not say"""
+    for i, l in enumerate(spec.layers):
+        if l.mixer_kind == S.MIX_WKV and not l.decay_rank:
+            l.decay_rank = int(shape_of(f"l{i}.mix.w1")[0])
+    if not spec.pos_rows:
+        spec.pos_rows = int(shape_of("pos")[0])
+
+
+register_architecture("Gasavik", gasavik_spec)
 
 
 def read_config(model_dir: str) -> dict:

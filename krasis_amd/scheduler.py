@@ -34,7 +34,7 @@ class BatchEngine:
                                   max_slots=max_slots, pool_tokens=max_tokens, device=device, build=build, block_kind=spec.block_kind, pre_norm=spec.pre_norm,
                                   post_norm=spec.post_norm, norm_bias=spec.norm_bias, residual_mult=spec.residual_mult, norm_groups=spec.norm_groups,
                                   embed_scale=spec.embed_scale, canon_taps=spec.canon_taps, res_gate=spec.res_gate, norm_weight_offset=spec.norm_weight_offset,
-                                  embed_norm=spec.embed_norm, bigram=spec.bigram, logit_scale=spec.logit_scale)
+                                  embed_norm=spec.embed_norm, bigram=spec.bigram, logit_scale=spec.logit_scale, pos_rows=spec.pos_rows, token_side=spec.token_side)
         self.vocab = spec.vocab
         self._slot: Dict[object, int] = {}
 
@@ -135,6 +135,9 @@ class Scheduler:
         r = _Request(len(self._all), list(prompt), max_new_tokens, temperature, top_k, top_p, frozenset(stop_ids), seed)
         if self._pages(r) * self.engine.store.page_tokens > self.engine.store.pool_tokens:
             raise ValueError(f"request needs {self._pages(r)} pages; the pool holds {self.engine.store.pool_tokens // self.engine.store.page_tokens}")
+        limit = getattr(self.engine.store, "max_positions", None)
+        if limit and len(r.prompt) + max_new_tokens - 1 > limit:      # the last token sampled is not fed
+            raise ValueError(f"request needs {len(r.prompt) + max_new_tokens - 1} positions; the model has {limit}")
         self._all[r.rid] = r
         self._wait.append(r)
         return r.rid

@@ -17,7 +17,7 @@ NORM_LAYER, NORM_RMS = 0, 1
 MLP_NONE, MLP_DENSE, MLP_MOE = 0, 1, 2
 ACT_GELU_TANH, ACT_CLAMPED_SWIGLU, ACT_SILU, ACT_RELU2 = 0, 1, 2, 3
 BLOCK_PARALLEL, BLOCK_SEQUENTIAL = 0, 1
-MIX_ATTENTION, MIX_LATENT, MIX_RETENTION, MIX_MLSTM, MIX_GLA, MIX_SSD, MIX_RGLRU = 0, 1, 2, 3, 4, 5, 6
+MIX_ATTENTION, MIX_LATENT, MIX_RETENTION, MIX_MLSTM, MIX_GLA, MIX_SSD, MIX_RGLRU, MIX_WKV, MIX_DELTA, MIX_LIGHTNING = 0, 1, 2, 3, 4, 5, 6, 7, 8, 9
 QKNORM_NONE, QKNORM_AFTER_ROT, QKNORM_WEIGHTED, QKNORM_WHOLE = 0, 1, 2, 3
 RBIAS_NONE, RBIAS_LOGIT, RBIAS_CHOICE = 0, 1, 2
 RSCORE_SOFTMAX, RSCORE_SIGMOID = 0, 1
@@ -35,7 +35,9 @@ ROLES = {n: i for i, n in enumerate(["embed", "final_norm_w", "final_norm_b", "h
                                      "lin_norm", "lin_decay", "igate", "igate_b", "fgate", "fgate_b",
                                      "embed_norm", "bigram", "pre_add", "v_bias", "q_conv", "k_conv", "v_conv", "decay_a1", "decay_a2", "decay_a2_b",
                                      "ssd_in", "ssd_conv", "ssd_conv_b", "ssd_dt_bias", "ssd_a_log", "ssd_d", "ssd_norm", "ssd_o",
-                                     "rg_y", "rg_y_b", "rg_x", "rg_x_b", "rg_conv", "rg_conv_b", "rg_ra", "rg_ra_b", "rg_ri", "rg_ri_b", "rg_lam"])}
+                                     "rg_y", "rg_y_b", "rg_x", "rg_x_b", "rg_conv", "rg_conv_b", "rg_ra", "rg_ra_b", "rg_ri", "rg_ri_b", "rg_lam",
+                                     "pos", "side_embed", "side_gate", "side_proj", "side_norm", "gate_b", "up_b", "down_b", "wkv_mu", "wkv_u", "delta_b", "delta_a",
+                                     "lt_q", "lt_k", "lt_v", "lt_g", "lt_norm", "lt_o", "lt_decay"])}
 
 
 @dataclass
@@ -108,6 +110,11 @@ class LayerSpec:
     rg_blocks: int = 0
     rg_conv: int = 0
     rg_rate: float = 0.0
+    keep_first: int = 0                  # with window: the first positions of a request that stay visible
+    ff_bias: int = 0                     # biases on the dense feed-forward's three projections
+    lt_heads: int = 0                    # MIX_LIGHTNING, as the layer's mixer or as side_mixer
+    lt_dim: int = 0
+    lt_vdim: int = 0
 
 
 class ServeStore:
@@ -115,7 +122,7 @@ class ServeStore:
                  max_slots: int = 4, pool_tokens: int = 4096, page_tokens: int = PAGE_TOKENS, device: int = 0, build: bool = False,
                  block_kind: int = BLOCK_PARALLEL, pre_norm: int = 1, post_norm: int = 0, norm_bias: Optional[int] = None, residual_mult: float = 1.0,
                  norm_groups: int = 0, embed_scale: float = 0.0, canon_taps: int = 0, res_gate: int = 0, norm_weight_offset: float = 0.0, embed_norm: int = 0,
-                 bigram: Optional[Tuple[int, int, int]] = None, logit_scale: float = 0.0):
+                 bigram: Optional[Tuple[int, int, int]] = None, logit_scale: float = 0.0, pos_rows: int = 0, token_side: int = 0):
         self._lib = load_serve_library(build=build)
         self.vocab, self.width, self.layers, self.dtype = vocab, width, list(layers), dtype
         self.page_tokens = page_tokens
@@ -124,7 +131,8 @@ class ServeStore:
         if norm_bias is None:
             norm_bias = int(norm_kind == NORM_LAYER)
         cfg = ServeConfigC(vocab, width, len(self.layers), dtype, norm_kind, norm_eps, max_slots, page_tokens, pool_tokens, block_kind, pre_norm, post_norm, norm_bias,
-                           residual_mult, norm_groups, embed_scale, canon_taps, res_gate, norm_weight_offset, embed_norm, *(bigram or (0, 0, 0)), logit_scale)
+                           residual_mult, norm_groups, embed_scale, canon_taps, res_gate, norm_weight_offset, embed_norm, *(bigram or (0, 0, 0)), logit_scale, pos_rows, token_side)
+        self.max_positions = pos_rows or None       # a learned row per position: no request can be longer
         arr = (ServeLayerC * len(self.layers))()
         for i, l in enumerate(self.layers):
             for f in fields(LayerSpec):
