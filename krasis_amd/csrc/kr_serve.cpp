@@ -115,7 +115,7 @@ struct kr_serve {
     DevBuf ssd_z;                                         // the state-space mixer's rows in the block recurrence's layout [q | k | v] per head (prompt portions)
     DevBuf rg_ab, rg_agg, rg_start;                       // real-gated linear recurrence, portions: per token and per chunk of 64
     DevBuf qkv2, sconv, ga1, gz;                          // convolved q | k | v; convolved x | B | C; the gla decay's low-rank input (storage type) and logits
-    DevBuf mixes, sgate;                                 // wkv: the shifted inputs [5][T][width]; the token input's gate logits
+    DevBuf mixes, sgate, lin_aux;                                 // wkv: the shifted inputs [5][T][width]; the token input's gate logits
     DevBuf v_first;                                      // [T, kv_heads * vdim] f32: the values of the first value-mixing layer
     DevBuf lq_c, lq_2, lq_n, lq_e, att2, head_i;         // latent mixer: query latent, W_uq output, plain query parts, folded queries, per-head values, head row tables
     void* h_meta = nullptr; size_t h_meta_bytes = 0;     // pinned staging of the per-step arrays
@@ -1014,7 +1014,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
     const bool lin_chunked = max_count >= 32;
     // the gated linear recurrence: one launch when every entry brings one token, else chunks of 64 tokens
     const bool rg_step = max_count == 1;
-    size_t max_rg = 0; bool any_wkv = false;
+    size_t max_rg = 0, lin_aux = 0; bool any_wkv = false;
     for (const SvLayer& l : s->L) {
         const kr_serve_layer& d = l.d;
         if (d.proj_conv) max_pconv = std::max(max_pconv, (size_t)l.pconv_c());
@@ -1039,7 +1039,8 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         if (l.gla()) { max_ga1 = std::max(max_ga1, (size_t)d.decay_rank); max_gz = std::max(max_gz, (size_t)d.heads * d.dim); }
         if (l.recurrent()) {
             max_lin = std::max(max_lin, (size_t)d.heads * d.vdim);
-            if (lin_chunked && l.chunkable() && kr_sv_lin_chunked_fits(d.dim, d.vdim)) {
+            if (lin_chunked && ((l.chunkable() && kr_sv_lin_chunked_fits(d.dim, d.vdim)) || ((l.wkv() || l.delta()) && kr_sv_lin_blocks_fit(d.dim, d.vdim)))) {
+                if (l.delta()) lin_aux = std::max(lin_aux, (size_t)d.heads * d.dim);
                 lin_tok = std::max(lin_tok, (size_t)d.heads); lin_sb = std::max(lin_sb, (size_t)d.heads * d.dim * d.vdim); lin_nb = std::max(lin_nb, (size_t)d.heads * d.dim);
             }
         }
@@ -1076,6 +1077,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         return kr_fail(KR_ERR_HIP, "block scratch for %d tokens", T);
     if ((max_pconv && s->qkv2.ensure(Ts * max_pconv * 4)) || (max_sconv && s->sconv.ensure(Ts * max_sconv * 4)) || (max_ga1 && s->ga1.ensure(Ts * max_ga1 * s->esz)) || (max_gz && s->gz.ensure(Ts * max_gz * 4)))
         return kr_fail(KR_ERR_HIP, "convolution / decay scratch for %d tokens", T);
+    if (lin_aux && s->lin_aux.ensure(Ts * lin_aux * 4)) return kr_fail(KR_ERR_HIP, "delta rule scratch for %d tokens", T);
     if (max_rg && (s->rg_ab.ensure(Ts * max_rg * 8) || s->rg_agg.ensure((size_t)n_chunks * max_rg * 8) || s->rg_start.ensure((size_t)n_chunks * max_rg * 4)))
         return kr_fail(KR_ERR_HIP, "recurrence scratch for %d tokens", T);
     if (max_ssdz && s->ssd_z.ensure(Ts * max_ssdz * 4)) return kr_fail(KR_ERR_HIP, "state-space block scratch for %d tokens", T);
@@ -1232,6 +1234,8 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             {
                 Timer tm(s, 3);
                 if (lin_chunked && l.chunkable() && kr_sv_lin_chunked_fits(d.dim, d.vdim)) kr_sv_lin_chunked(q, st);
+                else if (lin_chunked && l.wkv() && kr_sv_lin_blocks_fit(d.dim, d.vdim)) kr_sv_lin_chan_blocks(q, st);
+                else if (lin_chunked && l.delta() && kr_sv_lin_blocks_fit(d.dim, d.vdim)) { q.aux = (float*)s->lin_aux.p; kr_sv_delta_blocks(q, st); }
                 else if (lin_chunked && kr_sv_lin_scan_wide_fits(q.kind, d.dim)) kr_sv_lin_scan_wide(q, st);
                 else kr_sv_lin_scan(q, st);
             }

@@ -219,6 +219,7 @@ struct KrSvLin {
     const int* ent_chunk0; int n_chunks;
     float4* tok;                     // [T, heads]: per token (u = F - m, w = b - F, g = exp(F + m_start - m), exp(-m)); F = log decay summed from the block's start
     float* sbuf; float* nbuf;        // [n_chunks, heads, dim, vdim] / [n_chunks, heads, dim]: state and normaliser at every block's start
+    float* aux;                      // kind 8: [T, heads * dim] (kr_sv_delta_blocks)
     float* cmeta;                    // [n_chunks, heads, 4]: a block's last F, its last prefix maximum of b - F, the running maximum at its start
 };
 // token by token, the state in registers: decode steps and short portions
@@ -232,6 +233,13 @@ bool kr_sv_lin_scan_wide_fits(int kind, int dim);
 void kr_sv_lin_scan_wide(const KrSvLin& a, hipStream_t st);
 bool kr_sv_lin_chunked_fits(int dim, int vdim);
 void kr_sv_lin_chunked(const KrSvLin& a, hipStream_t st);
+// the last of the block launches alone: outputs from sbuf, tok and the rows z (kinds 2 and 8; 8: heads share keys in groups of qk_group)
+void kr_sv_lin_block_out(const KrSvLin& a, hipStream_t st);
+// prompt portions of kinds 4 (a.gz = log decays) and 7 in blocks of 64 tokens: sbuf and nbuf as above, gz is overwritten with running sums
+bool kr_sv_lin_blocks_fit(int dim, int vdim);
+void kr_sv_lin_chan_blocks(const KrSvLin& a, hipStream_t st);
+// prompt portions of kind 8 in blocks of 64 tokens: sbuf, tok and aux are scratch, the value rows are overwritten; z / ld name the same rows as qsrc
+void kr_sv_delta_blocks(const KrSvLin& a, hipStream_t st);
 // the state-space recurrence (kind 5 fields of `a`) written as a retention with a decay per token: z_out [T, ldz] = per head [q = C | k = dt B | v = x] in
 // the recurrent mixers' layout, a.tok[t][head].x = the token's log decay.  Follow with kr_sv_lin_chunked on a kind-2 description with prepped = 1.
 void kr_sv_ssd_expand(const KrSvLin& a, float* z_out, int ldz, hipStream_t st);

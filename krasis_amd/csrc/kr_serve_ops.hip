@@ -1626,7 +1626,7 @@ template <bool ML, int DB>
 __global__ void __launch_bounds__(256) sv_lin_cout_kernel(const KrSvLin a) {
     extern __shared__ __attribute__((aligned(16))) float sl[];      // [32][lds] rows of the block's start state | [4 waves][dq][64] the waves' queries
     const int gc = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, kq = lane >> 4;
-    const int H = a.heads, dim = a.dim, vdim = a.vdim, dq = 4 * ((dim + 15) / 16), nct = (vdim + 15) / 16;
+    const int H = a.heads, dim = a.dim, vdim = a.vdim, dq = 4 * ((dim + 15) / 16);
     const int lds = ((vdim + 31) / 32) * 32 + 16;                   // rows 16 banks apart: the lanes of two neighbouring rows fall into distinct banks
     float* qs = sl + 32 * lds + (size_t)wave * dq * 64;             // this wave's queries, one word per (step, lane): a register file that loops can index
     int e = 0;
@@ -1636,7 +1636,8 @@ __global__ void __launch_bounds__(256) sv_lin_cout_kernel(const KrSvLin a) {
     const int trow = wave * 16 + r; const bool tv = trow < nt;
     const size_t tg = (size_t)tb + min(trow, nt - 1);
     const float4 me = a.tok[tg * H + h];
-    const float* zq = a.z + (size_t)h * dim; const float* zk = zq + (size_t)H * dim; const float* zv = a.z + (size_t)2 * H * dim + (size_t)h * vdim;
+    const int grp = a.qk_group > 1 ? a.qk_group : 1, hq = h / grp, Hq = H / grp;      // heads of a group share one query and one key
+    const float* zq = a.z + (size_t)hq * dim; const float* zk = zq + (size_t)Hq * dim; const float* zv = a.z + (size_t)2 * Hq * dim + (size_t)h * vdim;
     // the reduction index of a matrix instruction is spread over the four 16-lane groups: in step i lane group kq takes the key coordinate
     // d = 16 (i / 4) + 4 kq + i % 4, so that four steps of a lane are 16 contiguous bytes of a key row
     auto dof = [&](int i) { return 16 * (i >> 2) + 4 * kq + (i & 3); };
@@ -2096,6 +2097,10 @@ void kr_sv_lin_chunked(const KrSvLin& a, hipStream_t st) {
     const dim3 gs(a.n_entries, a.heads, (a.dim * a.vdim + (ml ? a.dim : 0) + 255) / 256);
     if (ml) hipLaunchKernelGGL(sv_lin_cscan_kernel<true>, gs, dim3(256), 0, st, a);
     else hipLaunchKernelGGL(sv_lin_cscan_kernel<false>, gs, dim3(256), 0, st, a);
+    kr_sv_lin_block_out(a, st);
+}
+void kr_sv_lin_block_out(const KrSvLin& a, hipStream_t st) {
+    const bool ml = a.kind == 3;
     const dim3 go(a.n_chunks, a.heads);
     const bool small = a.dim <= 64 && a.vdim <= 64;
     const size_t lds = ((size_t)32 * (((a.vdim + 31) / 32) * 32 + 16) + (size_t)4 * (4 * ((a.dim + 15) / 16)) * 64) * sizeof(float);
