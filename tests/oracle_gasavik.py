@@ -4,7 +4,10 @@ No cache, no state object, no code shared with the package: the recurrences are 
 the token shift as a shifted array, attention as a full score matrix with a mask.  `forward(cfg, w, tokens)` returns the logits of every position and the
 residual stream after every layer.  `w` maps checkpoint tensor names to float arrays; `cfg` is the dictionary of config.json.
 """
+import json
 import math
+import os
+import struct
 
 import numpy as np
 
@@ -203,3 +206,115 @@ def forward(cfg, w, tokens):
             x = x + m * token_side(cfg, w, i, tokens, x, eps)
         states.append(x.copy())
     return (rms_unit(x, eps) * w["final.norm"]) @ w["head"].T, states
+
+
+# ------------------------------------------------------------------------------------------------ configurations and weights of the tests
+def wkv(heads, dim, rank=4):
+    """rank: only the checkpoint's tensors show it"""
+    return {"type": "wkv", "mixer": {"heads": heads, "dim": dim}, "rank": rank}
+
+
+def delta(heads, kv_heads, dim, vdim, conv):
+    return {"type": "delta", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def parallel(heads, kv_heads, dim, vdim, size, keep_first, lt_heads, lt_dim, lt_vdim, scale=None, left_scale=0.7, right_scale=1.3, decay=None):
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5 if scale is None else scale}
+    if size:
+        left["mask"] = {"size": size, "keep_first": keep_first}
+    dec = [1.0 - 2.0 ** (-1.0 - 7.0 * (h + 1) / lt_heads) for h in range(lt_heads)] if decay is None else list(decay)
+    return {"type": "parallel", "mixer": {"left": left, "left_scale": left_scale, "right": {"heads": lt_heads, "dim": lt_dim, "vdim": lt_vdim, "decay": dec}, "right_scale": right_scale}}
+
+
+def dense(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def layer(mixer, mlp):
+    return {**mixer, "mlp": mlp}
+
+
+def make_config(width, vocab, layers, eps=1e-5, residual_mult=0.6, side=5, positions=1536):
+    cfg = {"architecture": "Gasavik", "vocab": vocab, "width": width, "norm": {"eps": eps}, "residual_mult": residual_mult, "max_positions": positions,
+           "layers": [{k: v for k, v in l.items() if k != "rank"} for l in layers], "_ranks": [l.get("rank", 0) for l in layers]}
+    if side:
+        cfg["token_side"] = {"dim": side}
+    return cfg
+
+
+def random_weights(cfg, seed):
+    rng = np.random.default_rng(seed)
+    W, V, out = cfg["width"], cfg["vocab"], {}
+
+    def mat(name, *shape, gain=1.0):
+        out[name] = (rng.standard_normal(shape) * gain / math.sqrt(shape[-1])).astype(np.float32)
+
+    def vec(name, *shape, mid=0.0, amp=0.2):
+        out[name] = (mid + amp * rng.standard_normal(shape)).astype(np.float32)
+    vec("embed", V, W, amp=0.8); vec("pos", cfg["max_positions"], W, amp=0.4)
+    vec("embed.norm", W, mid=1.0); vec("final.norm", W, mid=1.0)
+    mat("head", V, W)
+    ns = int((cfg.get("token_side") or {}).get("dim", 0))
+    if ns:
+        vec("side.embed", V, ns * len(cfg["layers"]), amp=1.0)
+    for i, lc in enumerate(cfg["layers"]):
+        p, m, f = f"l{i}.", lc["mixer"], lc.get("mlp")
+        q = p + "mix."
+        vec(p + "norm1", W, mid=1.0)
+        if lc["type"] == "wkv":
+            H, d, rank = m["heads"], m["dim"], cfg["_ranks"][i]
+            for n in "rkvgw":
+                out[q + "mu." + n] = rng.uniform(0.0, 1.0, W).astype(np.float32)
+            for n in "rkvg":
+                mat(q + n, H * d, W, gain=1.2)
+            mat(q + "w1", rank, W, gain=2.0); mat(q + "w2", H * d, rank); vec(q + "w0", H * d, mid=-2.0, amp=1.5); vec(q + "u", H, d, amp=0.8)
+            vec(q + "norm", H * d, mid=1.0); mat(q + "o", W, H * d)
+        elif lc["type"] == "delta":
+            H, G, d, dv, taps = (m[k] for k in ("heads", "kv_heads", "dim", "vdim", "conv"))
+            for n, rows in (("q", G * d), ("k", G * d), ("v", H * dv)):
+                mat(q + n, rows, W, gain=1.5)
+                out[q + n + ".conv"] = (rng.standard_normal((rows, taps)) * 0.6).astype(np.float32)
+            mat(q + "b", H, W, gain=2.0); mat(q + "a", H, W); vec(q + "A_log", H, mid=-1.0, amp=1.0); vec(q + "dt_bias", H, mid=-1.0, amp=1.0)
+            vec(q + "norm", dv, mid=1.0); mat(q + "g", H * dv, W); mat(q + "o", W, H * dv)
+        else:
+            a, b = m["left"], m["right"]
+            H, G, d, dv = (a[k] for k in ("heads", "kv_heads", "dim", "vdim"))
+            for n, rows in (("q", H * d), ("k", G * d), ("v", G * dv)):
+                mat(q + "left." + n, rows, W, gain=1.5); vec(q + "left." + n + ".b", rows)
+            vec(q + "left.q.norm", d, mid=1.5); vec(q + "left.k.norm", d, mid=1.5)
+            mat(q + "left.g", H, W); mat(q + "left.o", W, H * dv)
+            H, d, dv = (b[k] for k in ("heads", "dim", "vdim"))
+            for n, rows in (("q", H * d), ("k", H * d), ("v", H * dv), ("g", H * dv)):
+                mat(q + "right." + n, rows, W, gain=1.3)
+            vec(q + "right.norm", H * dv, mid=1.0); mat(q + "right.o", W, H * dv)
+        if f is not None:
+            for n, shape in (("gate", (f["ff"], W)), ("up", (f["ff"], W)), ("down", (W, f["ff"]))):
+                mat(p + "mlp." + n, *shape); vec(p + "mlp." + n + ".b", shape[0])
+        if ns:
+            mat(p + "side.gate", ns, W, gain=1.5); mat(p + "side.proj", W, ns); vec(p + "side.norm", W, mid=0.7)
+    return out
+
+
+def bf16_round(a):
+    """float32 -> the nearest bfloat16 (ties to even), back as float32"""
+    b = np.ascontiguousarray(a, np.float32).view(np.uint32).astype(np.uint64)
+    b = ((b + 0x7FFF + ((b >> 16) & 1)) >> 16) << 16
+    return b.astype(np.uint32).view(np.float32).reshape(np.shape(a))
+
+
+def write_checkpoint(path, cfg, W):
+    """config.json + model.safetensors with the weights as bfloat16 (the caller's oracle should use bf16_round of W)"""
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump({k: v for k, v in cfg.items() if not k.startswith("_")}, f)
+    header, blobs, at = {}, [], 0
+    for name, a in W.items():
+        raw = (np.ascontiguousarray(bf16_round(a), np.float32).view(np.uint32) >> 16).astype("<u2").tobytes()
+        header[name] = {"dtype": "BF16", "shape": list(np.shape(a)), "data_offsets": [at, at + len(raw)]}
+        blobs.append(raw); at += len(raw)
+    hj = json.dumps(header).encode()
+    hj += b" " * (-len(hj) % 8)
+    with open(os.path.join(path, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(hj))); f.write(hj)
+        for b in blobs:
+            f.write(b)
