@@ -347,9 +347,9 @@ def parse():
                          "sizes -- prompt pass and decode throughput, kernel-family times -- beside the closest model of the decode graph (GQA + softmax top-k MoE, INT4) at "
                          "the same sizes; prints its own JSON line")
     ap.add_argument("--arch-sizes", default="small,large", help="sizes of --arch-compare (ARCH_SIZES)")
-    ap.add_argument("--arch-design", default="lomutar", choices=["lomutar", "pamulix", "midisun", "lufozen", "ripupel"],
+    ap.add_argument("--arch-design", default="lomutar", choices=["lomutar", "pamulix", "midisun", "lufozen", "ripupel", "gasavik"],
                     help="which layer-described design --arch-compare measures: lomutar (beside the decode graph's GQA + MoE model), pamulix or midisun (beside "
-                         "Lomutar), lufozen (beside Midisun with a dense feed-forward), ripupel (beside Pamulix's latent layers and Midisun's retention) -- both on the batched serving store, at the same layer sizes")
+                         "Lomutar), lufozen (beside Midisun with a dense feed-forward), ripupel (beside Pamulix's latent layers and Midisun's retention), gasavik (beside Lufozen's parallel and gla layers and Midisun's retention) -- all on the batched serving store, at the same layer sizes")
     return ap.parse_args()
 
 
@@ -865,6 +865,89 @@ def arch_compare_ripupel(args):
             "retention_TFLOPs": L * ret_flops / (ms * 1e-3) / 1e12, "retention_frac_of_f32_matrix_peak": L * ret_flops / (ms * 1e-3) / 1e12 / F32_MATRIX_PEAK_TFLOPS,
             "retention_bytes_GBs": ret_bytes / (ms * 1e-3) / 1e9, "retention_frac_of_hbm_peak": ret_bytes / (ms * 1e-3) / 1e9 / HBM_PEAK_GBS})
         del eng; gc.collect()
+        out["sizes"][name] = res
+    flush_native_stdout()
+    print(json.dumps(out), flush=True)
+    return out
+
+
+def gasavik_serve_engine(z, kinds, ff):
+    """A Gasavik model with random bf16 weights on the batched serving store at the layer sizes z (ARCH_SIZES); kinds: one letter per layer, W = wkv (the size's heads, keys and
+    values of the head size, decay projections of rank 64), D = gated delta rule (half as many keys as value heads, four taps), P = attention (the size's heads and window,
+    four kept tokens) beside lightning attention (the size's heads, keys and values of the head size).  Every layer: a SiLU-gated feed-forward with biases of ff columns and a
+    token input of 256 numbers."""
+    from krasis_amd import model_registry as R, scheduler as SCH, serve_store as S
+    W, H, G, D, V, P = (z[c] for c in ("width", "heads", "kv_heads", "dim", "vocab", "prompt"))
+    mlp = dict(mlp_kind=S.MLP_DENSE, ff=ff, dense_act=S.ACT_SILU, ff_bias=1)
+    mk = {"W": lambda: S.LayerSpec(heads=H, kv_heads=H, dim=D, vdim=D, mixer_kind=S.MIX_WKV, lin_norm_weight=1, decay_rank=64, **mlp),
+          "D": lambda: S.LayerSpec(heads=H, kv_heads=H // 2, dim=D, vdim=D, mixer_kind=S.MIX_DELTA, lin_norm_weight=2, proj_conv=4, **mlp),
+          "P": lambda: S.LayerSpec(heads=H, kv_heads=G, dim=D, vdim=D, qk_unit_norm=S.QKNORM_WEIGHTED, scale=D ** -0.5, window=z["window"], keep_first=4, proj_bias=3,
+                                   out_gate=S.OGATE_HEAD_SIGMOID, side_mixer=S.MIX_LIGHTNING, lt_heads=H, lt_dim=D, lt_vdim=D, mix_scale=0.8, side_scale=1.1, **mlp)}
+    spec = R.ServeModelSpec(V, W, S.NORM_RMS, 1e-6, [mk[c]() for c in kinds], None, block_kind=S.BLOCK_PARALLEL, pre_norm=1, post_norm=0, norm_bias=0, residual_mult=0.5, embed_norm=1,
+                            pos_rows=2 * P, token_side=GASAVIK_SIDE)
+    eng = SCH.BatchEngine(spec, dtype="bfloat16", max_tokens=4 * (P + 256), max_slots=4)
+    eng.load_synthetic(seed=7, amp=1.0)
+    return eng
+
+
+GASAVIK_SIDE = 256
+
+
+def arch_compare_gasavik(args):
+    """The Gasavik design beside the designs of the store that come closest, all with random bf16 weights and a dense feed-forward of top x expert-ff columns at the layer
+    sizes of ARCH_SIZES: Lufozen's parallel layers (attention beside a state-space mixer) and gla layers (a decay per key channel) and Midisun's windowed attention and
+    retention.  Four Gasavik models per size: the mixed order wkv, delta, parallel, wkv (the throughput), and one mixer kind alone each (what its kernels reach).  Mixer flops
+    are the design's own: 4 x visible keys x dim per query for attention; per state element and token 4 (lightning, retention, state space), 5 (gla, wkv: the decay's product) or 6
+    (delta: the read at k) for the recurrences."""
+    import numpy as np
+    from krasis_amd import model_registry as R, scheduler as SCH, serve_store as S
+    out = {"metric": "arch_compare_gasavik_vs_lufozen_and_midisun", "unit": "tok/s", "sizes": {}}
+    for name in [x for x in args.arch_sizes.split(",") if x]:
+        z = ARCH_SIZES[name]; W, H, G, D, L, V, P = (z[c] for c in ("width", "heads", "kv_heads", "dim", "layers", "vocab", "prompt"))
+        ff = z["top"] * z["ff"]; SG = min(8, H); ns = GASAVIK_SIDE
+        res = {"shape": dict(z, token_side=ns), "dense_ff": ff}
+        windowed = 2.0 * 2 * H * D * sum(min(i + 1, z["window"]) for i in range(P))
+        causal = 2.0 * 2 * H * D * sum(i + 1 for i in range(P))
+        rec = 1.0 * P * H * D * D                                      # state elements x tokens of one recurrent layer
+        st = H * D * D
+        # per layer: (matrix elements a token is multiplied by, mixer flops, state elements)
+        lay = {"W": (5 * H * D * W + 64 * W + 3 * W * ff + 2 * ns * W, 5 * rec, st), "D": (H * D * W + 3 * H * D * W + 2 * H * W + 3 * W * ff + 2 * ns * W, 6 * rec, st),
+               "P": ((2 * H * D + 2 * G * D + H) * W + 5 * H * D * W + 3 * W * ff + 2 * ns * W, windowed + 4 * rec, st)}
+        luf = {"P": ((H * D + 2 * G * D) * W + (2 * H * D + 2 * SG * D + H) * W + W * 2 * H * D + 2 * W * ff, causal + 4 * rec, st), "G": (5 * H * D * W + 32 * W + 2 * W * ff, 5 * rec, st)}
+        mid = {"A": ((H * D + G * D + H) * W + W * H * D + 3 * W * ff + 2 * W * W, windowed, 0), "R": (5 * H * D * W + 3 * W * ff + 2 * W * W, 4 * rec, st)}
+
+        def price(eng, table, ran, batches):
+            m = serve_measure(eng, V, P, np.random.default_rng(3), decode_batches=batches)
+            fam = m["prefill_family_ms"]; w = sum(table[c][0] for c in ran); fl = sum(table[c][1] for c in ran); sts = sum(table[c][2] for c in ran)
+            r = {"layers": len(ran), "prefill": {"tok_s": P / m["prefill_s"], "ms": m["prefill_s"] * 1e3, "tokens": P, "family_ms": {n: round(v, 3) for n, v in zip(SERVE_FAMILIES, fam)},
+                                                 "gemm_family_frac_of_bf16_peak": 2.0 * P * (w + V * W / P) / (fam[1] * 1e-3) / 1e12 / F16_PEAK_TFLOPS,
+                                                 "mixer_family_TFLOPs": fl / (fam[3] * 1e-3) / 1e12, "mixer_frac_of_f32_matrix_peak": fl / (fam[3] * 1e-3) / 1e12 / F32_MATRIX_PEAK_TFLOPS}}
+            for B, d in m["decode"].items():
+                st_b = 2.0 * 4 * B * sts                               # the matrix states, read and written, f32
+                byts = 2.0 * (w + V * W) + st_b
+                r["decode_b%d" % B] = {"tok_s": B / d["s_per_step"], "ms_per_step": d["s_per_step"] * 1e3, "weight_and_state_bytes_per_step": byts,
+                                       "frac_of_hbm_peak": byts / d["s_per_step"] / 1e9 / HBM_PEAK_GBS, "family_ms": {n: round(v, 4) for n, v in zip(SERVE_FAMILIES, d["family_ms"])},
+                                       "gemm_family_frac_of_hbm_peak": (byts - st_b) / (d["family_ms"][1] * 1e-3) / 1e9 / HBM_PEAK_GBS, "state_bytes_per_step": st_b}
+            return r
+        order = "".join("WDPW"[i % 4] for i in range(L)) if L >= 3 else "DP"[:L]
+        for label, kinds in (("mixed_" + order, order), ("wkv_only", "W" * L), ("delta_only", "D" * L), ("parallel_only", "P" * L)):
+            eng = gasavik_serve_engine(z, kinds, ff)
+            res["gasavik_" + label] = price(eng, lay, kinds, (1, 4) if label.startswith("mixed") else (1,))
+            del eng; gc.collect()
+        for label, kind in (("parallel_only", "P"), ("gla_only", "G")):
+            eng, runs = lufozen_serve_engine(z, kind * L, ff)
+            res["lufozen_" + label] = price(eng, luf, kind * runs, (1,))
+            del eng; gc.collect()
+        mk = {"A": lambda: S.LayerSpec(heads=H, kv_heads=G, dim=D, vdim=D, qk_unit_norm=S.QKNORM_WHOLE, scale=D ** -0.5, window=z["window"], has_sink=S.SINK_TENSOR, dist_bias=1, proj_bias=1,
+                                       v_from_k=1, softcap=30.0, out_gate=S.OGATE_HEAD_SIGMOID, mlp_kind=S.MLP_DENSE, ff=ff, dense_act=S.ACT_SILU),
+              "R": lambda: S.LayerSpec(heads=H, kv_heads=H, dim=D, vdim=D, mixer_kind=S.MIX_RETENTION, rot_dims=D, rot_interleaved=0, rot_base=1e6, mlp_kind=S.MLP_DENSE, ff=ff, dense_act=S.ACT_SILU)}
+        for label, kinds in (("attention_only", "A" * L), ("retention_only", "R" * L)):
+            spec = R.ServeModelSpec(V, W, S.NORM_RMS, 1e-5, [mk[c]() for c in kinds], None, block_kind=S.BLOCK_SEQUENTIAL, pre_norm=1, post_norm=0, norm_bias=0, norm_groups=4, embed_scale=2.0,
+                                    canon_taps=4, res_gate=1)
+            eng = SCH.BatchEngine(spec, dtype="bfloat16", max_tokens=4 * (P + 256), max_slots=4)
+            eng.load_synthetic(seed=7, amp=1.0)
+            res["midisun_" + label] = price(eng, mid, kinds, (1, 4) if kinds[0] == "R" else (1,))
+            del eng; gc.collect()
         out["sizes"][name] = res
     flush_native_stdout()
     print(json.dumps(out), flush=True)
@@ -1829,7 +1912,8 @@ def main_multi(args, torch, dist, world, rank, local_rank):
 def main():
     args = parse()
     if args.arch_compare:
-        return {"pamulix": arch_compare_pamulix, "midisun": arch_compare_midisun, "lufozen": arch_compare_lufozen, "ripupel": arch_compare_ripupel}.get(args.arch_design, arch_compare)(args)
+        return {"pamulix": arch_compare_pamulix, "midisun": arch_compare_midisun, "lufozen": arch_compare_lufozen, "ripupel": arch_compare_ripupel,
+                "gasavik": arch_compare_gasavik}.get(args.arch_design, arch_compare)(args)
     import torch
     import torch.distributed as dist
 
