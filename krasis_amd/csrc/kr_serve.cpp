@@ -1177,6 +1177,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         }
         g.A = mixer_in; g.lda = W; g.W = l.hw.p; g.C = hz; g.ldc = l.n_h; g.M = T; g.N = seq ? l.n_qkv : l.n_h; g.K = W;
         g.bias = d.ff_bias ? (const float*)l.h_bias.p : nullptr;
+        if (l.has_lt()) { g.silu_lo = l.off_lt; g.silu_hi = l.off_lt + l.lt_cols(); }
         if (g.N > 0) { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
         const SvLayer& kvl = d.kv_from >= 0 ? s->L[d.kv_from] : run;
         KrSvAttn a{};
@@ -1344,17 +1345,16 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             { Timer tm(s, 2); kr_sv_ssd_out(so, s->f32, st); }
         }
         if (l.has_lt()) {
-            // [q | k | v | g] came out of the layer's one GEMM; a retention on silu'd rows, then one norm over the heads laid side by side
+            // [q | k | v | g] came out of the layer's one GEMM, q, k, v through silu; a retention on them, then one norm over the heads laid side by side
             float* zin = hz + l.off_lt;
             KrSvLin q{};
             q.kind = KR_SERVE_MIX_RETENTION; q.z = zin; q.ld = l.n_h; q.heads = d.lt_heads; q.dim = d.lt_dim; q.vdim = d.lt_vdim; q.q_scale = q.k_scale = 1.0f; q.decay = (const float*)l.lt_decay.p;
-            q.qkv_act = 1; q.state = (float*)run.lt_state.p; q.state_stride = l.lt_state_stride; q.ent_off = d_eoff; q.ent_slot = d_eslot; q.n_entries = n_entries; q.pos = d_pos; q.T = T;
+            q.state = (float*)run.lt_state.p; q.state_stride = l.lt_state_stride; q.ent_off = d_eoff; q.ent_slot = d_eslot; q.n_entries = n_entries; q.pos = d_pos; q.T = T;
             q.o = (float*)s->lin_o.p; q.ent_chunk0 = d_echunk; q.n_chunks = n_chunks; q.tok = (float4*)s->lin_tok.p; q.sbuf = (float*)s->lin_sbuf.p; q.nbuf = (float*)s->lin_nbuf.p; q.cmeta = (float*)s->lin_cm.p;
             {
                 Timer tm(s, 3);
                 if (lin_chunked && kr_sv_lin_chunked_fits(d.lt_dim, d.lt_vdim)) {
-                    kr_sv_lt_prep(zin, l.n_h, l.lt_cols(), q.decay, d.lt_heads, q.tok, T, st);
-                    q.prepped = 1; kr_sv_lin_chunked(q, st);
+                    q.prepped = 2; kr_sv_lin_chunked(q, st);
                 } else kr_sv_lin_scan(q, st);
             }
             Timer tm(s, 2);

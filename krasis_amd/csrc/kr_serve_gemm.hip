@@ -25,6 +25,7 @@ __device__ __forceinline__ void gm_store(const KrSvGemm& g, int m, int n, float 
     const int row = g.c_rows ? g.c_rows[m] : m;
     const size_t i = (size_t)row * g.ldc + n;
     if (g.bias) v += g.bias[n];
+    if (n >= g.silu_lo && n < g.silu_hi) v = v / (1.0f + expf(-v));
     if (g.o_gate) v *= 1.0f / (1.0f + expf(-g.o_gate[(size_t)(row / g.o_gate_div) * g.o_gate_ld + (size_t)(row % g.o_gate_div) * g.N + n]));
     if (BF && g.c_storage) ((uint16_t*)g.C)[i] = kr_f32_to_bf16(v);
     else g.C[i] = v;
@@ -50,7 +51,8 @@ __device__ __forceinline__ float gm_act(float g, float u, int kind, float limit,
     if (kind == KR_SV_ACT_RELU2) { g = fmaxf(g, 0.0f); return g * g; }
     if (kind == KR_SV_ACT_GELU_TANH) return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
     if (kind == KR_SV_ACT_CLAMPED_SWIGLU) { g = fminf(g, limit); u = fminf(fmaxf(u, -limit), limit); return g / (1.0f + expf(-alpha * g)) * (u + 1.0f); }
-    return g / (1.0f + expf(-g)) * u;
+    // silu on the hardware exponential and reciprocal (one ulp each): every wave of a decode step's down projection forms it again
+    return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * g)) * u;
 }
 template <typename T> __device__ __forceinline__ float gm_round(float v) { return v; }
 template <> __device__ __forceinline__ float gm_round<uint16_t>(float v) { return kr_bf16_to_f32(kr_f32_to_bf16(v)); }

@@ -1,5 +1,6 @@
 // kr_serve_linear.hip -- linear-recurrence mixers of the batched serving step around their scans (gfx950, wave64): the token shift and the decays of the wkv mixer,
-// the preparation of the gated delta rule (convolution, unit vectors, gates), lightning attention's preparation and output norm.
+// the preparation of the gated delta rule (convolution, unit vectors, gates), lightning attention's output norm, and the block forms of
+// both recurrences for prompt portions.
 // Everything is f32 but the storage-type inputs and outputs of the projections.
 #include <hip/hip_runtime.h>
 #include <math.h>
@@ -20,23 +21,52 @@ __device__ __forceinline__ float ln_wave_sum(float v) {
     return v;
 }
 
-// ---- wkv: the n shifted inputs of a token (KrSvShift): one thread per (token, channel)
-template <typename T>
+// ---- wkv: the n shifted inputs of a token (KrSvShift): a thread per VC channels of TT consecutive tokens
+template <typename T, int VC, int TT>
 __global__ void __launch_bounds__(256) ln_shift_kernel(const KrSvShift a, T* __restrict__ out) {
-    const int t = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
-    if (blockIdx.y == 0 && (int)threadIdx.x < a.n) {        // the grouped problem's tables
-        const int i = threadIdx.x, r = i * a.T + t;
-        a.group[r] = i;
-        a.c_rows[r] = i < a.n - 1 ? t * (a.n - 1) + i : (a.n - 1) * a.T + t * a.last_rows;
-        if (t == 0) { a.seg[i] = i * a.T; if (i == 0) a.seg[a.n] = a.n * a.T; }
+    const int t0 = blockIdx.x * TT, c = (blockIdx.y * 256 + threadIdx.x) * VC;
+    if (blockIdx.y == 0) {                                  // the grouped problem's tables
+        for (int i = threadIdx.x; i < a.n * TT; i += 256) {
+            const int t = t0 + i / a.n, k = i % a.n;
+            if (t >= a.T) break;
+            a.group[k * a.T + t] = k;
+            a.c_rows[k * a.T + t] = k < a.n - 1 ? t * (a.n - 1) + k : (a.n - 1) * a.T + t * a.last_rows;
+        }
+        if (t0 == 0 && (int)threadIdx.x <= a.n) a.seg[threadIdx.x] = threadIdx.x * a.T;
     }
     if (c >= a.width) return;
-    const int p = a.pos[t], sl = a.slot[t];
-    const float h = a.h32[(size_t)t * a.width + c];
-    float prev = 0.0f;
-    if (p > 0) prev = (t > 0 && a.slot[t - 1] == sl) ? a.h32[(size_t)(t - 1) * a.width + c] : a.state[(size_t)sl * a.width + c];
-    const float d = prev - h;
-    for (int i = 0; i < a.n; i++) ln_st(out + ((size_t)i * a.T + t) * a.width + c, __builtin_fmaf(d, a.mu[(size_t)i * a.width + c], h));
+    float h[TT + 1][VC];                                    // h[0]: the token before t0
+    auto load = [&](const float* p, float* v) {
+        if constexpr (VC == 4) { const float4 x = *reinterpret_cast<const float4*>(p); v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w; }
+        else v[0] = *p;
+    };
+#pragma unroll
+    for (int i = 0; i <= TT; i++) load(a.h32 + (size_t)min(max(t0 + i - 1, 0), a.T - 1) * a.width + c, h[i]);
+    float prev[TT][VC];
+#pragma unroll
+    for (int i = 0; i < TT; i++) {
+        const int t = min(t0 + i, a.T - 1), sl = a.slot[t];
+        const bool own = t > 0 && a.slot[t - 1] == sl, first = a.pos[t] == 0;      // the token before: a row of this step, nothing, or the request's state
+#pragma unroll
+        for (int k = 0; k < VC; k++) prev[i][k] = first ? 0.0f : h[i][k];
+        if (!own && !first) load(a.state + (size_t)sl * a.width + c, prev[i]);
+    }
+    for (int n = 0; n < a.n; n++) {
+        float mu[VC];
+        load(a.mu + (size_t)n * a.width + c, mu);
+#pragma unroll
+        for (int i = 0; i < TT; i++) {
+            if (t0 + i >= a.T) break;
+            T* o = out + ((size_t)n * a.T + t0 + i) * a.width + c;
+            float v[VC];
+#pragma unroll
+            for (int k = 0; k < VC; k++) v[k] = __builtin_fmaf(prev[i][k] - h[i + 1][k], mu[k], h[i + 1][k]);
+            if constexpr (VC == 4 && sizeof(T) == 2) {
+                *reinterpret_cast<uint2*>(o) = make_uint2((uint32_t)kr_f32_to_bf16(v[0]) | ((uint32_t)kr_f32_to_bf16(v[1]) << 16), (uint32_t)kr_f32_to_bf16(v[2]) | ((uint32_t)kr_f32_to_bf16(v[3]) << 16));
+            } else if constexpr (VC == 4) *reinterpret_cast<float4*>(o) = make_float4(v[0], v[1], v[2], v[3]);
+            else ln_st(o, v[0]);
+        }
+    }
 }
 
 // log decays of TT tokens x 256 channels: tanh of the low-rank rows in LDS, a channel's weights through registers, sixteen ranks at a time
@@ -93,39 +123,79 @@ __global__ void __launch_bounds__(256) ln_wkv_decay_kernel(const float* __restri
     for (int tt = 0; tt < TT; tt++) if (t0 + tt < T_) out[(size_t)(t0 + tt) * cols + c] = -expf(acc[tt] + b);
 }
 
-// ---- gated delta rule: one wave per (token, q / k / v head).  The head's channels stay in registers (channel = lane + 64 i)
+// ---- gated delta rule: one wave per (TT consecutive tokens, q / k / v head); channel = lane + 64 i of the head.  NT > 0: that many taps, whose rows pass through
+// registers (a row is read once for all the tokens it reaches); NT = 0: any number, read again for every token.
+template <int NT, int TT>
 __global__ void __launch_bounds__(64) ln_delta_prep_kernel(const KrSvDelta a) {
-    const int t = blockIdx.x, y = blockIdx.y, lane = threadIdx.x, G = a.kv_heads;
+    const int t0 = blockIdx.x * TT, y = blockIdx.y, lane = threadIdx.x, G = a.kv_heads;
     const bool isv = y >= 2 * G;
     const int n = isv ? a.vdim : a.dim, c0 = isv ? 2 * G * a.dim + (y - 2 * G) * a.vdim : y * a.dim, C = 2 * G * a.dim + a.heads * a.vdim;
-    const int p = a.pos[t], sl = a.slot[t], taps = a.taps;
-    float v[8], ss = 0.0f;
+    const int taps = NT ? NT : a.taps;
+    float ss[TT];
 #pragma unroll
-    for (int i = 0; i < 8; i++) {
-        const int d = lane + 64 * i;
-        v[i] = 0.0f;
-        if (d < n) {
-            const int c = c0 + d;
-            const float* w = a.conv + (size_t)c * taps;
-            const float u0 = a.z[(size_t)t * a.ld + c];
-            float acc = w[taps - 1] * u0;
-            for (int b = 1; b < taps; b++) {      // b positions back
-                if (p - b < 0) break;
-                const float u = (t - b >= 0 && a.slot[t - b] == sl) ? a.z[(size_t)(t - b) * a.ld + c] : a.ring[((size_t)sl * taps + (p - b) % taps) * C + c];
-                acc = __builtin_fmaf(w[taps - 1 - b], u, acc);
+    for (int i = 0; i < TT; i++) ss[i] = 0.0f;
+    float* o = a.out + (size_t)t0 * C + c0;
+    for (int d = lane; d < n; d += 64) {
+        const int c = c0 + d;
+        const float* w = a.conv + (size_t)c * taps;
+        const float* zc = a.z + c;
+        if constexpr (NT > 0) {
+            float wt[NT], u[TT + NT - 1];                       // u[i]: row t0 - (NT - 1) + i of the step
+#pragma unroll
+            for (int b = 0; b < NT; b++) wt[b] = w[b];
+#pragma unroll
+            for (int i = 0; i < TT + NT - 1; i++) u[i] = zc[(size_t)min(max(t0 + i - (NT - 1), 0), a.T - 1) * a.ld];
+#pragma unroll
+            for (int i = 0; i < TT; i++) {
+                const int t = t0 + i, tc = min(t, a.T - 1), p = a.pos[tc], sl = a.slot[tc];
+                float r[NT];                                    // r[b]: b positions back
+#pragma unroll
+                for (int b = 0; b < NT; b++) {
+                    r[b] = u[i + NT - 1 - b];
+                    if (b > 0) {
+                        const bool own = tc - b >= 0 && a.slot[max(tc - b, 0)] == sl;
+                        if (p - b < 0) r[b] = 0.0f;
+                        else if (!own) r[b] = a.ring[((size_t)sl * NT + (p - b) % NT) * C + c];
+                    }
+                }
+                float acc = wt[NT - 1] * r[0];
+#pragma unroll
+                for (int b = 1; b < NT; b++) acc = __builtin_fmaf(wt[NT - 1 - b], r[b], acc);
+                if (t >= a.T) break;
+                if (a.single && NT > 1) a.ring[((size_t)sl * NT + p % NT) * C + c] = r[0];
+                const float v = acc / (1.0f + expf(-acc));
+                ss[i] = __builtin_fmaf(v, v, ss[i]);
+                o[(size_t)i * C + d] = v;
             }
-            if (a.single && taps > 1) a.ring[((size_t)sl * taps + p % taps) * C + c] = u0;
-            v[i] = acc / (1.0f + expf(-acc));
-            ss = __builtin_fmaf(v[i], v[i], ss);
+        } else {
+#pragma unroll
+            for (int i = 0; i < TT; i++) {
+                const int t = t0 + i;
+                if (t >= a.T) break;
+                const int p = a.pos[t], sl = a.slot[t];
+                const float u0 = zc[(size_t)t * a.ld];
+                float acc = w[taps - 1] * u0;
+                for (int b = 1; b < taps && p - b >= 0; b++) {
+                    const float u = (t - b >= 0 && a.slot[t - b] == sl) ? zc[(size_t)(t - b) * a.ld] : a.ring[((size_t)sl * taps + (p - b) % taps) * C + c];
+                    acc = __builtin_fmaf(w[taps - 1 - b], u, acc);
+                }
+                if (a.single) a.ring[((size_t)sl * taps + p % taps) * C + c] = u0;
+                const float v = acc / (1.0f + expf(-acc));
+                ss[i] = __builtin_fmaf(v, v, ss[i]);
+                o[(size_t)i * C + d] = v;
+            }
         }
     }
-    float sc = 1.0f;
-    if (!isv) { sc = 1.0f / sqrtf(ln_wave_sum(ss) + 1e-6f); if (y < G) sc *= 1.0f / sqrtf((float)a.dim); }
-    float* o = a.out + (size_t)t * C + c0;
+    if (!isv) {
+        const float qs = y < G ? 1.0f / sqrtf((float)a.dim) : 1.0f;
 #pragma unroll
-    for (int i = 0; i < 8; i++) { const int d = lane + 64 * i; if (d < n) o[d] = v[i] * sc; }
-    if (isv && lane == 0) {
-        const int h = y - 2 * G;
+        for (int i = 0; i < TT; i++) {
+            if (t0 + i >= a.T) break;
+            const float sc = qs / sqrtf(ln_wave_sum(ss[i]) + 1e-6f);
+            for (int d = lane; d < n; d += 64) o[(size_t)i * C + d] *= sc;      // a lane's own words
+        }
+    } else if (lane < TT && t0 + lane < a.T) {
+        const int h = y - 2 * G, t = t0 + lane;
         const float zb = a.bz[(size_t)t * a.ld + h], za = a.az[(size_t)t * a.ld + h] + a.dt_bias[h];
         const float sp = fmaxf(za, 0.0f) + log1pf(expf(-fabsf(za)));      // softplus
         a.tok[(size_t)t * a.heads + h] = make_float4(-expf(a.a_log[h]) * sp, 0.0f, 0.0f, 1.0f / (1.0f + expf(-zb)));
@@ -139,12 +209,7 @@ __global__ void __launch_bounds__(256) ln_delta_save_kernel(const KrSvDelta a) {
     a.ring[((size_t)a.slot[t] * a.taps + a.pos[t] % a.taps) * C + c] = a.z[(size_t)t * a.ld + c];
 }
 
-// ---- lightning attention
-__global__ void __launch_bounds__(256) ln_lt_prep_kernel(float* __restrict__ z, int ld, int cols, const float* __restrict__ decay, int heads, float4* __restrict__ tok) {
-    const size_t t = blockIdx.x; const int c = blockIdx.y * 256 + threadIdx.x;
-    if (c < heads) tok[t * heads + c] = make_float4(fmaxf(logf(decay[c]), -1.0e4f), 0.0f, 0.0f, 0.0f);
-    if (c < cols) { const float v = z[t * ld + c]; z[t * ld + c] = v / (1.0f + expf(-v)); }
-}
+// ---- lightning attention: the heads side by side as one row
 template <typename T>
 __global__ void __launch_bounds__(256) ln_row_out_kernel(const float* __restrict__ o, int n, const float* __restrict__ w, const float* __restrict__ gate, int gate_ld, float eps, float scale,
                                                          T* __restrict__ out, int out_ld) {
@@ -241,46 +306,65 @@ __global__ void __launch_bounds__(256) ln_chan_scan_kernel(const KrSvLin a) {
     *Sg = S;
 }
 // (3) in parallel over (block, head), wave w = sub-block w: both products transposed (S^T[s][t] = K Q^T, O^T[c][t] = V^T P^T) so that the weights meet the values where the
-// first product left them.  The wave's queries live in LDS, one word per (step, lane), and collect the decays of the sub-blocks they pass on the way back.
-template <int DB, bool WKV>
+// first product left them.  The wave's queries stay in registers and collect the decays of the sub-blocks they pass on the way back.
+template <int DT, int DB, bool WKV>
 __global__ void __launch_bounds__(256) ln_chan_out_kernel(const KrSvLin a) {
+    constexpr int DP = DT * 16, LK = DP + 4, LS = DB * 16 + 16;
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int gc = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, kq = lane >> 4;
-    const int H = a.heads, dim = a.dim, vdim = a.vdim, dimp = ((dim + 15) / 16) * 16, dq = dimp / 4, LK = dimp + 4, LS = ((vdim + 31) / 32) * 32 + 16;
-    float* kd = lds; float* tot = kd + 64 * LK; float* et = tot + 4 * dimp; float* sl = et + 4 * dimp; float* qs = sl + 32 * LS + (size_t)wave * dq * 64;
+    const int H = a.heads, dim = a.dim, vdim = a.vdim;
+    float* tot = lds; float* et = tot + 4 * DP; float* kd = et + 4 * DP; float* sl = kd;      // [4][DP] twice, [64][LK], later [32][LS] rows of the block's start state
     const int e = ln_entry_of(a, gc), tb = a.ent_off[e] + 64 * (gc - a.ent_chunk0[e]), nt = min(64, a.ent_off[e + 1] - tb);
     const bool active = wave * 16 < nt;
     const int trow = wave * 16 + r; const bool tv = trow < nt;
     const int tc = min(trow, nt - 1);
-    auto dof = [&](int i) { return 16 * (i >> 2) + 4 * kq + (i & 3); };      // reduction step i of lane group kq
+    // reduction step i of lane group kq takes channel 16 (i / 4) + 4 kq + i % 4: four steps of a lane are 16 contiguous bytes
+    const bool vec = dim == DP && ((a.src_ld | a.gz_ld) & 3) == 0 && (((uintptr_t)a.qsrc | (uintptr_t)a.ksrc | (uintptr_t)a.gz | (uintptr_t)a.bonus) & 15) == 0;
+    auto ld4 = [&](const float* p, int d) {
+        if (vec) return *reinterpret_cast<const float4*>(p + d);
+        return make_float4(p[min(d, dim - 1)], p[min(d + 1, dim - 1)], p[min(d + 2, dim - 1)], p[min(d + 3, dim - 1)]);
+    };
     const float* fz = a.gz + (size_t)tb * a.gz_ld + (size_t)h * dim;
     const float* kz = a.ksrc + (size_t)tb * a.src_ld + (size_t)h * dim; const float* qz = a.qsrc + (size_t)tb * a.src_ld + (size_t)h * dim;
     const float* vz = a.vsrc + (size_t)tb * a.src_ld + (size_t)h * vdim;
-    for (int i = tid; i < 4 * dimp; i += 256) {
-        const int m = i / dimp, d = i - m * dimp;
+    for (int i = tid; i < 4 * DP; i += 256) {
+        const int m = i / DP, d = i - m * DP;
         const float v = (d < dim && 16 * m < nt) ? fz[(size_t)min(16 * m + 15, nt - 1) * a.gz_ld + d] : 0.0f;
         tot[i] = v; et[i] = expf(v);
     }
-    __syncthreads();
-    for (int i = tid; i < 64 * dimp; i += 256) {
-        const int s = i / dimp, d = i - s * dimp;
-        kd[s * LK + d] = (s < nt && d < dim) ? kz[(size_t)s * a.src_ld + d] * expf(tot[(s >> 4) * dimp + d] - fz[(size_t)s * a.gz_ld + d]) : 0.0f;
-    }
-    float bonus = 0.0f, big = 0.0f;
-    for (int i = 0; i < dq; i++) {
-        const int d = dof(i);
-        float q = 0.0f;
-        if (active && d < dim) {
-            const float x = qz[(size_t)tc * a.src_ld + d] * a.q_scale;
-            float ev = 0.0f;
-            if constexpr (WKV) { if (r > 0) ev = fz[(size_t)(tc - (trow < nt)) * a.gz_ld + d]; bonus = __builtin_fmaf(x * a.bonus[(size_t)h * dim + d], kz[(size_t)tc * a.src_ld + d], bonus); }
-            else ev = fz[(size_t)tc * a.gz_ld + d];
-            q = x * expf(ev);
-            big = fmaxf(big, -tot[wave * dimp + d]);
+    float4 q4[DT];
+    float bonus = 0.0f;
+    {
+        const float* qp = qz + (size_t)tc * a.src_ld; const float* kp = kz + (size_t)tc * a.src_ld; const float* fp = fz + (size_t)(WKV ? max(tc - 1, 0) : tc) * a.gz_ld;
+        const bool past = !WKV || r > 0;                          // a sub-block's first token reads what the sub-block before left
+#pragma unroll
+        for (int i = 0; i < DT; i++) {
+            const int d = 16 * i + 4 * kq;
+            float4 x = ld4(qp, d); const float4 f = ld4(fp, d);
+            x.x *= a.q_scale; x.y *= a.q_scale; x.z *= a.q_scale; x.w *= a.q_scale;
+            if (d >= dim) x.x = 0.0f; if (d + 1 >= dim) x.y = 0.0f; if (d + 2 >= dim) x.z = 0.0f; if (d + 3 >= dim) x.w = 0.0f;
+            if constexpr (WKV) {
+                const float4 u = ld4(a.bonus + (size_t)h * dim, d), k = ld4(kp, d);
+                bonus = __builtin_fmaf(x.x * u.x, k.x, bonus); bonus = __builtin_fmaf(x.y * u.y, k.y, bonus); bonus = __builtin_fmaf(x.z * u.z, k.z, bonus); bonus = __builtin_fmaf(x.w * u.w, k.w, bonus);
+            }
+            if (past) { x.x *= expf(f.x); x.y *= expf(f.y); x.z *= expf(f.z); x.w *= expf(f.w); }
+            q4[i] = x;
         }
-        qs[i * 64 + lane] = q;
     }
     if constexpr (WKV) { bonus += __shfl_xor(bonus, 16); bonus += __shfl_xor(bonus, 32); }
+    __syncthreads();
+#pragma unroll 4
+    for (int i = tid; i < 64 * (DP / 4); i += 256) {
+        const int s = i / (DP / 4), d = 4 * (i - s * (DP / 4)), sc = min(s, nt - 1);
+        float4 k = ld4(kz + (size_t)sc * a.src_ld, d); const float4 f = ld4(fz + (size_t)sc * a.gz_ld, d), t4 = *reinterpret_cast<const float4*>(tot + (s >> 4) * DP + d);
+        const bool ok = s < nt;
+        k.x = ok && d < dim ? k.x * expf(t4.x - f.x) : 0.0f; k.y = ok && d + 1 < dim ? k.y * expf(t4.y - f.y) : 0.0f;
+        k.z = ok && d + 2 < dim ? k.z * expf(t4.z - f.z) : 0.0f; k.w = ok && d + 3 < dim ? k.w * expf(t4.w - f.w) : 0.0f;
+        *reinterpret_cast<float4*>(kd + s * LK + d) = k;
+    }
+    float big = 0.0f;
+#pragma unroll
+    for (int i = 0; i < DT; i++) { const float4 t4 = *reinterpret_cast<const float4*>(tot + wave * DP + 16 * i + 4 * kq); big = fmaxf(big, fmaxf(fmaxf(-t4.x, -t4.y), fmaxf(-t4.z, -t4.w))); }
     big = fmaxf(big, __shfl_xor(big, 16)); big = fmaxf(big, __shfl_xor(big, 32));      // the same in every lane of a wave: lanes of one group share their channels
     __syncthreads();
     ln_f4 acc[DB];
@@ -289,9 +373,16 @@ __global__ void __launch_bounds__(256) ln_chan_out_kernel(const KrSvLin a) {
     if (active) {
 #pragma nounroll
         for (int j = wave; j >= 0; j--) {
+            size_t srow[4]; float vf[4][DB];                      // the value rows of the tile's keys: requested before the first product
+#pragma unroll
+            for (int i = 0; i < 4; i++) srow[i] = (size_t)min(16 * j + 4 * kq + i, nt - 1) * a.src_ld;
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int c = 0; c < DB; c++) vf[i][c] = vz[srow[i] + min(c * 16 + r, vdim - 1)];
             ln_f4 st = ln_f4{0.0f, 0.0f, 0.0f, 0.0f};
             const float* krow = kd + (16 * j + r) * LK + 4 * kq;
-            const float* ep = et + j * dimp + 4 * kq;
+            const float* ep = et + j * DP + 4 * kq;
             if (j == wave && big > 60.0f) {
                 for (int d = 0; d < dim; d++) {
                     const float x = qz[(size_t)tc * a.src_ld + d] * a.q_scale;
@@ -303,32 +394,23 @@ __global__ void __launch_bounds__(256) ln_chan_out_kernel(const KrSvLin a) {
                     }
                 }
             } else {
-                for (int i0 = 0; i0 < dq; i0 += 4) {
-                    const float4 k4 = *reinterpret_cast<const float4*>(krow + 4 * i0), e4 = *reinterpret_cast<const float4*>(ep + 4 * i0);
-                    float q4[4];
+                // inside the own sub-block the queries go back to its end first (exp(e_t - tot)); on the way to the one before an earlier one they take that one's decay along
+                const bool own = j == wave;
 #pragma unroll
-                    for (int u = 0; u < 4; u++) q4[u] = qs[(i0 + u) * 64 + lane];
-                    const float x0 = j == wave ? 1.0f / e4.x : 1.0f, x1 = j == wave ? 1.0f / e4.y : 1.0f, x2 = j == wave ? 1.0f / e4.z : 1.0f, x3 = j == wave ? 1.0f / e4.w : 1.0f;
-                    st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.x, q4[0] * x0, st, 0, 0, 0); st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.y, q4[1] * x1, st, 0, 0, 0);
-                    st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.z, q4[2] * x2, st, 0, 0, 0); st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.w, q4[3] * x3, st, 0, 0, 0);
-                    if (j < wave) {          // on to the sub-block before: the queries take this one's decay along
-                        qs[i0 * 64 + lane] = q4[0] * e4.x; qs[(i0 + 1) * 64 + lane] = q4[1] * e4.y; qs[(i0 + 2) * 64 + lane] = q4[2] * e4.z; qs[(i0 + 3) * 64 + lane] = q4[3] * e4.w;
-                    }
+                for (int i = 0; i < DT; i++) {
+                    const float4 k4 = *reinterpret_cast<const float4*>(krow + 16 * i), e4 = *reinterpret_cast<const float4*>(ep + 16 * i);
+                    const float4 x = own ? make_float4(q4[i].x / e4.x, q4[i].y / e4.y, q4[i].z / e4.z, q4[i].w / e4.w) : q4[i];
+                    st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.x, x.x, st, 0, 0, 0); st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.y, x.y, st, 0, 0, 0);
+                    st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.z, x.z, st, 0, 0, 0); st = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.w, x.w, st, 0, 0, 0);
+                    if (!own) q4[i] = make_float4(q4[i].x * e4.x, q4[i].y * e4.y, q4[i].z * e4.z, q4[i].w * e4.w);
                 }
             }
-            size_t srow[4];
 #pragma unroll
             for (int i = 0; i < 4; i++) {
                 const int s = 16 * j + 4 * kq + i;
-                srow[i] = (size_t)min(s, nt - 1) * a.src_ld;
                 if (j == wave) { if (WKV && s == trow) st[i] = bonus; else if (s > trow) st[i] = 0.0f; }
                 if (!tv) st[i] = 0.0f;
             }
-            float vf[4][DB];
-#pragma unroll
-            for (int i = 0; i < 4; i++)
-#pragma unroll
-                for (int c = 0; c < DB; c++) { const int cc = c * 16 + r; vf[i][c] = cc < vdim ? vz[srow[i] + cc] : 0.0f; }
 #pragma unroll
             for (int i = 0; i < 4; i++)
 #pragma unroll
@@ -336,7 +418,9 @@ __global__ void __launch_bounds__(256) ln_chan_out_kernel(const KrSvLin a) {
         }
     }
     const float* Sc = a.sbuf + ((size_t)gc * H + h) * dim * vdim;
-    for (int p0 = 0; p0 < dim; p0 += 32) {          // the state's share: passes over 32 of its rows
+#pragma unroll
+    for (int p0 = 0; p0 < DP; p0 += 32) {           // the state's share: passes over 32 of its rows
+        if (p0 >= dim) break;
         const int rows = min(32, dim - p0);
         __syncthreads();
         if ((vdim & 3) == 0) {
@@ -347,13 +431,14 @@ __global__ void __launch_bounds__(256) ln_chan_out_kernel(const KrSvLin a) {
         }
         __syncthreads();
         if (active) {
-#pragma unroll 2
+#pragma unroll
             for (int i = 0; i < 8; i++) {
-                const int lr = dof(i);
-                const float qi = lr < rows ? qs[(p0 / 4 + i) * 64 + lane] : 0.0f;
+                const int lr = 16 * (i >> 2) + 4 * kq + (i & 3);
+                const float4 qq = q4[p0 / 16 + (i >> 2)];
+                const float qi = (i & 3) == 0 ? qq.x : (i & 3) == 1 ? qq.y : (i & 3) == 2 ? qq.z : qq.w;      // zero past dim
                 const float* srow = sl + min(lr, rows - 1) * LS + r;
 #pragma unroll
-                for (int c = 0; c < DB; c++) acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(c * 16 + r < vdim ? srow[c * 16] : 0.0f, qi, acc[c], 0, 0, 0);
+                for (int c = 0; c < DB; c++) acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(srow[c * 16], qi, acc[c], 0, 0, 0);      // columns past vdim are not stored
             }
         }
     }
@@ -463,34 +548,47 @@ __global__ void __launch_bounds__(256) ln_delta_solve_kernel(const KrSvLin a) {
     }
 }
 // (2) block after block of an entry, one workgroup per (entry, head, 16 value columns): U = X - Y S (wave w: tokens 16 w ..), then S <- e^{F_last} S + sum_s e^{F_last - F_s} k_s u_s^T
-// (wave w: key rows 16 w .. and 16 (w + 4) ..).  S lives in the accumulators and, as the next block's operand, in LDS; the operands of the next block are requested
-// before the current one is worked on.  Leaves S at the block's start in a.sbuf and U in place of v; the outputs are sv_lin_cout_kernel's.
-template <int DT>          // 16-row tiles of a head's keys: 4 or 8
+// (wave w: NW tiles of key rows, row 16 NW w + NW r + n in tile n, so that a lane's rows stand together in memory).  S lives in the accumulators and, as the next block's
+// operand, in LDS; the operands of the next block are requested before the current one is worked on.  Leaves S at the block's start in a.sbuf and U in place of v; the outputs
+// are sv_lin_cout_kernel's.
+template <int DT, bool VEC>          // 16-row tiles of a head's keys, 4 or 8; VEC: dim fills them and the rows are 16-byte aligned
 __global__ void __launch_bounds__(256) ln_delta_state_kernel(const KrSvLin a) {
-    constexpr int DP = DT * 16, NW = DT / 4, LS = 20;      // NW key-row tiles per wave; LDS rows of 16 columns, 20 floats apart
+    constexpr int DP = DT * 16, NW = DT / 4, LS = 20;      // LDS rows of 16 columns, 20 floats apart
     __shared__ __attribute__((aligned(16))) float Sl[DP * LS], Ul[64 * LS];
     const int e = blockIdx.x, h = blockIdx.y, cb = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, kq = lane >> 4;
     const int H = a.heads, dim = a.dim, vdim = a.vdim, hq = h / a.qk_group, col = cb * 16 + r; const bool cv = col < vdim; const int colc = cv ? col : 0;
     const int t0 = a.ent_off[e], t1 = a.ent_off[e + 1], nch = (t1 - t0 + 63) / 64, c0 = a.ent_chunk0[e];
     const bool fresh = a.pos[t0] == 0;
     float* Sg = a.state + (size_t)a.ent_slot[e] * a.state_stride + ((size_t)h * vdim + colc) * dim;
+    auto drow = [&](int n, int i) { return 16 * NW * wave + NW * (4 * kq + i) + n; };      // the key row of accumulator i of tile n
     ln_f4 S[NW];
 #pragma unroll
     for (int n = 0; n < NW; n++)
 #pragma unroll
-        for (int i = 0; i < 4; i++) { const int d = (wave + 4 * n) * 16 + 4 * kq + i; S[n][i] = (!fresh && cv && d < dim) ? Sg[d] : 0.0f; }
-    float y[2][DP / 4], kk[2][NW][16], xv[2][4], fs[2][4], fl[2];
+        for (int i = 0; i < 4; i++) { const int d = drow(n, i); const float v = Sg[VEC ? d : min(d, dim - 1)]; S[n][i] = (!fresh && cv && (VEC || d < dim)) ? v : 0.0f; }
+    float y[2][DP / 4], kk[2][16][NW], xv[2][4], fs[2][4], fl[2];
     auto fetch = [&](int b, int c) {
         const int tb = t0 + 64 * c, nt = min(64, t1 - tb);
         const float* yp = a.aux + (size_t)(tb + min(16 * wave + r, nt - 1)) * H * dim + (size_t)h * dim;
 #pragma unroll
-        for (int i = 0; i < DP / 4; i++) { const int d = 16 * (i >> 2) + 4 * kq + (i & 3); y[b][i] = d < dim ? yp[d] : 0.0f; }
+        for (int i = 0; i < DT; i++) {
+            const int d = 16 * i + 4 * kq;
+            if constexpr (VEC) { const float4 v = *reinterpret_cast<const float4*>(yp + d); y[b][4 * i] = v.x; y[b][4 * i + 1] = v.y; y[b][4 * i + 2] = v.z; y[b][4 * i + 3] = v.w; }
+            else {
+#pragma unroll
+                for (int u = 0; u < 4; u++) y[b][4 * i + u] = yp[min(d + u, dim - 1)];      // meets a zero row of S past dim
+            }
+        }
         const float* kp = a.ksrc + (size_t)tb * a.src_ld + (size_t)hq * dim;
+        const int d0 = 16 * NW * wave + NW * r;
 #pragma unroll
-        for (int n = 0; n < NW; n++) {
-            const int d = (wave + 4 * n) * 16 + r;
+        for (int j = 0; j < 16; j++) {
+            const float* kr = kp + (size_t)min(4 * j + kq, nt - 1) * a.src_ld;
+            if constexpr (VEC && NW == 2) { const float2 v = *reinterpret_cast<const float2*>(kr + d0); kk[b][j][0] = v.x; kk[b][j][NW - 1] = v.y; }
+            else {
 #pragma unroll
-            for (int j = 0; j < 16; j++) kk[b][n][j] = d < dim ? kp[(size_t)min(4 * j + kq, nt - 1) * a.src_ld + d] : 0.0f;
+                for (int n = 0; n < NW; n++) kk[b][j][n] = kr[VEC ? d0 + n : min(d0 + n, dim - 1)];
+            }
         }
 #pragma unroll
         for (int i = 0; i < 4; i++) {
@@ -506,14 +604,18 @@ __global__ void __launch_bounds__(256) ln_delta_state_kernel(const KrSvLin a) {
         for (int n = 0; n < NW; n++)
 #pragma unroll
             for (int i = 0; i < 4; i++) {
-                const int d = (wave + 4 * n) * 16 + 4 * kq + i;
-                Sl[d * LS + r] = S[n][i];
-                if (cv && d < dim) sb[(size_t)d * vdim] = S[n][i];
+                const int d = drow(n, i);
+                Sl[d * LS + r] = (VEC || d < dim) ? S[n][i] : 0.0f;
+                if (cv && (VEC || d < dim)) sb[(size_t)d * vdim] = S[n][i];
             }
         __syncthreads();
-        ln_f4 u = ln_f4{0.0f, 0.0f, 0.0f, 0.0f};
+        ln_f4 u = ln_f4{0.0f, 0.0f, 0.0f, 0.0f}, u1 = u;      // two chains: a dependent product waits for the one before
 #pragma unroll
-        for (int i = 0; i < DP / 4; i++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(y[b][i], Sl[(16 * (i >> 2) + 4 * kq + (i & 3)) * LS + r], u, 0, 0, 0);
+        for (int i = 0; i < DP / 4; i += 2) {
+            u = __builtin_amdgcn_mfma_f32_16x16x4f32(y[b][i], Sl[(16 * (i >> 2) + 4 * kq + (i & 3)) * LS + r], u, 0, 0, 0);
+            u1 = __builtin_amdgcn_mfma_f32_16x16x4f32(y[b][i + 1], Sl[(16 * (i >> 2) + 4 * kq + (i & 3) + 1) * LS + r], u1, 0, 0, 0);
+        }
+        u += u1;
         float* up = const_cast<float*>(a.vsrc) + (size_t)tb * a.src_ld + (size_t)h * vdim + col;
 #pragma unroll
         for (int i = 0; i < 4; i++) {
@@ -522,15 +624,15 @@ __global__ void __launch_bounds__(256) ln_delta_state_kernel(const KrSvLin a) {
             Ul[s * LS + r] = v * expf(fl[b] - fs[b][i]);
             if (ok) up[(size_t)s * a.src_ld] = v;
         }
-        __syncthreads();
         const float dec = expf(fl[b]);
 #pragma unroll
         for (int n = 0; n < NW; n++) S[n] *= dec;
+        __syncthreads();
 #pragma unroll
         for (int j = 0; j < 16; j++) {
             const float uu = Ul[(4 * j + kq) * LS + r];
 #pragma unroll
-            for (int n = 0; n < NW; n++) S[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[b][n][j], uu, S[n], 0, 0, 0);
+            for (int n = 0; n < NW; n++) S[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[b][j][n], uu, S[n], 0, 0, 0);
         }
     };
     fetch(0, 0);
@@ -543,7 +645,7 @@ __global__ void __launch_bounds__(256) ln_delta_state_kernel(const KrSvLin a) {
 #pragma unroll
     for (int n = 0; n < NW; n++)
 #pragma unroll
-        for (int i = 0; i < 4; i++) { const int d = (wave + 4 * n) * 16 + 4 * kq + i; if (cv && d < dim) Sg[d] = S[n][i]; }
+        for (int i = 0; i < 4; i++) { const int d = drow(n, i); if (cv && (VEC || d < dim)) Sg[d] = S[n][i]; }
 }
 }  // namespace
 
@@ -551,14 +653,15 @@ bool kr_sv_lin_blocks_fit(int dim, int vdim) { return dim <= 128 && vdim <= 128;
 void kr_sv_lin_chan_blocks(const KrSvLin& a, hipStream_t st) {
     if (a.T <= 0 || a.n_entries <= 0 || a.n_chunks <= 0) return;
     const dim3 g(a.n_chunks, a.heads);
-    const int dimp = ((a.dim + 15) / 16) * 16;
 #define LN_LDS(K_, B_) do { if ((B_) > 48 * 1024) (void)hipFuncSetAttribute((const void*)K_, hipFuncAttributeMaxDynamicSharedMemorySize, (int)(B_)); } while (0)
     if (a.dim <= 64) { const size_t b = (size_t)(64 * 80 + 4 * 64) * 4; hipLaunchKernelGGL(ln_chan_local_kernel<4>, g, dim3(256), b, st, a); }
     else { const size_t b = (size_t)(64 * 144 + 4 * 128) * 4; LN_LDS(ln_chan_local_kernel<8>, b); hipLaunchKernelGGL(ln_chan_local_kernel<8>, g, dim3(256), b, st, a); }
     hipLaunchKernelGGL(ln_chan_scan_kernel, dim3(a.n_entries, a.heads, (a.dim * a.vdim + 255) / 256), dim3(256), 0, st, a);
-    const size_t lds = ((size_t)64 * (dimp + 4) + 8 * dimp + 32 * (((a.vdim + 31) / 32) * 32 + 16) + (size_t)4 * (dimp / 4) * 64) * 4;
-#define LN_CO(DB_, W_) do { LN_LDS((ln_chan_out_kernel<DB_, W_>), lds); hipLaunchKernelGGL((ln_chan_out_kernel<DB_, W_>), g, dim3(256), lds, st, a); } while (0)
-    if (a.vdim <= 64) { if (a.kind == 7) LN_CO(4, true); else LN_CO(4, false); } else { if (a.kind == 7) LN_CO(8, true); else LN_CO(8, false); }
+#define LN_CO(DT_, DB_, W_) do { const size_t b_ = (size_t)(8 * DT_ * 16 + (64 * (DT_ * 16 + 4) > 32 * (DB_ * 16 + 16) ? 64 * (DT_ * 16 + 4) : 32 * (DB_ * 16 + 16))) * 4; \
+        LN_LDS((ln_chan_out_kernel<DT_, DB_, W_>), b_); hipLaunchKernelGGL((ln_chan_out_kernel<DT_, DB_, W_>), g, dim3(256), b_, st, a); } while (0)
+#define LN_CO_W(DT_, DB_) do { if (a.kind == 7) LN_CO(DT_, DB_, true); else LN_CO(DT_, DB_, false); } while (0)
+    if (a.dim <= 64) { if (a.vdim <= 64) LN_CO_W(4, 4); else LN_CO_W(4, 8); } else { if (a.vdim <= 64) LN_CO_W(8, 4); else LN_CO_W(8, 8); }
+#undef LN_CO_W
 #undef LN_CO
 }
 void kr_sv_delta_blocks(const KrSvLin& a, hipStream_t st) {
@@ -567,16 +670,19 @@ void kr_sv_delta_blocks(const KrSvLin& a, hipStream_t st) {
     LN_LDS(ln_delta_solve_kernel, lds);
     hipLaunchKernelGGL(ln_delta_solve_kernel, dim3(a.n_chunks, a.heads), dim3(256), lds, st, a);
     const dim3 gs(a.n_entries, a.heads, (a.vdim + 15) / 16);
-    if (a.dim <= 64) hipLaunchKernelGGL(ln_delta_state_kernel<4>, gs, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL(ln_delta_state_kernel<8>, gs, dim3(256), 0, st, a);
+    const bool vec = (a.dim == 64 || a.dim == 128) && (a.src_ld & 3) == 0 && (((uintptr_t)a.ksrc | (uintptr_t)a.aux) & 15) == 0;
+    if (a.dim <= 64) { if (vec) hipLaunchKernelGGL((ln_delta_state_kernel<4, true>), gs, dim3(256), 0, st, a); else hipLaunchKernelGGL((ln_delta_state_kernel<4, false>), gs, dim3(256), 0, st, a); }
+    else { if (vec) hipLaunchKernelGGL((ln_delta_state_kernel<8, true>), gs, dim3(256), 0, st, a); else hipLaunchKernelGGL((ln_delta_state_kernel<8, false>), gs, dim3(256), 0, st, a); }
     kr_sv_lin_block_out(a, st);
 }
 
 void kr_sv_shift(const KrSvShift& a, bool f32, hipStream_t st) {
     if (a.T <= 0) return;
-    const dim3 grid(a.T, (a.width + 255) / 256);
-    if (f32) hipLaunchKernelGGL(ln_shift_kernel<float>, grid, dim3(256), 0, st, a, (float*)a.out);
-    else hipLaunchKernelGGL(ln_shift_kernel<uint16_t>, grid, dim3(256), 0, st, a, (uint16_t*)a.out);
+#define LN_SH(T_, VC_, TT_) hipLaunchKernelGGL((ln_shift_kernel<T_, VC_, TT_>), dim3((a.T + TT_ - 1) / TT_, (a.width / VC_ + 255) / 256), dim3(256), 0, st, a, (T_*)a.out)
+#define LN_SH_T(T_) do { if (a.width % 4) LN_SH(T_, 1, 1); else if (a.T <= 64) LN_SH(T_, 4, 1); else LN_SH(T_, 4, 4); } while (0)
+    if (f32) LN_SH_T(float); else LN_SH_T(uint16_t);
+#undef LN_SH_T
+#undef LN_SH
 }
 void kr_sv_wkv_decay(const float* z, int ld, const void* w2, bool f32, const float* w0, int T, int rank, int cols, float* out, hipStream_t st) {
     if (T <= 0) return;
@@ -588,14 +694,13 @@ void kr_sv_wkv_decay(const float* z, int ld, const void* w2, bool f32, const flo
 }
 void kr_sv_delta_prep(const KrSvDelta& a, hipStream_t st) {
     if (a.T <= 0) return;
-    hipLaunchKernelGGL(ln_delta_prep_kernel, dim3(a.T, 2 * a.kv_heads + a.heads), dim3(64), 0, st, a);
+#define LN_DP(NT_, TT_) hipLaunchKernelGGL((ln_delta_prep_kernel<NT_, TT_>), dim3((a.T + TT_ - 1) / TT_, 2 * a.kv_heads + a.heads), dim3(64), 0, st, a)
+#define LN_DP_T(NT_) do { if (a.T <= 64) LN_DP(NT_, 1); else LN_DP(NT_, 8); } while (0)
+    switch (a.taps) { case 1: LN_DP_T(1); break; case 2: LN_DP_T(2); break; case 3: LN_DP_T(3); break; case 4: LN_DP_T(4); break; default: LN_DP_T(0); break; }
+#undef LN_DP_T
+#undef LN_DP
     const int C = 2 * a.kv_heads * a.dim + a.heads * a.vdim;
     if (!a.single && a.taps > 1) hipLaunchKernelGGL(ln_delta_save_kernel, dim3(a.n_entries, a.taps - 1, (C + 255) / 256), dim3(256), 0, st, a);
-}
-void kr_sv_lt_prep(float* z, int ld, int cols, const float* decay, int heads, float4* tok, int T, hipStream_t st) {
-    if (T <= 0) return;
-    const int n = cols > heads ? cols : heads;
-    hipLaunchKernelGGL(ln_lt_prep_kernel, dim3(T, (n + 255) / 256), dim3(256), 0, st, z, ld, cols, decay, heads, tok);
 }
 void kr_sv_row_out(const float* o, int n, const float* w, const float* gate, int gate_ld, float eps, float scale, void* out, int out_ld, bool f32, int T, hipStream_t st) {
     if (T <= 0) return;

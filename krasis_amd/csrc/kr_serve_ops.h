@@ -28,6 +28,7 @@ struct KrSvGemm {
     // [*, o_gate_ld] f32 or null: an element of C is multiplied by sigmoid(o_gate[row / o_gate_div][(row % o_gate_div) * N + n]) before it is stored, row = its row in C
     const float* o_gate; int o_gate_ld, o_gate_div;
     const float* bias;               // [N] f32 or null: joins every row of C before it is stored (or gated)
+    int silu_lo, silu_hi;            // columns [silu_lo, silu_hi) of C pass silu before they are stored
     int n_last;                      // grouped, > 0: the last group's matrix has n_last rows (columns of C) instead of N; N is then the larger of the two
     int n_first;                     //   ... and the other groups' matrices have n_first
     // with act_gu: the up columns come from a table instead: element k of problem row r is up_tab[up_rows[r] * up_ld + up_off + k] (storage type)
@@ -196,12 +197,11 @@ struct KrSvLin {
     int kind;                        // KR_SERVE_MIX_RETENTION (2) | _MLSTM (3) | _GLA (4) | _SSD (5) | _WKV (7) | _DELTA (8)
     const float* qsrc; const float* ksrc; const float* vsrc; int src_ld, qk_group;      // kinds 4, 5, 7, 8: heads h of a group of qk_group share one q and one k
     const float* bonus;              // kind 7: [heads * dim]
-    int qkv_act;                     // kind 2: 1 = silu on q, k and v as they are read (kr_sv_lin_scan; the block launches take prepped rows)
     const float* gate; int gate_ld, gate_act;      // kr_sv_lin_out: gate logits [T, gate_ld] (null: they stand behind v in z); gate_act 0: by kind, 1: silu, 2: sigmoid
     const float* gz; int gz_ld; const float* gz_bias; float inv_tau;                     // kind 4
     const float* dtz; int dtz_ld; const float* dt_bias; const float* a_log;              // kind 5
     int norm_shared;                 // norm_w is [vdim], shared by the heads
-    int prepped;                     // kr_sv_lin_chunked: z already holds q, k as the block launches read them and tok the log decays (kr_sv_ssd_expand)
+    int prepped;                     // kr_sv_lin_chunked: z already holds q, k as the block launches read them; 1: and tok the log decays (kr_sv_ssd_expand); 2: the decays are `decay`
     float* z; int ld;                // [T, ld] f32: q [heads * dim] | k [heads * dim] | v [heads * vdim] | g [heads * vdim] | (mlstm) z_i [heads] | z_f [heads]
     int heads, dim, vdim, rot_dims;
     const float2* cs;                // rotation table of the step [T, rot_dims / 2] (pairs (i, i + rot_dims / 2))
@@ -310,8 +310,6 @@ struct KrSvDelta {
     float4* tok;                     // [T, heads]
 };
 void kr_sv_delta_prep(const KrSvDelta& a, hipStream_t st);
-// lightning attention before the block launches: silu on the row block [q | k | v] in place, tok[t][h].x = log decay
-void kr_sv_lt_prep(float* z, int ld, int cols, const float* decay, int heads, float4* tok, int T, hipStream_t st);
 // out[t][c] = o[t] / rms(o[t]) * w[c] * sigmoid(gate[t][c]) * scale over the whole row of n
 void kr_sv_row_out(const float* o, int n, const float* w, const float* gate, int gate_ld, float eps, float scale, void* out, int out_ld, bool f32, int T, hipStream_t st);
 void kr_sv_argmax(const float* logits, int R, int vocab, int* out, hipStream_t st);

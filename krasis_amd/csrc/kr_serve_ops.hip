@@ -1141,16 +1141,15 @@ __global__ void __launch_bounds__(64) sv_lin_scan_kernel(const KrSvLin a) {
             }
             if (DELTA && lane < nt) { const float4 tk = a.tok[(size_t)(tb + lane) * H + h]; gs[2 * lane] = tk.w; gs[2 * lane + 1] = tk.x; }
         } else {
-        auto in = [&](float v) { return a.qkv_act ? v / (1.0f + expf(-v)) : v; };
         for (int idx = lane; idx < nt * dimp; idx += 64) {
             const int tt = idx / dimp, d = idx - tt * dimp;
             const float* zr = a.z + (size_t)(tb + tt) * a.ld + (size_t)h * dim;
-            qs[idx] = d < dim ? in(zr[d]) * a.q_scale : 0.0f;
-            ks[idx] = d < dim ? in(zr[(size_t)H * dim + d]) * a.k_scale : 0.0f;
+            qs[idx] = d < dim ? zr[d] * a.q_scale : 0.0f;
+            ks[idx] = d < dim ? zr[(size_t)H * dim + d] * a.k_scale : 0.0f;
         }
         for (int idx = lane; idx < nt * 16; idx += 64) {
             const int tt = idx >> 4, c = cb * 16 + (idx & 15);
-            vs[idx] = c < vdim ? in(a.z[(size_t)(tb + tt) * a.ld + (size_t)2 * H * dim + (size_t)h * vdim + c]) : 0.0f;
+            vs[idx] = c < vdim ? a.z[(size_t)(tb + tt) * a.ld + (size_t)2 * H * dim + (size_t)h * vdim + c] : 0.0f;
         }
         if (ML && lane < nt) {
             const float* zg = a.z + (size_t)(tb + lane) * a.ld + (size_t)2 * H * dim + (size_t)2 * H * vdim;
@@ -1487,7 +1486,8 @@ __global__ void __launch_bounds__(64) sv_lin_mlocal_kernel(const KrSvLin a) {
     const int tb = a.ent_off[e] + 64 * (gc - a.ent_chunk0[e]), nt = min(64, a.ent_off[e + 1] - tb);
     const bool ok = lane < nt;
     const size_t ti = (size_t)(tb + lane) * H + h;
-    const float4 ab = ok ? a.tok[ti] : make_float4(0.0f, -INFINITY, 0.0f, 0.0f);
+    float4 ab = make_float4(0.0f, -INFINITY, 0.0f, 0.0f);
+    if (ok) { if (!ML && a.prepped == 2) ab.x = fmaxf(logf(a.decay[h]), -1.0e4f); else ab = a.tok[ti]; }
     float F = ab.x;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) { const float up = __shfl_up(F, o); if (lane >= o) F += up; }
