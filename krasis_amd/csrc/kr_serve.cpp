@@ -1039,7 +1039,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         if (l.gla()) { max_ga1 = std::max(max_ga1, (size_t)d.decay_rank); max_gz = std::max(max_gz, (size_t)d.heads * d.dim); }
         if (l.recurrent()) {
             max_lin = std::max(max_lin, (size_t)d.heads * d.vdim);
-            if (lin_chunked && ((l.chunkable() && kr_sv_lin_chunked_fits(d.dim, d.vdim)) || ((l.wkv() || l.delta()) && kr_sv_lin_blocks_fit(d.dim, d.vdim)))) {
+            if (lin_chunked && ((l.chunkable() && kr_sv_lin_chunked_fits(d.dim, d.vdim)) || ((l.wkv() || l.gla() || l.delta()) && kr_sv_lin_blocks_fit(d.dim, d.vdim)))) {
                 if (l.delta()) lin_aux = std::max(lin_aux, (size_t)d.heads * d.dim);
                 lin_tok = std::max(lin_tok, (size_t)d.heads); lin_sb = std::max(lin_sb, (size_t)d.heads * d.dim * d.vdim); lin_nb = std::max(lin_nb, (size_t)d.heads * d.dim);
             }
@@ -1235,7 +1235,7 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
             {
                 Timer tm(s, 3);
                 if (lin_chunked && l.chunkable() && kr_sv_lin_chunked_fits(d.dim, d.vdim)) kr_sv_lin_chunked(q, st);
-                else if (lin_chunked && l.wkv() && kr_sv_lin_blocks_fit(d.dim, d.vdim)) kr_sv_lin_chan_blocks(q, st);
+                else if (lin_chunked && (l.wkv() || l.gla()) && kr_sv_lin_blocks_fit(d.dim, d.vdim)) kr_sv_lin_chan_blocks(q, st);
                 else if (lin_chunked && l.delta() && kr_sv_lin_blocks_fit(d.dim, d.vdim)) { q.aux = (float*)s->lin_aux.p; kr_sv_delta_blocks(q, st); }
                 else if (lin_chunked && kr_sv_lin_scan_wide_fits(q.kind, d.dim)) kr_sv_lin_scan_wide(q, st);
                 else kr_sv_lin_scan(q, st);

@@ -229,6 +229,13 @@ __global__ void __launch_bounds__(256) ln_row_out_kernel(const float* __restrict
 // exp(e_t) * prod(sub-blocks between) * exp(tot - f_s) (e_t = f_t, or the sum before t where the read-out comes before the write): all three factors are <= 1, so
 // strong decays cannot overflow.  Inside a sub-block the split would be exp(e_t - tot) * exp(tot - f_s), whose first factor is >= 1: it is taken while the
 // sub-block's sums stay above -60, and below that the sixteen tokens' weights are formed pair by pair.
+// gla: log decays from their logits, in place: log sigmoid(z + b) / tau
+__global__ void __launch_bounds__(256) ln_gla_log_kernel(float* __restrict__ gz, const float* __restrict__ bias, size_t n, int cols, float inv_tau) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    const float z = gz[i] + bias[i % cols];
+    gz[i] = (fminf(z, 0.0f) - log1pf(expf(-fabsf(z)))) * inv_tau;
+}
 // (1) in parallel over (block, head): f in place of the log decays, the block's own contribution U = sum_s exp(F_last - F_s) k_s v_s^T to a.sbuf, exp(F_last) to a.nbuf
 __device__ __forceinline__ int ln_entry_of(const KrSvLin& a, int gc) { int e = 0; while (e + 1 < a.n_entries && a.ent_chunk0[e + 1] <= gc) e++; return e; }
 template <int DT>          // 16-row tiles of a head's keys: 4 (dim <= 64) or 8 (dim <= 128)
@@ -610,10 +617,21 @@ __global__ void __launch_bounds__(256) ln_delta_state_kernel(const KrSvLin a) {
             }
         __syncthreads();
         ln_f4 u = ln_f4{0.0f, 0.0f, 0.0f, 0.0f}, u1 = u;      // two chains: a dependent product waits for the one before
+        float sv[2][8];                                      // the state's rows, eight steps read ahead of the eight that are multiplied
+        auto read8 = [&](float (&v)[8], int i0) {
 #pragma unroll
-        for (int i = 0; i < DP / 4; i += 2) {
-            u = __builtin_amdgcn_mfma_f32_16x16x4f32(y[b][i], Sl[(16 * (i >> 2) + 4 * kq + (i & 3)) * LS + r], u, 0, 0, 0);
-            u1 = __builtin_amdgcn_mfma_f32_16x16x4f32(y[b][i + 1], Sl[(16 * (i >> 2) + 4 * kq + (i & 3) + 1) * LS + r], u1, 0, 0, 0);
+            for (int k = 0; k < 8; k++) v[k] = Sl[(16 * ((i0 + k) >> 2) + 4 * kq + (k & 3)) * LS + r];
+        };
+        read8(sv[0], 0);
+#pragma unroll
+        for (int i = 0; i < DP / 4; i += 8) {
+            if (i + 8 < DP / 4) read8(sv[((i >> 3) + 1) & 1], i + 8);
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int k = 0; k < 8; k += 2) {
+                u = __builtin_amdgcn_mfma_f32_16x16x4f32(y[b][i + k], sv[(i >> 3) & 1][k], u, 0, 0, 0);
+                u1 = __builtin_amdgcn_mfma_f32_16x16x4f32(y[b][i + k + 1], sv[(i >> 3) & 1][k + 1], u1, 0, 0, 0);
+            }
         }
         u += u1;
         float* up = const_cast<float*>(a.vsrc) + (size_t)tb * a.src_ld + (size_t)h * vdim + col;
@@ -628,19 +646,24 @@ __global__ void __launch_bounds__(256) ln_delta_state_kernel(const KrSvLin a) {
 #pragma unroll
         for (int n = 0; n < NW; n++) S[n] *= dec;
         __syncthreads();
+        float uu[16];
 #pragma unroll
-        for (int j = 0; j < 16; j++) {
-            const float uu = Ul[(4 * j + kq) * LS + r];
+        for (int j = 0; j < 16; j++) uu[j] = Ul[(4 * j + kq) * LS + r];
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-            for (int n = 0; n < NW; n++) S[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[b][j][n], uu, S[n], 0, 0, 0);
-        }
+        for (int j = 0; j < 16; j++)
+#pragma unroll
+            for (int n = 0; n < NW; n++) S[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[b][j][n], uu[j], S[n], 0, 0, 0);
     };
+    // blocks in pairs, every request unconditional (past the last block it repeats that one): the wait for a block's operands then leaves the next block's in flight
+    int c = 0;
     fetch(0, 0);
-    for (int c = 0; c < nch; c += 2) {
-        if (c + 1 < nch) fetch(1, c + 1);
+    if (nch & 1) { block(0, 0); c = 1; fetch(0, min(1, nch - 1)); }
+    for (; c < nch; c += 2) {
+        fetch(1, c + 1);
         block(0, c);
-        if (c + 2 < nch) fetch(0, c + 2);
-        if (c + 1 < nch) block(1, c + 1);
+        fetch(0, min(c + 2, nch - 1));
+        block(1, c + 1);
     }
 #pragma unroll
     for (int n = 0; n < NW; n++)
@@ -654,6 +677,10 @@ void kr_sv_lin_chan_blocks(const KrSvLin& a, hipStream_t st) {
     if (a.T <= 0 || a.n_entries <= 0 || a.n_chunks <= 0) return;
     const dim3 g(a.n_chunks, a.heads);
 #define LN_LDS(K_, B_) do { if ((B_) > 48 * 1024) (void)hipFuncSetAttribute((const void*)K_, hipFuncAttributeMaxDynamicSharedMemorySize, (int)(B_)); } while (0)
+    if (a.kind == 4) {
+        const size_t n = (size_t)a.T * a.heads * a.dim;
+        hipLaunchKernelGGL(ln_gla_log_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, const_cast<float*>(a.gz), a.gz_bias, n, a.heads * a.dim, a.inv_tau);
+    }
     if (a.dim <= 64) { const size_t b = (size_t)(64 * 80 + 4 * 64) * 4; hipLaunchKernelGGL(ln_chan_local_kernel<4>, g, dim3(256), b, st, a); }
     else { const size_t b = (size_t)(64 * 144 + 4 * 128) * 4; LN_LDS(ln_chan_local_kernel<8>, b); hipLaunchKernelGGL(ln_chan_local_kernel<8>, g, dim3(256), b, st, a); }
     hipLaunchKernelGGL(ln_chan_scan_kernel, dim3(a.n_entries, a.heads, (a.dim * a.vdim + 255) / 256), dim3(256), 0, st, a);

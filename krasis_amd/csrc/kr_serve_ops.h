@@ -235,7 +235,7 @@ bool kr_sv_lin_chunked_fits(int dim, int vdim);
 void kr_sv_lin_chunked(const KrSvLin& a, hipStream_t st);
 // the last of the block launches alone: outputs from sbuf, tok and the rows z (kinds 2 and 8; 8: heads share keys in groups of qk_group)
 void kr_sv_lin_block_out(const KrSvLin& a, hipStream_t st);
-// prompt portions of kinds 4 (a.gz = log decays) and 7 in blocks of 64 tokens: sbuf and nbuf as above, gz is overwritten with running sums
+// prompt portions of kinds 4 (gz: the decays' logits) and 7 (gz: log decays) in blocks of 64 tokens: sbuf and nbuf as above, gz is overwritten with running sums
 bool kr_sv_lin_blocks_fit(int dim, int vdim);
 void kr_sv_lin_chan_blocks(const KrSvLin& a, hipStream_t st);
 // prompt portions of kind 8 in blocks of 64 tokens: sbuf, tok and aux are scratch, the value rows are overwritten; z / ld name the same rows as qsrc
