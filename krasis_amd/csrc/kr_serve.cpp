@@ -41,7 +41,7 @@ struct SvLayer {
     // the previous token's input row of every slot.  Gated delta: the ring of projected rows, taps of them per slot
     DevBuf wk, mu, bonus, shift_state, delta_ring;
     // biases of hw's rows (the feed-forward's; zero elsewhere) and of the down projection; the per-layer token input; lightning attention: decays, norm weight, per-slot state
-    DevBuf h_bias, down_b, side_gate, side_proj, side_norm, lt_decay, lt_norm, lt_state;
+    DevBuf h_bias, down_b, side_gate, side_gate_p /* packed by fragments, see kr_sv_narrow_act */, side_proj, side_norm, lt_decay, lt_norm, lt_state;
     size_t lt_state_stride = 0;
     char have_mu[5] = {0, 0, 0, 0, 0};
     int wsrc = 0;                // the layer whose tensors this one uses (itself, or d.weights_of - 1); cache pools and state are always the layer's own
@@ -562,7 +562,16 @@ int kr_serve_set_tensor(kr_serve* s, int layer, int role, int index, const void*
     case KR_SV_LT_NORM: SHAPE(1, lti); rc = upload(s, l.lt_norm, n, 0, host, src_dtype, n, true); break;
     case KR_SV_LT_DECAY: SHAPE(1, d.lt_heads); rc = upload(s, l.lt_decay, n, 0, host, src_dtype, n, true); break;
     case KR_SV_LT_O: SHAPE(W, lti); rc = upload_cols(s, l.o, W, l.o_cols(), l.att_out_cols(), host, src_dtype, lti); break;
-    case KR_SV_SIDE_GATE: SHAPE(s->c.token_side, W); rc = upload(s, l.side_gate, n, 0, host, src_dtype, n, false); break;
+    case KR_SV_SIDE_GATE: {
+        SHAPE(s->c.token_side, W); rc = upload(s, l.side_gate, n, 0, host, src_dtype, n, false);
+        if (rc || s->f32 || W % 128) break;
+        const int ntt = (rows + 15) / 16;
+        std::vector<uint16_t> pk((size_t)ntt * 16 * W, 0);
+        for (int r = 0; r < rows; r++)
+            for (int k = 0; k < W; k++)
+                pk[((size_t)(k / 32) * ntt + r / 16) * 512 + (16 * (k % 32 / 8) + r % 16) * 8 + k % 8] = src_dtype == KR_SERVE_F32 ? f32_to_bf16_host(((const float*)host)[(size_t)r * W + k]) : ((const uint16_t*)host)[(size_t)r * W + k];
+        rc = upload(s, l.side_gate_p, pk.size(), 0, pk.data(), KR_SERVE_BF16, pk.size(), false); break;
+    }
     case KR_SV_SIDE_PROJ: SHAPE(W, s->c.token_side); rc = upload(s, l.side_proj, n, 0, host, src_dtype, n, false); break;
     case KR_SV_SIDE_NORM: SHAPE(1, W); rc = upload(s, l.side_norm, n, 0, host, src_dtype, n, true); break;
     case KR_SV_GATE_B: case KR_SV_UP_B:
@@ -785,6 +794,7 @@ int kr_serve_fill_synthetic(kr_serve* s, uint64_t seed, float amp) {
             if (!bad) bad |= hipMemcpy(l.lt_decay.p, dc.data(), dc.size() * 4, hipMemcpyHostToDevice) != hipSuccess;
         }
         if (d.ff_bias) bad |= vec(l.h_bias, l.n_h, false) | vec(l.down_b, W, false);
+        if (s->c.token_side > 0 && !s->f32 && W % 128 == 0) bad |= mat(l.side_gate_p, (size_t)(s->c.token_side + 15) / 16 * 16 * W, W);
         if (s->c.token_side > 0) bad |= mat(l.side_gate, (size_t)s->c.token_side * W, W) | mat(l.side_proj, (size_t)W * s->c.token_side, s->c.token_side) | vec(l.side_norm, W, true);
         std::fill(l.have_mu, l.have_mu + 5, (char)1);
         if (l.has_ssd()) {
@@ -1414,11 +1424,17 @@ int kr_serve_step(kr_serve* s, int n_entries, const int* slots, const int* count
         if (side) {
             // the token's own row for this layer: gate from the stream as it stands, times the row, projected, normed, added; the next layer's input from the same launch
             const int ns = c.token_side;
-            g = KrSvGemm{}; g.A = s->h.p; g.lda = W; g.W = l.side_gate.p; g.C = (float*)s->sgate.p; g.ldc = ns; g.M = T; g.N = ns; g.K = W;
-            { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
-            g = KrSvGemm{}; g.W = l.side_proj.p; g.C = (float*)s->mix.p; g.ldc = W; g.M = T; g.N = W; g.K = ns;
-            g.up_tab = s->side_embed.p; g.up_rows = d_tok; g.up_ld = c.n_layers * ns; g.up_off = li * ns;
-            down_proj(g, (const float*)s->sgate.p, ns, T, ns, KR_SV_ACT_GELU_TANH, 0.0f, 1.0f);
+            KrSvGemm gp{}; gp.W = l.side_proj.p; gp.C = (float*)s->mix.p; gp.ldc = W; gp.M = T; gp.N = W; gp.K = ns;
+            g = KrSvGemm{}; g.A = s->h.p; g.lda = W; g.W = l.side_gate.p; g.M = T; g.N = ns; g.K = W;
+            g.up_tab = gp.up_tab = s->side_embed.p; g.up_rows = gp.up_rows = d_tok; g.up_ld = gp.up_ld = c.n_layers * ns; g.up_off = gp.up_off = li * ns;
+            if (l.side_gate_p.p && kr_sv_narrow_act_fits(g, s->f32)) {
+                g.W = l.side_gate_p.p; g.C = (float*)s->y.p; g.ldc = ns; gp.A = s->y.p; gp.lda = ns;
+                Timer tm(s, 1); kr_sv_narrow_act(g, st); kr_sv_gemm(gp, s->f32, st);
+            } else {
+                g.C = (float*)s->sgate.p; g.ldc = ns; g.up_tab = nullptr;
+                { Timer tm(s, 1); kr_sv_gemm(g, s->f32, st); }
+                down_proj(gp, (const float*)s->sgate.p, ns, T, ns, KR_SV_ACT_GELU_TANH, 0.0f, 1.0f);
+            }
             res_layer = nullptr; res_run = nullptr; res_gate_kind = 0; res_to_mixer = true;
             residual((const float*)s->mix.p, nullptr, nullptr, nullptr, nullptr, 0, &l.side_norm, nullptr, hand, (nx && c.pre_norm) ? &nx->norm_w : nullptr, nx ? &nx->norm_b : nullptr);
         }

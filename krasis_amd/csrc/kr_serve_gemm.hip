@@ -311,7 +311,78 @@ __global__ void __launch_bounds__(256) sv_gemm_bf16_kernel(const KrSvGemm g) {
             }
         }
 }
+
+// ---------------------------------------------------------------------------------------------------------------- bf16, few columns, activation inside
+// Y = gelu_tanh(A W^T) * table rows, N <= 32 NT columns: a problem as narrow as this one leaves an LDS-tiled launch with a handful of workgroups that each walk the whole K
+// range.  Here a workgroup owns 32 rows and all columns; its eight waves take quarters of K times halves of N straight from global memory and the quarters meet in LDS,
+// where the activation is formed.  W comes packed by fragments -- [K / 32][N / 16][lane = 16 (k % 32 / 8) + n % 16][8] -- so that a fragment is one contiguous 1 KB read.
+typedef float gv4f __attribute__((ext_vector_type(4)));
+template <int NT>            // 16-column tiles per wave
+__global__ void __launch_bounds__(512) sv_narrow_act_kernel(const KrSvGemm g) {
+    constexpr int LD = NT * 32 + 4;
+    extern __shared__ __attribute__((aligned(16))) float part[];      // [4][32][LD]
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, q = lane >> 4, kg = wave & 3, ng = wave >> 2, m0 = blockIdx.x * 32;
+    const uint16_t* ap[2]; const uint16_t* bp[NT];
+    const int kq = g.K / 4, k0 = kg * kq + q * 8, ntt = (g.N + 15) / 16;
+#pragma unroll
+    for (int a = 0; a < 2; a++) ap[a] = (const uint16_t*)g.A + (size_t)min(m0 + a * 16 + r, g.M - 1) * g.lda + k0;
+#pragma unroll
+    for (int c = 0; c < NT; c++) bp[c] = (const uint16_t*)g.W + ((size_t)(kg * kq / 32) * ntt + min(ng * NT + c, ntt - 1)) * 512 + lane * 8;
+    gv4f acc[2][NT];
+#pragma unroll
+    for (int a = 0; a < 2; a++)
+#pragma unroll
+        for (int c = 0; c < NT; c++) acc[a][c] = gv4f{0.0f, 0.0f, 0.0f, 0.0f};
+    gu4 af[3][2], bf[3][NT];                         // fragments of three steps of 32: a step's are requested two steps before its products
+    auto fetch = [&](int set, int k) {
+        k = min(k, kq - 32);
+#pragma unroll
+        for (int a = 0; a < 2; a++) af[set][a] = *reinterpret_cast<const gu4*>(ap[a] + k);
+#pragma unroll
+        for (int c = 0; c < NT; c++) bf[set][c] = *reinterpret_cast<const gu4*>(bp[c] + (size_t)k * ntt * 16);
+    };
+    auto step = [&](int set) {
+#pragma unroll
+        for (int a = 0; a < 2; a++)
+#pragma unroll
+            for (int c = 0; c < NT; c++) acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(gb8, af[set][a]), __builtin_bit_cast(gb8, bf[set][c]), acc[a][c], 0, 0, 0);
+    };
+    fetch(0, 0); fetch(1, 32);
+    for (int k = 0; k < kq; k += 96) {
+        fetch(2, k + 64); __builtin_amdgcn_sched_barrier(0); step(0);
+        fetch(0, k + 96); __builtin_amdgcn_sched_barrier(0); if (k + 32 < kq) step(1);
+        fetch(1, k + 128); __builtin_amdgcn_sched_barrier(0); if (k + 64 < kq) step(2);
+    }
+#pragma unroll
+    for (int a = 0; a < 2; a++)
+#pragma unroll
+        for (int c = 0; c < NT; c++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) part[(kg * 32 + a * 16 + 4 * q + i) * LD + (ng * NT + c) * 16 + r] = acc[a][c][i];
+    __syncthreads();
+#pragma unroll 4
+    for (int i = tid; i < 32 * NT * 32; i += 512) {
+        const int row = i / (NT * 32), n = i - row * (NT * 32), m = m0 + row;
+        if (m >= g.M || n >= g.N) continue;
+        const float e = kr_bf16_to_f32(((const uint16_t*)g.up_tab)[(size_t)g.up_rows[m] * g.up_ld + g.up_off + n]);
+        const float v = (part[row * LD + n] + part[(32 + row) * LD + n]) + (part[(64 + row) * LD + n] + part[(96 + row) * LD + n]);
+        // gelu with the tanh form: v (1 + tanh w) / 2 = v sigmoid(2 w)
+        const float w2 = 1.5957691216057308f * __builtin_fmaf(0.044715f * v * v, v, v);
+        ((uint16_t*)g.C)[(size_t)m * g.ldc + n] = kr_f32_to_bf16(v * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * w2)) * e);
+    }
+}
 }  // namespace
+
+bool kr_sv_narrow_act_fits(const KrSvGemm& g, bool f32) {
+    return !f32 && g.M > 64 && g.N <= 256 && g.K % 128 == 0 && g.lda % 8 == 0 && (((uintptr_t)g.A | (uintptr_t)g.W) % 16 == 0) && g.up_tab && !g.a_rows && !g.seg;
+}
+void kr_sv_narrow_act(const KrSvGemm& g, hipStream_t st) {
+    const dim3 grid((g.M + 31) / 32);
+    if (g.N <= 128) { const size_t b = (size_t)4 * 32 * (4 * 32 + 4) * 4; (void)hipFuncSetAttribute((const void*)sv_narrow_act_kernel<4>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)b);
+        hipLaunchKernelGGL(sv_narrow_act_kernel<4>, grid, dim3(512), b, st, g); }
+    else { const size_t b = (size_t)4 * 32 * (8 * 32 + 4) * 4; (void)hipFuncSetAttribute((const void*)sv_narrow_act_kernel<8>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)b);
+        hipLaunchKernelGGL(sv_narrow_act_kernel<8>, grid, dim3(512), b, st, g); }
+}
 
 bool kr_sv_gemm_small(const KrSvGemm& g) {
     // decode-sized problems: a pass over the weights per 8 rows; grouped problems take one row per workgroup row (each row has its own expert)
@@ -349,7 +420,8 @@ void kr_sv_gemm(const KrSvGemm& g, bool f32, hipStream_t st) {
     }
     // grouped problems have few rows per expert: the 64-row tile wastes less of the matrix cores.  (A 256-row tile -- wave tiles of 128 x 64, six fragment
     // reads per eight MFMAs -- was measured and did not pay: two workgroups per compute unit instead of three.)
-    const bool small = grouped ? (g.M / (g.n_groups > 0 ? g.n_groups : 1) < 96) : g.M <= 64;
+    // and so do narrow problems: with 128-row tiles they would leave most compute units idle
+    const bool small = grouped ? (g.M / (g.n_groups > 0 ? g.n_groups : 1) < 96) : g.M <= 64 || (long)((g.N + 127) / 128) * ((g.M + 127) / 128) < 128;
     if (small) {
         const int tiles = grouped ? (g.M + 63) / 64 + g.n_groups : (g.M + 63) / 64;
         hipLaunchKernelGGL(sv_gemm_bf16_kernel<64>, dim3((g.N + 127) / 128, tiles), dim3(256), 0, st, g);

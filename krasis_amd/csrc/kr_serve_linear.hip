@@ -210,20 +210,27 @@ __global__ void __launch_bounds__(256) ln_delta_save_kernel(const KrSvDelta a) {
 }
 
 // ---- lightning attention: the heads side by side as one row
-template <typename T>
-__global__ void __launch_bounds__(256) ln_row_out_kernel(const float* __restrict__ o, int n, const float* __restrict__ w, const float* __restrict__ gate, int gate_ld, float eps, float scale,
-                                                         T* __restrict__ out, int out_ld) {
-    __shared__ float red[4];
+// NT threads: 256 for prompt-sized steps, 1024 where a row's workgroup is alone on its compute unit
+template <typename T, int NT>
+__global__ void __launch_bounds__(NT) ln_row_out_kernel(const float* __restrict__ o, int n, const float* __restrict__ w, const float* __restrict__ gate, int gate_ld, float eps, float scale,
+                                                        T* __restrict__ out, int out_ld) {
+    __shared__ float red[NT / 64];
     const size_t t = blockIdx.x;
     const float* r = o + t * n;
     float ss = 0.0f;
-    for (int c = threadIdx.x; c < n; c += 256) ss = __builtin_fmaf(r[c], r[c], ss);
+#pragma unroll 4
+    for (int c = threadIdx.x; c < n; c += NT) ss = __builtin_fmaf(r[c], r[c], ss);
     ss = ln_wave_sum(ss);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
     __syncthreads();
-    const float inv = scale / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)n + eps);
-    for (int c = threadIdx.x; c < n; c += 256) ln_st(out + t * out_ld + c, r[c] * inv * w[c] / (1.0f + expf(-gate[t * gate_ld + c])));
+    float all = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NT / 64; i++) all += red[i];
+    const float inv = scale / sqrtf(all / (float)n + eps);
+#pragma unroll 4
+    for (int c = threadIdx.x; c < n; c += NT) ln_st(out + t * out_ld + c, r[c] * inv * w[c] / (1.0f + expf(-gate[t * gate_ld + c])));
 }
+
 // ---- block form of the recurrences with a decay per key channel (gla, wkv), prompt portions: blocks of 64 tokens, four sub-blocks of 16.
 // With f_s the sum of the log decays from the start of s's sub-block to s, and tot_m that of a whole sub-block, every weight between two tokens splits into
 // exp(e_t) * prod(sub-blocks between) * exp(tot - f_s) (e_t = f_t, or the sum before t where the read-out comes before the write): all three factors are <= 1, so
@@ -731,6 +738,8 @@ void kr_sv_delta_prep(const KrSvDelta& a, hipStream_t st) {
 }
 void kr_sv_row_out(const float* o, int n, const float* w, const float* gate, int gate_ld, float eps, float scale, void* out, int out_ld, bool f32, int T, hipStream_t st) {
     if (T <= 0) return;
-    if (f32) hipLaunchKernelGGL(ln_row_out_kernel<float>, dim3(T), dim3(256), 0, st, o, n, w, gate, gate_ld, eps, scale, (float*)out, out_ld);
-    else hipLaunchKernelGGL(ln_row_out_kernel<uint16_t>, dim3(T), dim3(256), 0, st, o, n, w, gate, gate_ld, eps, scale, (uint16_t*)out, out_ld);
+#define LN_RO(T_, NT_) hipLaunchKernelGGL((ln_row_out_kernel<T_, NT_>), dim3(T), dim3(NT_), 0, st, o, n, w, gate, gate_ld, eps, scale, (T_*)out, out_ld)
+    if (f32) { if (T <= 64) LN_RO(float, 1024); else LN_RO(float, 256); }
+    else { if (T <= 64) LN_RO(uint16_t, 1024); else LN_RO(uint16_t, 256); }
+#undef LN_RO
 }

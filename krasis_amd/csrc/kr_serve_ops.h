@@ -35,6 +35,10 @@ struct KrSvGemm {
     const void* up_tab; const int* up_rows; int up_ld, up_off;
 };
 void kr_sv_gemm(const KrSvGemm& g, bool f32, hipStream_t st);
+// prompt-sized, at most 256 columns, bf16: C (storage type) = gelu_tanh(A W^T) * rows of up_tab, in one launch; W packed by fragments: element (n, k) of [N, K] at
+// ((k / 32) * ceil(N / 16) + n / 16) * 512 + (16 * (k % 32 / 8) + n % 16) * 8 + k % 8
+bool kr_sv_narrow_act_fits(const KrSvGemm& g, bool f32);
+void kr_sv_narrow_act(const KrSvGemm& g, hipStream_t st);
 bool kr_sv_gemm_small(const KrSvGemm& g);      // true: kr_sv_gemm takes the wave-per-column form for this problem (and honours act_gu)
 
 enum { KR_SV_NORM_LAYER = 0, KR_SV_NORM_RMS = 1 };

@@ -87,6 +87,25 @@ def test_bf16_store_close_to_oracle(make, n):
     assert np.median(e) < 3e-2 and e.max() < 8e-2
 
 
+@pytest.mark.parametrize("width,side,n", [(384, 200, 130), (256, 17, 65), (128, 256, 97), (640, 128, 66), (192, 40, 90)])
+def test_token_rows_of_prompts_in_bf16(width, side, n):
+    """prompt-sized steps form gate and activation of the token rows in one launch when the rows are whole fragments (widths that are multiples of 128), else in two"""
+    cfg = O.make_config(width=width, vocab=61, side=side, layers=[O.layer(O.wkv(2, 8, 3), None), O.layer(O.delta(2, 1, 8, 8, 2), O.dense(24))])
+    W = {k: O.bf16_round(v) for k, v in O.random_weights(cfg, 43).items()}
+    W["side.embed"] = O.bf16_round(W["side.embed"] * 3.0); W["l0.side.norm"][:] = 2.0; W["l1.side.norm"][:] = 2.0
+    toks = tokens(cfg, n, 44)
+    ref, streams = O.forward(cfg, W, toks)
+    swapped, _ = O.forward(cfg, {**W, "l1.side.gate": W["l1.side.gate"][::-1]}, toks)
+    assert rel(swapped, ref) > 0.3
+    eng = engine(cfg, W, "bfloat16")
+    eng.store.set_capture(True)
+    logits, _ = eng.step([("a", toks, list(range(n)))])
+    got = eng.store.read_capture(n)
+    for li in range(2):
+        assert rel(got[li], streams[li]) < 3e-2, li
+    assert rel(logits, ref) < 6e-2
+
+
 def small_model(layers, **kw):
     kw.setdefault("width", 64); kw.setdefault("vocab", 50)
     return O.make_config(layers=layers, **kw)

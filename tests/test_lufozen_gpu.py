@@ -568,9 +568,9 @@ def test_state_space_mixer_as_a_layers_only_mixer():
 
 
 def test_many_workgroups_take_the_plain_walk_of_the_scan():
-    """four prompts in one step, seven heads of 112 value columns: more workgroups than the pipelined form of the prompt scan is launched for, in the gla
-    mixer and in a state-space mixer whose 130 states are beyond the block form"""
-    cfg = small_model([O.layer(O.gla(7, 8, 112, tau=5.0), None),
+    """four prompts in one step, seven heads of 112 value columns: more workgroups than the pipelined form of the prompt scan is launched for, in a gla
+    mixer whose 132 keys and a state-space mixer whose 130 states are beyond the block forms"""
+    cfg = small_model([O.layer(O.gla(7, 132, 112, tau=5.0), None),
                        O.layer(O.parallel(O.left(2, 1, 8, 8), O.ssd(7, 112, 130, groups=7, conv=2, norm_groups=1), 0.5, 0.8), O.dense(24))])
     W = O.random_weights(cfg, 51)
     seqs = {k: tokens(cfg, n, 52 + i) for i, (k, n) in enumerate((("a", 40), ("b", 33), ("c", 57), ("d", 36)))}
